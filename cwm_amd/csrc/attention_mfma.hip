@@ -76,13 +76,31 @@ __device__ __forceinline__ float tanh_of(float x) {
   return 1.0f - 2.0f * __builtin_amdgcn_rcpf(e + 1.0f);
 }
 
+// A library built with -DDISTANCE_BIAS=1 takes slope_h * ln(1 + rate_h * (query - key)) off every scaled score.  In the
+// raw scores' units, with log2 from one v_log_f32: slope / (scale log2 e) * log2(.), whose argument is one addition a
+// key, since a lane's eight keys follow one another (SLOPE_RAW and RATE are the row's, DIST its distance to the lane's
+// first key; keys that the row does not read may give anything, the masks come after).
+#ifdef DISTANCE_BIAS
+#define BIAS_PARAMS , const float* __restrict__ bias_slope, const float* __restrict__ bias_rate
+#define BIAS_TILE(SLOPE_RAW, RATE, DIST)                                                                     \
+    {                                                                                                        \
+      const float far_arg = fmaf(RATE, (float)(DIST), 1.0f);                                                 \
+      _Pragma("unroll") for (int e = 0; e < 8; ++e)                                                          \
+        rv[e] = fmaf(-(SLOPE_RAW), __builtin_amdgcn_logf(fmaf(RATE, -(float)e, far_arg)), rv[e]);            \
+    }
+#else
+#define BIAS_PARAMS
+#define BIAS_TILE(SLOPE_RAW, RATE, DIST)
+#endif
+
 #define MAXIMUM(a, b) __builtin_elementwise_maximum(a, b)
-#define SOFTMAX_TILE(VOTE, ST0, ST1, NEED_MASK, OK_EXPR, M_RUN, NEG_MC, L_RUN, ALPHA, PF)                    \
+#define SOFTMAX_TILE(VOTE, ST0, ST1, NEED_MASK, OK_EXPR, M_RUN, NEG_MC, L_RUN, ALPHA, PF, SLOPE_RAW, RATE, DIST) \
   {                                                                                                          \
     float rv[8] = {ST0[0], ST0[1], ST0[2], ST0[3], ST1[0], ST1[1], ST1[2], ST1[3]};                          \
     if (cap_raw > 0.f) {                                                                                     \
       _Pragma("unroll") for (int e = 0; e < 8; ++e) rv[e] = cap_raw * tanh_of(rv[e] * inv_cap_raw);          \
     }                                                                                                        \
+    BIAS_TILE(SLOPE_RAW, RATE, DIST)                                                                         \
     if (NEED_MASK) {                                                                                         \
       _Pragma("unroll") for (int e = 0; e < 8; ++e) {                                                        \
         const int key = kt + 8 * j + e;                                                                      \
@@ -161,7 +179,7 @@ attention_mfma_kernel(const bf16_t* __restrict__ q, long q_stride, bf16_t* __res
                       const int* __restrict__ cu_q, const int* __restrict__ kv_len, const int* __restrict__ work,
                       int n_work, float* __restrict__ partial, int n_q_heads, int n_kv_heads, int page_size,
                       int page_shift, int num_pages, int window_left, int chunk, float scale_log2e, float cap_raw,
-                      const float* __restrict__ sink) {
+                      const float* __restrict__ sink BIAS_PARAMS) {
   const int lane = threadIdx.x & 63;
   const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
   const int id = blockIdx.x;  // (item, key/value head): the same for the whole block
@@ -191,6 +209,9 @@ attention_mfma_kernel(const bf16_t* __restrict__ q, long q_stride, bf16_t* __res
   const int ti = row_valid ? r / group : 0;
   const int hq = g * group + (row_valid ? r - ti * group : 0);
   const int row_end = n_old + ti;  // last key the row may read
+#ifdef DISTANCE_BIAS
+  const float slope_raw = bias_slope[hq] / scale_log2e, rate = bias_rate[hq];
+#endif
   const int row_start = chunk > 0 ? row_end - row_end % chunk : (window_left >= 0 ? max(0, row_end - window_left) : 0);
   // the span of keys that any row of the item reads (uniform): outside it values may be anything
   // (pages given back, slots never written) and are zeroed before use
@@ -325,7 +346,7 @@ attention_mfma_kernel(const bf16_t* __restrict__ q, long q_stride, bf16_t* __res
     float alpha;
     Frag8 pf;
     SOFTMAX_TILE(false, st[0], st[1], need_mask, row_valid && key >= row_start && key <= row_end && key >= key_begin && key < key_end,
-                 m_run, neg_mc_run, l_run, alpha, pf)
+                 m_run, neg_mc_run, l_run, alpha, pf, slope_raw, rate, row_end - (kt + 8 * j))
     if (__any(alpha != 1.0f)) {  // seldom after the first tiles
       asm volatile("" ::: "memory");  // keeps this a branch: unconditional, it is 4 multiplications per output tile
 #pragma unroll
@@ -467,7 +488,7 @@ attention_lds_kernel(const bf16_t* __restrict__ q, long q_stride, bf16_t* __rest
                      const int* __restrict__ cu_q, const int* __restrict__ kv_len, const int* __restrict__ work,
                      float* __restrict__ partial, int n_kv_heads_grid, int n_q_heads, int n_kv_heads, int page_size,
                      int page_shift, int num_pages, int window_left, int chunk, float scale_log2e, float cap_raw,
-                      const float* __restrict__ sink) {
+                      const float* __restrict__ sink BIAS_PARAMS) {
   constexpr bool FAST = MODE != LDS_PLAIN;
   constexpr int DMA_AHEAD = DMA_BUFFERS - 1;
   __shared__ __attribute__((aligned(16))) bf16_t lds_k[MODE == LDS_DMA ? 1 : 2][MODE == LDS_DMA ? 8 : 32 * LDS_K_STRIDE];
@@ -501,6 +522,9 @@ attention_lds_kernel(const bf16_t* __restrict__ q, long q_stride, bf16_t* __rest
   Frag8 qf[LDS_RT][K32_STEPS];
   float4v acc[LDS_RT][D_TILES];
   float m_run[LDS_RT], neg_mc_run[LDS_RT], l_run[LDS_RT];
+#ifdef DISTANCE_BIAS
+  float slope_raw[LDS_RT], rate[LDS_RT];
+#endif
   const float neg_inf = -__builtin_inff();
   const float lazy_raw = 8.0f / scale_log2e;  // 8 binary orders, in units of the raw scores
   const float inv_cap_raw = cap_raw > 0.f ? 1.0f / cap_raw : 0.f;
@@ -511,6 +535,10 @@ attention_lds_kernel(const bf16_t* __restrict__ q, long q_stride, bf16_t* __rest
     ti[rt] = row_valid[rt] ? r / group : 0;
     hq[rt] = g * group + (row_valid[rt] ? r - ti[rt] * group : 0);
     row_end[rt] = n_old + ti[rt];
+#ifdef DISTANCE_BIAS
+    slope_raw[rt] = bias_slope[hq[rt]] / scale_log2e;
+    rate[rt] = bias_rate[hq[rt]];
+#endif
     row_start[rt] = chunk > 0 ? row_end[rt] - row_end[rt] % chunk : (window_left >= 0 ? max(0, row_end[rt] - window_left) : 0);
     const bf16_t* qrow = q + (size_t)(q0 + ti[rt]) * q_stride + (size_t)hq[rt] * HEAD_DIM;
 #pragma unroll
@@ -707,7 +735,7 @@ attention_lds_kernel(const bf16_t* __restrict__ q, long q_stride, bf16_t* __rest
 #pragma unroll
     for (int rt = 0; rt < LDS_RT; ++rt) {
       SOFTMAX_TILE(true, st[rt][0], st[rt][1], need_mask, row_valid[rt] && key >= row_start[rt] && key <= row_end[rt], m_run[rt],
-                   neg_mc_run[rt], l_run[rt], alpha[rt], pf[rt])
+                   neg_mc_run[rt], l_run[rt], alpha[rt], pf[rt], slope_raw[rt], rate[rt], row_end[rt] - (kt + 8 * j))
       moved = moved || alpha[rt] != 1.0f;
     }
     if (__any(moved)) {  // seldom after the first tiles
@@ -1001,7 +1029,14 @@ extern "C" int cwm_attention_mfma(const void* q, long q_stride, void* out, long 
                                   int wide_three_blocks, const int* merge,
                                   int n_merge, int n_merge_mid, int n_merge_few, float* partial, int n_q_heads, int n_kv_heads, int head_dim,
                                   int page_size, int num_pages, int window_left, int chunk, float scale, float softcap,
-                                  const float* sink, hipStream_t stream) {
+                                  const float* sink, const float* bias_slope, const float* bias_rate, hipStream_t stream) {
+#ifdef DISTANCE_BIAS
+  CWM_REQUIRE(bias_slope && bias_rate, "attention_mfma: this library takes a distance bias off the scores, with a slope and a rate a head");
+#define BIAS_ARGS , bias_slope, bias_rate
+#else
+  CWM_REQUIRE(!bias_slope && !bias_rate, "attention_mfma: this library is built without a distance bias");
+#define BIAS_ARGS
+#endif
   // `chunk` > 0: instead of a window, a query reads the keys of its own block of that many positions (counted from 0)
   // up to itself; `softcap` > 0: scaled scores are capped, s <- softcap * tanh(s / softcap), before the softmax
   CWM_REQUIRE(chunk >= 0 && softcap >= 0.f && scale > 0.f, "attention_mfma: a block of keys and a cap cannot be negative, the scale is positive");
@@ -1034,7 +1069,7 @@ extern "C" int cwm_attention_mfma(const void* q, long q_stride, void* out, long 
   hipLaunchKernelGGL((attention_mfma_kernel<PAGE32>), dim3((unsigned)blocks), dim3(256), 0, stream, (const bf16_t*)q,     \
                      q_stride, (bf16_t*)out, out_stride, (const bf16_t*)cache, block_table, table_width, cu_q, kv_len,   \
                      work, n_work, partial, n_q_heads, n_kv_heads, page_size, page_shift, num_pages, window_left,        \
-                     chunk, scale_log2e, cap_raw, sink)
+                     chunk, scale_log2e, cap_raw, sink BIAS_ARGS)
     if (page_size % 32 == 0)
       CWM_LAUNCH_TEAM(true);
     else
@@ -1050,7 +1085,7 @@ extern "C" int cwm_attention_mfma(const void* q, long q_stride, void* out, long 
   hipLaunchKernelGGL((attention_lds_kernel<MODE, BUFFERS, MIN_BLOCKS>), dim3((unsigned)blocks), dim3(256), 0, stream,     \
                      (const bf16_t*)q, q_stride,                                                                          \
                      (bf16_t*)out, out_stride, (const bf16_t*)cache, block_table, table_width, cu_q, kv_len, work_wide,   \
-                     partial, n_kv_heads, n_q_heads, n_kv_heads, page_size, page_shift, num_pages, window_left, chunk, scale_log2e, cap_raw, sink)
+                     partial, n_kv_heads, n_q_heads, n_kv_heads, page_size, page_shift, num_pages, window_left, chunk, scale_log2e, cap_raw, sink BIAS_ARGS)
     // tiles of 32 keys that never straddle a page, and shares of a tile that divide evenly over the block
     if (page_size % 32 == 0 && LDS_K_CHUNKS % 256 == 0 && LDS_V_CHUNKS % 256 == 0) {
 #if DMA_HEAD_DIM_OK

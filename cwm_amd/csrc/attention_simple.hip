@@ -9,7 +9,8 @@
 // from 0); s_j = (q . k_j) * scale; o = sum_j softmax(s)_j v_j; query head h uses
 // key/value head h / (n_q_heads / n_kv_heads).  Two options beside it: `chunk` > 0 replaces the window by blocks
 // of that many positions counted from 0 (the query at p reads the keys of its own block up to p), and `softcap` > 0
-// caps the scaled score, s_j <- softcap * tanh(s_j / softcap), before the softmax.
+// caps the scaled score, s_j <- softcap * tanh(s_j / softcap), before the softmax.  A distance bias (`bias_slope`,
+// `bias_rate`: float32, one number a query head) then comes off it, s_j <- s_j - slope_h * ln(1 + rate_h * (p - j)).
 //
 // One block of four wavefronts per (token, key/value head, up to 8 of its query heads,
 // segment of the keys): a key and a value are loaded once and used for all the block's
@@ -75,7 +76,8 @@ attention_simple_kernel(const T* __restrict__ q, long q_stride, T* __restrict__ 
                         const T* __restrict__ cache, const int* __restrict__ block_table, int table_width,
                         const int* __restrict__ positions, const int* __restrict__ seq_of_token, float* __restrict__ partial,
                         int n_q_heads, int n_kv_heads, int head_groups, int head_dim, int page_size, int num_pages,
-                        int window_left, int chunk, float scale, float softcap, const float* __restrict__ sink) {
+                        int window_left, int chunk, float scale, float softcap, const float* __restrict__ sink,
+                        const float* __restrict__ bias_slope, const float* __restrict__ bias_rate) {
   __shared__ __attribute__((aligned(16))) float qs[HEADS][D_REGS * CWM_WAVE];
   // probabilities of a chunk, key jj at [in0 + jj] (in0: the first key's place in its block of 8 values), so that the
   // eight of a block lie at a multiple of 8
@@ -205,6 +207,7 @@ attention_simple_kernel(const T* __restrict__ q, long q_stride, T* __restrict__ 
         for (int h = 0; h < HEADS; ++h) {
           s[h] = dot[h] * scale;
           if (softcap > 0.f) s[h] = softcap * tanhf(s[h] / softcap);
+          if (bias_slope && h < nh) s[h] -= bias_slope[h0 + h] * log1pf(bias_rate[h0 + h] * (float)(p - j));
         }
         // values: blocks of v_block keys, [slot / v_block][dim][slot % v_block]
         vo = (long long)((size_t)page * 2 * plane + plane + (size_t)g * head_dim * page_size +
@@ -404,7 +407,9 @@ extern "C" int cwm_attention_simple(const void* q, long q_stride, void* out, lon
                                     int dtype, const int* block_table, int table_width, const int* positions,
                                     const int* seq_of_token, int n_tokens, int n_q_heads, int n_kv_heads,
                                     int head_dim, int page_size, int num_pages, int window_left, int chunk, float scale,
-                                    float softcap, int max_keys, float* partial, const float* sink, hipStream_t stream) {
+                                    float softcap, int max_keys, float* partial, const float* sink, const float* bias_slope,
+                                    const float* bias_rate, hipStream_t stream) {
+  CWM_REQUIRE((bias_slope == nullptr) == (bias_rate == nullptr), "attention: a distance bias has a slope and a rate a head");
   CWM_REQUIRE(chunk >= 0 && softcap >= 0.f, "attention: a block of keys and a cap on the scores cannot be negative");
   CWM_REQUIRE(n_tokens >= 0, "attention: negative token count");
   CWM_REQUIRE(head_dim > 0 && head_dim <= SIMPLE_MAX_HEAD_DIM, "attention: head_dim %d is outside 1..%d", head_dim,
@@ -433,7 +438,7 @@ extern "C" int cwm_attention_simple(const void* q, long q_stride, void* out, lon
   hipLaunchKernelGGL((attention_simple_kernel<float, HEADS, D_REGS>), grid, dim3(SIMPLE_WAVES * CWM_WAVE), 0, stream,     \
                      (const float*)q, q_stride, (float*)out, out_stride, (const float*)cache, block_table, table_width,   \
                      positions, seq_of_token, partial, n_q_heads, n_kv_heads, head_groups, head_dim, page_size, num_pages, \
-                     window_left, chunk, scale, softcap, sink)
+                     window_left, chunk, scale, softcap, sink, bias_slope, bias_rate)
 #define CWM_LAUNCH_SIMPLE_HEADS(D_REGS)   \
   do {                                    \
     if (heads <= 2)                       \
@@ -460,7 +465,7 @@ extern "C" int cwm_attention_simple(const void* q, long q_stride, void* out, lon
     hipLaunchKernelGGL((attention_simple_kernel<bf16_t, SIMPLE_HEADS, SIMPLE_D_REGS>), grid, dim3(SIMPLE_WAVES * CWM_WAVE), 0, stream, (const bf16_t*)q,
                        q_stride, (bf16_t*)out, out_stride, (const bf16_t*)cache, block_table, table_width, positions,
                        seq_of_token, partial, n_q_heads, n_kv_heads, head_groups, head_dim, page_size, num_pages, window_left,
-                       chunk, scale, softcap, sink);
+                       chunk, scale, softcap, sink, bias_slope, bias_rate);
     if (max_segments > 1)
       hipLaunchKernelGGL(attention_simple_join_kernel<bf16_t>, dim3((unsigned)join_blocks), dim3(CWM_WAVE), 0, stream,
                          (bf16_t*)out, out_stride, (const float*)partial, positions, n_q_heads, head_dim, window_left, chunk, max_segments, sink);

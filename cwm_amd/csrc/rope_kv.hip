@@ -518,7 +518,8 @@ extern "C" int cwm_qk_norm_rope_write(const void* src, int src_dtype, long src_s
 // position * inv_freq[pair] (adjacent pairs; a frequency of 0 leaves its pair alone).  Values: where `v_other` is
 // given, v <- (1 - mix) v + mix v_other, with `mix` one float32 on the device and v_other [T][Hkv * v_dim] the
 // values that another layer made of the same tokens; `v_keep`, where given, receives this layer's values as they go
-// into the cache, [T][Hkv * v_dim].  Heads are laid out with `head_dim` elements as in the kernel above.  All
+// into the cache, [T][Hkv * v_dim].  With `temp_every` > 0 the query at position p is also multiplied by the
+// temperature 1 + temp_coef ln(floor((p + 1) / temp_every) + 1).  Heads are laid out with `head_dim` elements as in the kernel above.  All
 // arithmetic float32.  A wavefront a head: the lanes hold the head's pairs, so a head's sum of squares is one
 // reduction over the lanes; the blocks of a token (gridDim.y of them) share its heads.
 template <typename TS, typename TO>
@@ -529,7 +530,8 @@ head_norm_rope_write_kernel(const TS* __restrict__ src, long src_stride, int n_p
                             const int* __restrict__ seq_of_token, const float* __restrict__ inv_freq, TO* __restrict__ cache,
                             const int* __restrict__ block_table, int table_width, int page_size, int num_pages, int n_q_heads,
                             int n_kv_heads, int qk_dim, int v_dim, int head_dim, const TO* __restrict__ v_other,
-                            long v_other_stride, const float* __restrict__ v_mix, TO* __restrict__ v_keep) {
+                            long v_other_stride, const float* __restrict__ v_mix, TO* __restrict__ v_keep, float temp_coef,
+                            int temp_every) {
   __shared__ __attribute__((aligned(16))) float cs[NORM_ROPE_MAX_HEAD];  // cos, sin of each pair
   const int t = blockIdx.x;
   const int pos = positions[t];
@@ -567,6 +569,7 @@ head_norm_rope_write_kernel(const TS* __restrict__ src, long src_stride, int n_p
   __syncthreads();
   const int n_heads = n_q_heads + (cache ? n_kv_heads : 0);
   const int waves = blockDim.x / CWM_WAVE;
+  const float q_gain = temp_every > 0 ? 1.f + temp_coef * logf((float)((pos + 1) / temp_every) + 1.f) : 1.f;
   for (int hh = blockIdx.y * waves + wave; hh < n_heads; hh += gridDim.y * waves) {
     const bool is_key = hh >= n_q_heads;
     const int head = is_key ? hh - n_q_heads : hh;
@@ -598,6 +601,7 @@ head_norm_rope_write_kernel(const TS* __restrict__ src, long src_stride, int n_p
           a *= rstd * (2 * i < qk_dim ? weight[2 * i] : 0.f);
           b *= rstd * (2 * i + 1 < qk_dim ? weight[2 * i + 1] : 0.f);
         }
+        if (!is_key) a *= q_gain, b *= q_gain;
         const float c = cs[2 * i], s = cs[2 * i + 1];
         Elem<TO>::store(dst + 2 * i, a * c - b * s);
         Elem<TO>::store(dst + 2 * i + 1, b * c + a * s);
@@ -626,12 +630,14 @@ head_norm_rope_write_kernel(const TS* __restrict__ src, long src_stride, int n_p
 // partial_stride apart.  bias: float32 [(Hq + Hkv) * qk_dim + Hkv * v_dim] or null.  q_weight, k_weight: float32
 // [qk_dim] or null.  inv_freq: float32 [head_dim / 2] or null.  v_other ([n_tokens][v_other_stride], the cache's type)
 // with v_mix (one float32 on the device): both or neither.  v_keep: [n_tokens][Hkv * v_dim] of the cache's type, or null.
+// temp_every > 0: queries are multiplied by their position's temperature (0: by nothing).
 extern "C" int cwm_head_norm_rope_write(const void* src, int src_dtype, long src_stride, int n_partials, long partial_stride,
                                         const float* bias, void* q_out, int out_dtype, const float* q_weight, const float* k_weight,
                                         float eps, const int* positions, const int* seq_of_token, const float* inv_freq, void* cache,
                                         const int* block_table, int table_width, int page_size, int num_pages, int n_tokens,
                                         int n_q_heads, int n_kv_heads, int qk_dim, int v_dim, int head_dim, const void* v_other,
-                                        long v_other_stride, const float* v_mix, void* v_keep, hipStream_t stream) {
+                                        long v_other_stride, const float* v_mix, void* v_keep, float temp_coef, int temp_every,
+                                        hipStream_t stream) {
   CWM_REQUIRE(n_tokens >= 0 && n_partials >= 1, "head_norm_rope_write: bad sizes");
   CWM_REQUIRE(n_partials == 1 || src_dtype == CWM_F32, "head_norm_rope_write: partial sums must be float32");
   CWM_REQUIRE(head_dim > 0 && head_dim % 2 == 0 && head_dim <= NORM_ROPE_MAX_HEAD,
@@ -641,6 +647,7 @@ extern "C" int cwm_head_norm_rope_write(const void* src, int src_dtype, long src
   CWM_REQUIRE(n_q_heads > 0 && n_kv_heads > 0, "head_norm_rope_write: no heads");
   CWM_REQUIRE(src && q_out && positions, "head_norm_rope_write: arguments missing");
   CWM_REQUIRE(eps > 0.f || (!q_weight && !k_weight), "head_norm_rope_write: eps must be positive");
+  CWM_REQUIRE(temp_every >= 0, "head_norm_rope_write: the temperature's step cannot be negative");
   CWM_REQUIRE((v_other == nullptr) == (v_mix == nullptr), "head_norm_rope_write: other values and their weight come together");
   if (cache) {
     CWM_REQUIRE(block_table && seq_of_token, "head_norm_rope_write: a cache write needs a block table");
@@ -655,7 +662,7 @@ extern "C" int cwm_head_norm_rope_write(const void* src, int src_dtype, long src
   hipLaunchKernelGGL((head_norm_rope_write_kernel<TS, TO>), dim3(n_tokens, gy), dim3(256), 0, stream, (const TS*)src,       \
                      src_stride, n_partials, partial_stride, bias, (TO*)q_out, q_weight, k_weight, eps, positions,         \
                      seq_of_token, inv_freq, (TO*)cache, block_table, table_width, page_size, num_pages, n_q_heads,        \
-                     n_kv_heads, qk_dim, v_dim, head_dim, (const TO*)v_other, v_other_stride, v_mix, (TO*)v_keep)
+                     n_kv_heads, qk_dim, v_dim, head_dim, (const TO*)v_other, v_other_stride, v_mix, (TO*)v_keep, temp_coef, temp_every)
   switch (key) {
     case 0: CWM_HEAD_NORM_ROPE(float, float); break;
     case 1: CWM_HEAD_NORM_ROPE(float, bf16_t); break;

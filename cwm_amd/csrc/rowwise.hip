@@ -40,6 +40,47 @@ extern "C" int cwm_embedding(void* out, const void* table, int table_dtype, cons
   return cwm_launch_status("embedding");
 }
 
+// out[t, :] = scale * table[token[t], :] + s(positions[t]), the sinusoidal position vector s(p)[2i] = sin(p f_i),
+// s(p)[2i + 1] = cos(p f_i).  `turns` holds f_i / (2 pi) in float64 (one value a pair): the angle in turns is reduced to
+// [-1/2, 1/2] in float64, so that a far position costs no digits of it.
+template <typename TW>
+__global__ void embedding_sinusoid_kernel(float* __restrict__ out, const TW* __restrict__ table, const int* __restrict__ tokens,
+                                          const int* __restrict__ positions, const double* __restrict__ turns, int dim, int vocab,
+                                          float scale) {
+  const int t = blockIdx.x;
+  const int tok = tokens[t];
+  const bool known = tok >= 0 && tok < vocab;
+  const double p = (double)positions[t];
+  float* dst = out + (size_t)t * dim;
+  const TW* src = table + (size_t)(known ? tok : 0) * dim;
+  for (int i = blockIdx.y * blockDim.x + threadIdx.x; 2 * i < dim; i += gridDim.y * blockDim.x) {
+    const double a = p * turns[i];
+    float s, c;
+    sincosf((float)(a - rint(a)) * 6.283185307179586f, &s, &c);
+    dst[2 * i] = known ? fmaf(scale, Elem<TW>::load(src + 2 * i), s) : __uint_as_float(0x7fc00000u);
+    if (2 * i + 1 < dim) dst[2 * i + 1] = known ? fmaf(scale, Elem<TW>::load(src + 2 * i + 1), c) : __uint_as_float(0x7fc00000u);
+  }
+}
+
+extern "C" int cwm_embedding_sinusoid(void* out, const void* table, int table_dtype, const int* tokens, const int* positions,
+                                      const double* turns, int n_tokens, int dim, int vocab, float scale, hipStream_t stream) {
+  CWM_REQUIRE(n_tokens >= 0 && dim > 0 && vocab > 0, "embedding_sinusoid: bad sizes T=%d D=%d V=%d", n_tokens, dim, vocab);
+  CWM_REQUIRE(out && table && tokens && positions && turns, "embedding_sinusoid: arguments missing");
+  if (n_tokens == 0) return 0;
+  const int pairs = (dim + 1) / 2;
+  const int threads = pairs >= 256 ? 256 : (pairs >= 128 ? 128 : 64);
+  const dim3 grid(n_tokens, n_tokens >= 512 ? 1 : (pairs + threads - 1) / threads);
+  if (table_dtype == CWM_F32)
+    hipLaunchKernelGGL(embedding_sinusoid_kernel<float>, grid, dim3(threads), 0, stream, (float*)out, (const float*)table, tokens,
+                       positions, turns, dim, vocab, scale);
+  else if (table_dtype == CWM_BF16)
+    hipLaunchKernelGGL(embedding_sinusoid_kernel<bf16_t>, grid, dim3(threads), 0, stream, (float*)out, (const bf16_t*)table, tokens,
+                       positions, turns, dim, vocab, scale);
+  else
+    return cwm_fail("embedding_sinusoid: unknown table dtype %d", table_dtype);
+  return cwm_launch_status("embedding_sinusoid");
+}
+
 // ---- h += delta (float32), out = h * rsqrt(mean(h^2) + eps) * w ---------------- //
 // One block per output row.  With `rows`, output row r is computed from source row
 // rows[r] and h is not modified.
@@ -374,8 +415,8 @@ extern "C" int cwm_sum_partials(void* out, int out_dtype, const float* partials,
 // ---- out = act(sum over p of x[p]) ------------------------------------------------ //
 // The activation between the two products of a feed-forward without a gate: `x` is [count] values of type TX, or
 // n_partials float32 slabs `count` apart that are added in order first; float32 arithmetic, rounded once.
-// kind 0: the square of relu; 1: relu; 2: gelu (tanh form); 3: silu.
-#define CWM_ACT_KINDS 4
+// kind 0: the square of relu; 1: relu; 2: gelu (tanh form); 3: silu; 4: gelu (erf form); 5: tanh.
+#define CWM_ACT_KINDS 6
 __device__ __forceinline__ float act_value(float z, int kind) {
   switch (kind) {
     case 0: {
@@ -386,6 +427,10 @@ __device__ __forceinline__ float act_value(float z, int kind) {
       return fmaxf(z, 0.f);
     case 2:
       return 0.5f * z * (1.f + tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z)));
+    case 4:
+      return 0.5f * z * (1.f + erff(z * 0.7071067811865476f));
+    case 5:
+      return tanhf(z);
     default:
       return z / (1.f + expf(-z));
   }

@@ -807,6 +807,16 @@ def _check_sink(sink: Optional[torch.Tensor], n_q: int) -> None:
         raise KernelError(f"the sinks must be a contiguous float32 [{n_q}] tensor, one a query head")
 
 
+def _check_bias(distance_bias: Optional[Tuple[torch.Tensor, torch.Tensor]], n_q: int) -> Tuple[Optional[torch.Tensor], Optional[torch.Tensor]]:
+    if distance_bias is None:
+        return None, None
+    for t in distance_bias:
+        _need_gpu(t)
+        if t.dtype != torch.float32 or t.shape != (n_q,) or not t.is_contiguous():
+            raise KernelError(f"a distance bias is two contiguous float32 [{n_q}] tensors, a slope and a rate a query head")
+    return distance_bias
+
+
 def _check_mask(window: Optional[int], chunk: Optional[int], softcap: Optional[float]) -> None:
     if window is not None and window < 1:
         raise KernelError("a window holds at least the query's own key")
@@ -828,6 +838,7 @@ def paged_attention_simple(
     sink: Optional[torch.Tensor] = None,
     softcap: Optional[float] = None,
     chunk: Optional[int] = None,
+    distance_bias: Optional[Tuple[torch.Tensor, torch.Tensor]] = None,
 ) -> torch.Tensor:
     """Causal attention of `q` [T, Hq, hd] over the paged cache by the plain kernel:
     float32 arithmetic, a key/value head's query heads sharing its keys and values, long
@@ -836,8 +847,10 @@ def paged_attention_simple(
     from the largest position, which costs a copy to the host).  `sink`: float32 [Hq], a term exp(sink) that
     each head's softmax denominator holds beside its keys (no key, no value, not scaled).  `softcap`: scaled scores
     become softcap * tanh(score / softcap) before the softmax.  `chunk` (instead of a window): a query reads the keys of
-    its own block of that many positions, counted from 0, up to itself.  Returns [T, Hq * hd]."""
+    its own block of that many positions, counted from 0, up to itself.  `distance_bias` (slope, rate), float32 [Hq]
+    each: slope_h * ln(1 + rate_h * (query's position - key's)) comes off the score.  Returns [T, Hq * hd]."""
     _need_gpu(q, cache, block_table, positions, seq_of_token, sink)
+    bias_slope, bias_rate = _check_bias(distance_bias, q.shape[1] if q.dim() == 3 else 0)
     _check_mask(window, chunk, softcap)
     _check_sink(sink, q.shape[1] if q.dim() == 3 else 0)
     if q.dim() != 3 or q.stride(2) != 1 or q.stride(1) != q.shape[2]:
@@ -871,7 +884,7 @@ def paged_attention_simple(
             _ptr(positions), _ptr(seq_of_token), ctypes.c_int(n_tokens), ctypes.c_int(n_q), ctypes.c_int(n_kv),
             ctypes.c_int(hd), ctypes.c_int(cache.shape[3] // hd), ctypes.c_int(cache.shape[0]),
             ctypes.c_int(-1 if window is None else window - 1), ctypes.c_int(chunk or 0), ctypes.c_float(scale),
-            ctypes.c_float(softcap or 0.0), ctypes.c_int(max_keys), _ptr(partial), _ptr(sink), _stream(),
+            ctypes.c_float(softcap or 0.0), ctypes.c_int(max_keys), _ptr(partial), _ptr(sink), _ptr(bias_slope), _ptr(bias_rate), _stream(),
         ),
     )
     return out
@@ -1010,9 +1023,12 @@ def paged_attention_mfma(
     sink: Optional[torch.Tensor] = None,
     softcap: Optional[float] = None,
     chunk: Optional[int] = None,
+    distance_bias: Optional[Tuple[torch.Tensor, torch.Tensor]] = None,
 ) -> torch.Tensor:
     """Matrix-core attention (bfloat16): prompt portions and decoded tokens in one
-    launch, long key ranges of short sequences split and merged.  `sink`, `softcap`, `chunk`: as in `paged_attention_simple`."""
+    launch, long key ranges of short sequences split and merged.  `sink`, `softcap`, `chunk`, `distance_bias`: as in
+    `paged_attention_simple`; the bias is a build of its own, so that the other models' kernel does without its instructions."""
+    bias_slope, bias_rate = _check_bias(distance_bias, q.shape[1] if q.dim() == 3 else 0)
     _need_gpu(q, cache, block_table, sink)
     _check_mask(window, chunk, softcap)
     _check_sink(sink, q.shape[1] if q.dim() == 3 else 0)
@@ -1039,7 +1055,7 @@ def paged_attention_mfma(
     partial = None
     if plan.n_partials:
         partial = torch.empty(plan.n_partials * n_kv * 16 * (hd + 4), dtype=torch.float32, device=q.device)
-    lib = _build.load("attention_mfma", {"HEAD_DIM": hd})
+    lib = _build.load("attention_mfma", {"HEAD_DIM": hd} if distance_bias is None else {"DISTANCE_BIAS": 1, "HEAD_DIM": hd})
     _check(
         lib,
         lib.cwm_attention_mfma(
@@ -1051,7 +1067,7 @@ def paged_attention_mfma(
             _ptr(plan.merge), ctypes.c_int(plan.n_merge), ctypes.c_int(plan.n_merge_mid), ctypes.c_int(plan.n_merge_wide), _ptr(partial),
             ctypes.c_int(n_q), ctypes.c_int(n_kv), ctypes.c_int(hd), ctypes.c_int(page_size),
             ctypes.c_int(cache.shape[0]), ctypes.c_int(-1 if window is None else window - 1), ctypes.c_int(chunk or 0),
-            ctypes.c_float(scale), ctypes.c_float(softcap or 0.0), _ptr(sink), _stream(),
+            ctypes.c_float(scale), ctypes.c_float(softcap or 0.0), _ptr(sink), _ptr(bias_slope), _ptr(bias_rate), _stream(),
         ),
     )
     return out
@@ -1067,6 +1083,7 @@ def paged_attention(
     sink: Optional[torch.Tensor] = None,
     softcap: Optional[float] = None,
     chunk: Optional[int] = None,
+    distance_bias: Optional[Tuple[torch.Tensor, torch.Tensor]] = None,
 ) -> torch.Tensor:
     """Attention of the step's tokens over the cache.  `batch` is the step's
     `StepBatch` (positions, sequence of each token and the per-sequence lengths).
@@ -1074,11 +1091,12 @@ def paged_attention(
     matrix cores; float32, and other sizes, on the plain kernel."""
     hd = q.shape[2]
     if q.is_cuda and mfma_attention_takes(q.dtype, hd, cache.shape[3] // hd):
-        return paged_attention_mfma(q, cache, block_table, batch, window, scale, sink, softcap, chunk)
+        return paged_attention_mfma(q, cache, block_table, batch, window, scale, sink, softcap, chunk, distance_bias)
     static = getattr(batch, "static", None)
     max_keys = batch.max_kv_len if static is None else static.max_keys
     return paged_attention_simple(
         q, cache, block_table, batch.positions, batch.seq_of_token, window, scale, max_keys=max_keys, sink=sink, softcap=softcap, chunk=chunk,
+        distance_bias=distance_bias,
     )
 
 
@@ -1231,7 +1249,7 @@ def measure_mfma_rate(device: torch.device, blocks: int, rounds: int, launches: 
 from .sequence import (  # noqa: E402
     MAX_CONV_TAPS, MAX_MEMORY_DIM, MAX_SSM_STATE, ScaledSum, add_layernorm, add_rows, cast_rows, causal_conv_silu, group_rmsnorm,
     layernorm_limits, matrix_memory, matrix_memory_state_elems, matrix_memory_state_unpack, scan_state_elems, scan_state_pack,
-    scan_state_unpack, selective_scan, sigmoid_mul, token_shift,
+    scan_state_unpack, selective_scan, sigmoid_mul, step_segments, token_shift,
 )
 from .routed import (  # noqa: E402
     MAX_EXPERTS, MAX_ROUTE_TOP, ExpertGroups, GatedActivation, absorb_queries, combine_routed, expand_values, group_by_expert,
@@ -1242,5 +1260,8 @@ from .streams import (  # noqa: E402
 )
 from .mixing import (  # noqa: E402
     MAX_GLA_DIM, MAX_SHORT_CONV_TAPS, MAX_SIDE_ADDENDS, MAX_SIDE_DIM, MAX_TALK_HEADS, gated_act_rows, gated_linear_attention, gla_state_elems,
-    gla_state_unpack, short_conv, talking_attention, token_side,
+    gla_state_unpack, short_conv, talking_attention, token_side, wkv,
+)
+from .recurrence import (  # noqa: E402
+    MAX_NORMED_ADDENDS, MAX_TOKEN_MIXES, NormedSum, add_normed_rmsnorm, embedding_sinusoid, min_gru, token_mixes,
 )

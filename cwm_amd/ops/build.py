@@ -65,7 +65,10 @@ SOURCES: Dict[str, Tuple[Mapping[str, int], ...]] = {
     "linear_attention": ({},),
     "short_conv": ({},),
     "token_side": ({},),
-    "attention_mfma": tuple({"HEAD_DIM": hd} for hd in (16, 32, 48, 64, 80, 96, 128, 256)),
+    "min_gru": ({},),
+    "token_mix": ({},),
+    "normed_sum": ({},),
+    "attention_mfma": tuple({"HEAD_DIM": hd} for hd in (16, 32, 48, 64, 80, 96, 128, 256)) + tuple({"DISTANCE_BIAS": 1, "HEAD_DIM": hd} for hd in (32, 48, 64, 128)),
 }
 
 

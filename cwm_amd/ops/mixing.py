@@ -205,16 +205,52 @@ def gated_linear_attention(
     same bits however a sequence is cut; in bfloat16 a step with a portion of more than `sequence.SCAN_SEGMENT` tokens
     runs its portions in segments side by side, the state carried across them, which differs from the walk by float32
     rounding."""
-    KernelError, _check, _code, _i32, _need_gpu, _ptr, _stream = _base()
-    _need_gpu(proj, decay_logits, weight, state)
-    n_tokens = proj.shape[0]
+    KernelError = _base()[0]
     width = heads * (2 * dim + 2 * vdim)
-    if proj.dim() != 2 or proj.stride(1) != 1 or proj.shape[1] < width or n_tokens != batch.n_tokens:
+    if proj.dim() != 2 or proj.stride(1) != 1 or proj.shape[1] < width:
         raise KernelError(f"the projection {tuple(proj.shape)} must be [{batch.n_tokens}, >= {width}] with contiguous rows")
+    if weight.shape != (vdim,):
+        raise KernelError(f"the weight must be a contiguous float32 [{vdim}]")
+    qk, vv = heads * dim, heads * vdim
+    parts = torch.split(proj[:, :width], (qk, qk, vv, vv), dim=1)
+    return _linear_attention(parts, None, decay_logits, weight, 0, state, batch, heads, dim, vdim, tau, eps, dim ** -0.5 if q_scale is None else q_scale)
+
+
+def wkv(
+    r: torch.Tensor, k: torch.Tensor, v: torch.Tensor, gate: torch.Tensor, decay_logits: torch.Tensor, bonus: torch.Tensor,
+    weight: torch.Tensor, state: torch.Tensor, batch: Any, heads: int, dim: int, vdim: int, eps: float,
+) -> torch.Tensor:
+    """Linear attention whose current token counts with a weight of its own (KIND_WKV of `csrc/linear_attention.hip`)
+    over the step's tokens.  `r`, `k` [T, heads * dim], `v`, `gate` [T, heads * vdim] of one type (rows may lie apart,
+    equally far in all four); `decay_logits` float32 [T, heads * dim]: a key channel decays by exp(-exp(logit)); `bonus`
+    float32 [heads * dim]; `weight` float32 [heads * vdim]; `state` float32 [slots, >= gla_state_elems], read and written
+    at the sequences' slots.  Returns [T, heads * vdim] in r's type: every head's result over its root mean square,
+    times weight, times silu(gate).  Portions are walked or cut into segments as in `gated_linear_attention`."""
+    KernelError, _check, _code, _i32, _need_gpu, _ptr, _stream = _base()
+    _need_gpu(bonus)
+    if bonus.dtype != torch.float32 or bonus.numel() != heads * dim or not bonus.is_contiguous():
+        raise KernelError(f"the bonus must be a contiguous float32 tensor of {heads * dim} values")
+    if weight.shape != (heads * vdim,):
+        raise KernelError(f"the weight must be a contiguous float32 [{heads * vdim}]")
+    return _linear_attention((r, k, v, gate), bonus, decay_logits, weight, vdim, state, batch, heads, dim, vdim, 1.0, eps, 1.0)
+
+
+def _linear_attention(
+    parts: Sequence[torch.Tensor], bonus: Optional[torch.Tensor], decay_logits: torch.Tensor, weight: torch.Tensor, weight_stride: int,
+    state: torch.Tensor, batch: Any, heads: int, dim: int, vdim: int, tau: float, eps: float, q_scale: float,
+) -> torch.Tensor:
+    """The launch that both forms share: `parts` are queries, keys, values and the output gate's projection."""
+    KernelError, _check, _code, _i32, _need_gpu, _ptr, _stream = _base()
+    proj = parts[0]
+    _need_gpu(*parts, decay_logits, weight, state)
+    n_tokens = proj.shape[0]
+    for t, n in zip(parts, (heads * dim, heads * dim, heads * vdim, heads * vdim)):
+        if t.dim() != 2 or tuple(t.shape) != (batch.n_tokens, n) or t.stride(1) != 1 or t.dtype != proj.dtype or (n_tokens > 1 and t.stride(0) != proj.stride(0)):
+            raise KernelError(f"a projection {tuple(t.shape)} {t.dtype} must be [{batch.n_tokens}, {n}] of {proj.dtype}, its rows as far apart as the others'")
     if decay_logits.dtype != torch.float32 or tuple(decay_logits.shape) != (n_tokens, heads * dim) or decay_logits.stride(1) != 1:
         raise KernelError(f"the decays' logits must be float32 [{n_tokens}, {heads * dim}]")
-    if weight.dtype != torch.float32 or weight.shape != (vdim,) or not weight.is_contiguous():
-        raise KernelError(f"the weight must be a contiguous float32 [{vdim}]")
+    if weight.dtype != torch.float32 or not weight.is_contiguous():
+        raise KernelError("the weight must be a contiguous float32 tensor")
     if dim > MAX_GLA_DIM:
         raise KernelError(f"heads of {dim} rows: the walking kernel takes up to {MAX_GLA_DIM}")
     need = gla_state_elems(heads, dim, vdim)
@@ -233,11 +269,12 @@ def gated_linear_attention(
     _check(
         lib,
         lib.cwm_gated_linear_attention(
-            _ptr(proj), ctypes.c_long(proj.stride(0) if n_tokens > 1 else proj.shape[1]), ctypes.c_int(_code(proj.dtype)),
-            _ptr(decay_logits), ctypes.c_long(decay_logits.stride(0) if n_tokens > 1 else heads * dim), _ptr(weight), _ptr(o_raw), _ptr(out),
+            *[_ptr(t) for t in parts], ctypes.c_long(proj.stride(0) if n_tokens > 1 else heads * dim), ctypes.c_int(_code(proj.dtype)), _ptr(bonus),
+            _ptr(decay_logits), ctypes.c_long(decay_logits.stride(0) if n_tokens > 1 else heads * dim), _ptr(weight), ctypes.c_int(weight_stride),
+            _ptr(o_raw), _ptr(out),
             _ptr(state), ctypes.c_long(state.shape[1]), _ptr(batch.state_slots), _ptr(batch.cu_q), ctypes.c_int(state.shape[0]),
             ctypes.c_int(n_tokens), ctypes.c_int(batch.n_seqs), ctypes.c_int(heads), ctypes.c_int(dim), ctypes.c_int(vdim),
-            ctypes.c_float(tau), ctypes.c_float(eps), ctypes.c_float(dim ** -0.5 if q_scale is None else q_scale), _ptr(segments),
+            ctypes.c_float(tau), ctypes.c_float(eps), ctypes.c_float(q_scale), _ptr(segments),
             ctypes.c_int(segments.shape[0] if segments is not None else 0), _ptr(seg_local), _ptr(seg_decay), _ptr(seg_start), ctypes.c_long(need), _stream(),
         ),
     )

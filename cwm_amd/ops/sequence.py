@@ -235,28 +235,37 @@ def scan_state_unpack(flat: torch.Tensor, heads: int, head_dim: int, n_state: in
 SCAN_SEGMENT = 256  # tokens of a segment; a step with a longer portion runs its portions' segments side by side
 
 
-def _scan_segments(batch: Any, device: torch.device):
-    """The step's list of segments for the scan kernel (int32 [n, 6] on the device: sequence, first token, end token,
-    number of the segment in its sequence, the sequence's first scratch entry, segments of the sequence), or None if
-    no portion is longer than a segment.  Built once a step from the host's copy of the portions' lengths."""
+def step_segments(batch: Any, device: torch.device, walk: int, segment: int, most: Optional[int] = None) -> Optional[torch.Tensor]:
+    """The step's portions cut into segments that a kernel runs side by side: int32 [n, 6] on the device, a row a
+    segment (sequence, first token, end token, number of the segment in its sequence, the sequence's first entry,
+    segments of the sequence), or None if no portion is longer than `walk` tokens.  A segment has `segment` tokens, or,
+    with `most`, as many more as leave the longest portion `most` segments.  Built once a step from the host's copy of
+    the portions' lengths."""
     q_lens = getattr(batch, "q_lens", None)
-    if not q_lens or max(q_lens) <= SCAN_SEGMENT:
+    if not q_lens or max(q_lens) <= walk:
         return None
+    if most is not None:
+        segment = max(segment, -(-max(q_lens) // most))
+    key = ("step_segments", segment)
     scratch = getattr(batch, "scratch", None)
-    if scratch is not None and "scan_segments" in scratch:
-        return scratch["scan_segments"]
+    if scratch is not None and key in scratch:
+        return scratch[key]
     rows, first, base = [], 0, 0
     for b, q in enumerate(q_lens):
-        n = -(-q // SCAN_SEGMENT)
-        for j in range(n):
-            rows.append((b, first + j * SCAN_SEGMENT, first + min(q, (j + 1) * SCAN_SEGMENT), j, base, n))
+        n = -(-q // segment)
+        rows.extend((b, first + j * segment, first + min(q, (j + 1) * segment), j, base, n) for j in range(n))
         first += q
         base += n
     host = torch.tensor(rows, dtype=torch.int32)
     table = (host.pin_memory() if device.type == "cuda" else host).to(device, non_blocking=True)
     if scratch is not None:
-        scratch["scan_segments"] = table
+        scratch[key] = table
     return table
+
+
+def _scan_segments(batch: Any, device: torch.device) -> Optional[torch.Tensor]:
+    """The segments of `SCAN_SEGMENT` tokens in which the scans with a matrix state run (`step_segments`)."""
+    return step_segments(batch, device, SCAN_SEGMENT, SCAN_SEGMENT)
 
 
 def selective_scan(

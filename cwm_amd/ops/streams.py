@@ -7,14 +7,14 @@ from __future__ import annotations
 
 import ctypes
 from dataclasses import dataclass
-from typing import Any, Optional, Union
+from typing import Any, Optional, Tuple, Union
 
 import torch
 
 from . import build as _build
 
 MAX_STREAMS = 8  # csrc/streams.hip: STREAMS_MAX
-ACTIVATIONS = {"relu2": 0, "relu": 1, "gelu_tanh": 2, "silu": 3}  # csrc/rowwise.hip: act_value
+ACTIVATIONS = {"relu2": 0, "relu": 1, "gelu_tanh": 2, "silu": 3, "gelu_erf": 4, "tanh": 5}  # csrc/rowwise.hip: act_value
 
 
 def _base():
@@ -252,6 +252,7 @@ def head_norm_rope_write(
     v_other: Optional[torch.Tensor] = None,
     v_mix: Optional[torch.Tensor] = None,
     keep_values: bool = False,
+    temperature: Optional[Tuple[float, int]] = None,
 ):
     """From the joined projection `qkv` ([T, >= Hq * qk_dim + Hkv * qk_dim + Hkv * v_dim] with q, k and v leading each
     row, or float32 partial sums [P, T, ...] of it) plus `bias` (float32, a value a column of q, k and v): every query
@@ -260,7 +261,8 @@ def head_norm_rope_write(
     [head_dim / 2], adjacent pairs, a frequency of 0 leaves its pair alone).  With `v_other` ([T, Hkv * v_dim] of
     `out_dtype`, rows may lie apart) and `v_mix` (one float32 on the device) the values become (1 - v_mix) v + v_mix
     v_other.  Returns the queries [T, Hq, head_dim] in `out_dtype` (zeros from qk_dim on), and with `keep_values` also
-    the values as they were cached, [T, Hkv * v_dim]; keys and values go into the paged `cache`.  float32 arithmetic."""
+    the values as they were cached, [T, Hkv * v_dim]; keys and values go into the paged `cache`.  With `temperature` =
+    (coef, every) the query at position p is multiplied by 1 + coef * ln(floor((p + 1) / every) + 1).  float32 arithmetic."""
     KernelError, _check, _code, _i32, _need_gpu, _ptr, _stream = _base()
     _need_gpu(qkv, bias, q_weight, k_weight, positions, inv_freq, cache, block_table, seq_of_token, v_other, v_mix)
     width = (n_q_heads + n_kv_heads) * qk_dim + n_kv_heads * v_dim
@@ -297,6 +299,8 @@ def head_norm_rope_write(
         if block_table.dim() != 2 or seq_of_token.numel() != n_tokens:
             raise KernelError("block_table must be [B, W] and seq_of_token [T]")
         num_pages, page_size, table_width = cache.shape[0], cache.shape[3] // head_dim, block_table.shape[1]
+    if temperature is not None and temperature[1] < 1:
+        raise KernelError("the queries' temperature rises every so many positions, at least one")
     if (v_other is None) != (v_mix is None):
         raise KernelError("another layer's values and their weight come together")
     other_stride = 0
@@ -317,7 +321,8 @@ def head_norm_rope_write(
             _ptr(positions), _ptr(seq_of_token), _ptr(inv_freq), _ptr(cache), _ptr(block_table),
             ctypes.c_int(table_width), ctypes.c_int(page_size), ctypes.c_int(num_pages), ctypes.c_int(n_tokens),
             ctypes.c_int(n_q_heads), ctypes.c_int(n_kv_heads), ctypes.c_int(qk_dim), ctypes.c_int(v_dim), ctypes.c_int(head_dim),
-            _ptr(v_other), ctypes.c_long(other_stride), _ptr(v_mix), _ptr(kept), _stream(),
+            _ptr(v_other), ctypes.c_long(other_stride), _ptr(v_mix), _ptr(kept), ctypes.c_float(temperature[0] if temperature else 0.0),
+            ctypes.c_int(temperature[1] if temperature else 0), _stream(),
         ),
     )
     return (q, kept) if keep_values else q

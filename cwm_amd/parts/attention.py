@@ -2,7 +2,7 @@
 
 from __future__ import annotations
 
-from typing import Any, Dict, Mapping, Optional
+from typing import Any, Dict, Mapping, Optional, Tuple
 
 import torch
 
@@ -414,8 +414,9 @@ register_part("mixer", "talking_attention", TalkingAttention)
 
 
 class HeadNormAttention(Mixer):
-    """Grouped-query attention over a paged cache with a norm of every query and key head, a cap on the scores, an
-    output gate, and optionally values blended with those of an earlier layer.
+    """Grouped-query attention over a paged cache with a norm of every query and key head, and, each where it is asked
+    for: a cap on the scores, an output gate, values blended with those of an earlier layer, queries that grow with
+    their position, scores that fall with the distance, and a softmax with one added to its denominator.
 
         q = W_q x + b_q, k = W_k x + b_k, v = W_v x + b_v        `n_heads` heads of `qk_dim`, `n_kv_heads` of `qk_dim` (keys)
                                                                  and `v_dim` (values); biases where `bias`
@@ -423,24 +424,27 @@ class HeadNormAttention(Mixer):
                                                                  (`qk_norm`; float32), before the rotation
         rotation of q and k by the position encoding             its table may turn fewer than qk_dim dimensions, in
                                                                  adjacent pairs or in halves of the turned part
+        q <- q (1 + coef ln(floor((p + 1) / every) + 1))         `query_temperature` = (coef, every), at position p
         v <- (1 - lam) v + lam v_source                          `value_mix="mix"`: v_source are the values that the layer
                                                                  with `value_mix="source"` and the same `value_mix_key`
                                                                  made of the same tokens in this step; lam is a stored
                                                                  scalar; the blended v is what is cached
         s_j = scale q . k_j;  s_j <- softcap tanh(s_j / softcap) where `softcap`
+        s_j <- s_j - r1_h ln(1 + r2_h (i - j))                   `distance_bias`: two stored numbers a query head
         softmax over the keys j <= i that the mask leaves: the last `window` keys (own included), or, with `chunk`, the keys
-            of the query's own block of `chunk` positions counted from the start of the sequence; neither: all
+            of the query's own block of `chunk` positions counted from the start of the sequence; neither: all.
+            With `unit_sink` its denominator is 1 + sum_j exp(s_j): a sink whose score is always 0
         out = W_o ([sum_j p_j v_j of every head] * sigmoid(W_g x))   the gate where `gate`, element by element
 
     Keys and values are cached with one head size, the larger of qk_dim and v_dim rounded up to a multiple of 16 (zeros
     beyond a head's own size; W_o and W_g are widened by zero columns and rows at load), so the attention kernels of
     equal key and value heads serve it.  `names` gives the tensors' local names for the roles q, k, v, o, g, q_bias,
-    k_bias, v_bias, q_norm, k_norm and value_mix."""
+    k_bias, v_bias, q_norm, k_norm, value_mix, bias_slope (r1) and bias_rate (r2)."""
 
     replayable = True
     DEFAULT_NAMES = {
         "q": "q", "k": "k", "v": "v", "o": "o", "g": "g", "q_bias": "q.b", "k_bias": "k.b", "v_bias": "v.b",
-        "q_norm": "q.norm", "k_norm": "k.norm", "value_mix": "vmix",
+        "q_norm": "q.norm", "k_norm": "k.norm", "value_mix": "vmix", "bias_slope": "r1", "bias_rate": "r2",
     }
 
     def __init__(
@@ -460,6 +464,9 @@ class HeadNormAttention(Mixer):
         gate: bool = True,
         value_mix: Optional[str] = None,
         value_mix_key: str = "values",
+        query_temperature: Optional[Tuple[float, int]] = None,
+        distance_bias: bool = False,
+        unit_sink: bool = False,
         position_encoding: Optional[PartChoice] = None,
         names: Optional[Mapping[str, str]] = None,
     ) -> None:
@@ -474,6 +481,8 @@ class HeadNormAttention(Mixer):
             raise ValueError("a window or a block holds at least the query's own key")
         if softcap is not None and not softcap > 0:
             raise ValueError("a cap on the scores must be positive")
+        if query_temperature is not None and query_temperature[1] < 1:
+            raise ValueError("the queries' temperature rises every so many positions, at least one")
         if value_mix not in (None, "source", "mix"):
             raise ValueError(f"value_mix {value_mix!r}: None, 'source' and 'mix' are known")
         self.dim, self.n_heads, self.n_kv_heads = dim, n_heads, n_kv_heads
@@ -481,6 +490,8 @@ class HeadNormAttention(Mixer):
         self.scale, self.window, self.chunk, self.softcap = float(scale), window, chunk, (float(softcap) if softcap is not None else None)
         self.bias, self.qk_norm, self.eps, self.gate = bias, qk_norm, float(eps), gate
         self.value_mix, self.value_mix_key = value_mix, value_mix_key
+        self.query_temperature = (float(query_temperature[0]), int(query_temperature[1])) if query_temperature is not None else None
+        self.distance_bias, self.unit_sink = distance_bias, unit_sink
         self.names = {**self.DEFAULT_NAMES, **dict(names or {})}
         self.position_encoding: Optional[PositionEncoding] = (
             position_encoding.build("position_encoding") if position_encoding is not None else None
@@ -511,6 +522,9 @@ class HeadNormAttention(Mixer):
             specs[n["g"]] = TensorSpec((self.n_heads * self.v_dim, self.dim))
         if self.value_mix is not None:  # the source layer stores the scalar too and does not use it
             specs[n["value_mix"]] = TensorSpec((), init="zeros", precision="stored")
+        if self.distance_bias:
+            specs[n["bias_slope"]] = TensorSpec((self.n_heads,), init="ones", precision="stored")
+            specs[n["bias_rate"]] = TensorSpec((self.n_heads,), init="ones", precision="stored")
         return specs
 
     def bind(self, tensors: Mapping[str, torch.Tensor], runtime: Runtime) -> None:
@@ -563,6 +577,10 @@ class HeadNormAttention(Mixer):
             wo = wide.reshape(self.dim, self.n_heads * self.head_dim)
         self.wo = LinearWeights(wo, stream_copy=runtime.stream_copies)
         self.lam = tensors[n["value_mix"]].float().reshape(1).contiguous() if self.value_mix == "mix" else None
+        self.bias_terms = None
+        if self.distance_bias:
+            self.bias_terms = (tensors[n["bias_slope"]].float().contiguous(), tensors[n["bias_rate"]].float().contiguous())
+        self.sinks = torch.zeros(self.n_heads, dtype=torch.float32, device=device) if self.unit_sink else None  # exp(0) = 1
 
     def forward(self, x: torch.Tensor, batch: Any, cache: Any, write_cache: bool = True) -> torch.Tensor:
         if not write_cache:
@@ -577,13 +595,16 @@ class HeadNormAttention(Mixer):
         result = ops.head_norm_rope_write(
             proj, self.n_heads, self.n_kv_heads, self.qk_dim, self.v_dim, self.head_dim, self.qkv_bias, self.q_weight, self.k_weight,
             self.eps, batch.positions, self.table, self.runtime.act_dtype, cache.cache, cache.block_table, batch.seq_of_token,
-            v_other=v_other, v_mix=self.lam, keep_values=self.value_mix == "source",
+            v_other=v_other, v_mix=self.lam, keep_values=self.value_mix == "source", temperature=self.query_temperature,
         )
         if self.value_mix == "source":
             q, batch.scratch[key] = result
         else:
             q = result
-        attn = ops.paged_attention(q, cache.cache, cache.block_table, batch, self.window, self.scale, softcap=self.softcap, chunk=self.chunk)
+        attn = ops.paged_attention(
+            q, cache.cache, cache.block_table, batch, self.window, self.scale, sink=self.sinks, softcap=self.softcap, chunk=self.chunk,
+            distance_bias=self.bias_terms,
+        )
         if self.gate:
             attn = ops.sigmoid_mul(attn, proj[:, self.qkv_width :])
         return self.wo(attn, partials_ok=True)  # added into the residual by the next norm
@@ -597,14 +618,21 @@ class SideBySide(Mixer):
     sum_i scale_i mixer_i(x).  `mixers` maps a name to (the mixer chosen, its factor); a child's tensors carry its
     name and a dot before their own.  Every child keeps a cache or state of its own (`children()` lists them in the
     order in which `forward` takes their views); the sum is left to whoever adds the result into the residual (an
-    `ops.ScaledSum`)."""
+    `ops.ScaledSum`).
 
-    def __init__(self, mixers: Mapping[str, Any]) -> None:
+    With `out_norm` (the eps) every child's result is divided by its rows' root mean square and multiplied by a weight of
+    the model's width (`dim`; tensor `<child>.<out_name>`) before its factor: sum_i scale_i rms(mixer_i(x)) w_i, an
+    `ops.NormedSum`."""
+
+    def __init__(self, mixers: Mapping[str, Any], out_norm: Optional[float] = None, dim: int = 0, out_name: str = "out") -> None:
         if not mixers:
             raise ValueError("at least one mixer is needed")
         self.names = list(mixers)
         self.parts = [mixers[name][0].build("mixer") for name in self.names]
         self.scales = [float(mixers[name][1]) for name in self.names]
+        self.out_norm, self.dim, self.out_name = out_norm, dim, out_name
+        if out_norm is not None and (dim < 1 or len(self.names) > ops.MAX_NORMED_ADDENDS):
+            raise ValueError(f"results that are normalised have a width, and at most {ops.MAX_NORMED_ADDENDS} of them are added up")
 
     @property
     def replayable(self) -> bool:
@@ -617,19 +645,27 @@ class SideBySide(Mixer):
         raise TypeError("mixers side by side have a cache each; the block asks `children()`")
 
     def tensor_specs(self) -> Dict[str, TensorSpec]:
-        return {f"{name}.{t}": spec for name, part in zip(self.names, self.parts) for t, spec in part.tensor_specs().items()}
+        specs = {f"{name}.{t}": spec for name, part in zip(self.names, self.parts) for t, spec in part.tensor_specs().items()}
+        if self.out_norm is not None:
+            specs.update({f"{name}.{self.out_name}": TensorSpec((self.dim,), init="norm", precision="stored") for name in self.names})
+        return specs
 
     def bind(self, tensors: Mapping[str, torch.Tensor], runtime: Runtime) -> None:
         super().bind(tensors, runtime)
         for name, part in zip(self.names, self.parts):
             prefix = name + "."
             part.bind({t[len(prefix):]: v for t, v in tensors.items() if t.startswith(prefix)}, runtime)
+        if self.out_norm is not None:
+            self.out_weights = [tensors[f"{name}.{self.out_name}"].float().contiguous() for name in self.names]
 
     def forward(self, x: torch.Tensor, batch: Any, cache: Any, write_cache: bool = True) -> Any:
         views = cache if isinstance(cache, tuple) else (cache,)
         if len(views) != len(self.parts):
             raise ValueError(f"{len(self.parts)} mixers side by side were given {len(views)} caches")
-        return ops.ScaledSum([(part.forward(x, batch, view, write_cache), scale) for part, view, scale in zip(self.parts, views, self.scales)])
+        results = [part.forward(x, batch, view, write_cache) for part, view in zip(self.parts, views)]
+        if self.out_norm is not None:
+            return ops.NormedSum(zip(results, self.out_weights, self.scales), self.out_norm)
+        return ops.ScaledSum(zip(results, self.scales))
 
 
 register_part("mixer", "side_by_side", SideBySide)

@@ -13,19 +13,36 @@ class PreNormBlock(Block):
     """h += mixer(norm1(h)); h += feed_forward(norm2(h))  (cwm/fastgen/forward.py:563-786).
 
     Each residual sum is done by the norm that follows it, in float32: the block
-    takes the previous layer's pending update and returns its own.
+    takes the previous layer's pending update and returns its own.  A layer without a feed-forward names none (a `norm2`
+    that it names all the same is not read).  A mixer that is several side by side (it lists them as `children()`) gets
+    a cache slot for each child.
     """
 
-    def __init__(self, names: Mapping[str, str], norm1: Norm, mixer: Mixer, norm2: Norm, feed_forward: FeedForward) -> None:
-        super().__init__(names, norm1=norm1, mixer=mixer, norm2=norm2, feed_forward=feed_forward)
+    def __init__(
+        self, names: Mapping[str, str], norm1: Norm, mixer: Mixer, norm2: Optional[Norm] = None, feed_forward: Optional[FeedForward] = None,
+    ) -> None:
+        if feed_forward is not None and norm2 is None:
+            raise ValueError("a feed-forward comes with its norm")
+        parts = dict(norm1=norm1, mixer=mixer)
+        if norm2 is not None:
+            parts["norm2"] = norm2
+        if feed_forward is not None:
+            parts["feed_forward"] = feed_forward
+        super().__init__(names, **parts)
         self.norm1 = norm1
         self.mixer = mixer
         self.norm2 = norm2
         self.feed_forward = feed_forward
 
-    def forward(self, h: torch.Tensor, delta: Optional[torch.Tensor], batch: Any, cache: Any, write_cache: bool = True) -> torch.Tensor:
+    def mixers(self):
+        children = getattr(self.mixer, "children", None)
+        return list(children()) if children is not None else [self.mixer]
+
+    def forward(self, h: torch.Tensor, delta: Any, batch: Any, cache: Any, write_cache: bool = True) -> Any:
         x = self.norm1.forward(h, delta)
         mixed = self.mixer.forward(x, batch, cache, write_cache)
+        if self.feed_forward is None:
+            return mixed
         x = self.norm2.forward(h, mixed)
         return self.feed_forward.forward(x, batch)
 

@@ -2,6 +2,7 @@
 
 from __future__ import annotations
 
+import math
 from typing import Any, Dict, Mapping, Optional
 
 import torch
@@ -71,6 +72,25 @@ class NormedTokenEmbedding(TokenEmbedding):
         return self.norm.normalize_(super().forward(batch))
 
 
+class SinusoidalTokenEmbedding(TokenEmbedding):
+    """h = scale * table[tokens] + s(position), with s(p)[2i] = sin(p * base^(-2i / dim)) and s(p)[2i + 1] the cosine of
+    the same angle; the angle is formed in float64 and the sum in float32."""
+
+    def __init__(self, vocab_size: int, dim: int, base: float, scale: Optional[float] = None, tensor: str = "weight") -> None:
+        super().__init__(vocab_size, dim, scale, tensor)
+        if not base > 0:
+            raise ValueError("the positions' base must be positive")
+        self.base = float(base)
+
+    def bind(self, tensors: Mapping[str, torch.Tensor], runtime: Runtime) -> None:
+        super().bind(tensors, runtime)
+        pair = torch.arange((self.dim + 1) // 2, dtype=torch.float64)
+        self.turns = (self.base ** (-2.0 * pair / self.dim) / (2.0 * math.pi)).to(self.table.device)
+
+    def forward(self, batch: Any) -> torch.Tensor:
+        return ops.embedding_sinusoid(batch.tokens, self.table, batch.positions, self.turns, self.scale)
+
+
 class LinearHead(Head):
     """logits = x W^T in float32 (cwm/fastgen/forward.py:820-821).  A model whose head is its embedding table
     gives this part the embedding's prefix: both then name the same tensor."""
@@ -95,4 +115,5 @@ class LinearHead(Head):
 
 register_part("embedding", "token_embedding", TokenEmbedding)
 register_part("embedding", "normed_embedding", NormedTokenEmbedding)
+register_part("embedding", "sinusoidal_embedding", SinusoidalTokenEmbedding)
 register_part("head", "linear_head", LinearHead)

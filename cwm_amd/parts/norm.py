@@ -19,24 +19,41 @@ class RMSNorm(Norm):
 
     replayable = True
 
-    def __init__(self, dim: int, eps: float, offset: float = 0.0, tensor: str = "weight") -> None:
+    def __init__(
+        self, dim: int, eps: float, offset: float = 0.0, tensor: str = "weight", scalar: bool = False, gain: float = 1.0, optional: bool = False,
+    ) -> None:
         """`offset` is added to the stored weight (1 for a weight that is stored around zero and applied as
-        1 + w); `tensor` is the weight's local name ("" where the folder names it by the part's prefix alone)."""
+        1 + w); `tensor` is the weight's local name ("" where the folder names it by the part's prefix alone).
+        `scalar`: the folder holds one number (a tensor of no dimensions) for all coordinates.  `gain`: a constant on
+        the result, which rides on the weight (a factor on the logits of a model whose head is a plain product, say).
+        `optional`: a norm that nothing reads (of a sublayer that the layer does not have); a folder may hold it."""
         self.dim = dim
         self.eps = float(eps)
         self.offset = float(offset)
         self.tensor = tensor
+        self.scalar = scalar
+        self.gain = float(gain)
+        self.optional = optional
 
     def tensor_specs(self) -> Dict[str, TensorSpec]:
-        return {self.tensor: TensorSpec((self.dim,), init="norm" if self.offset == 0.0 else "normal", precision="stored")}
+        shape = () if self.scalar else (self.dim,)
+        return {self.tensor: TensorSpec(shape, init="norm" if self.offset == 0.0 else "normal", precision="stored", optional=self.optional)}
 
     def bind(self, tensors: Mapping[str, torch.Tensor], runtime: Runtime) -> None:
         super().bind(tensors, runtime)
+        if self.optional:
+            return
         self.weight = tensors[self.tensor]
         if self.offset != 0.0:
             self.weight = (self.weight.float() + self.offset).contiguous()  # the sum in float32, once
+        if self.scalar or self.gain != 1.0:
+            self.weight = (self.weight.float() * self.gain).expand(self.dim).contiguous()
 
-    def forward(self, h: torch.Tensor, delta: Optional[torch.Tensor], rows: Optional[torch.Tensor] = None) -> torch.Tensor:
+    def forward(self, h: torch.Tensor, delta: Any, rows: Optional[torch.Tensor] = None) -> torch.Tensor:
+        if isinstance(delta, ops.NormedSum):
+            if self.weight.dtype != torch.float32:
+                self.weight = self.weight.float()
+            return ops.add_normed_rmsnorm(h, delta, self.weight, self.eps, self.runtime.act_dtype, rows)
         return ops.add_rmsnorm(h, delta, self.weight, self.eps, self.runtime.act_dtype, rows)
 
 

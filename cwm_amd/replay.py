@@ -17,7 +17,7 @@ little-endian float32 in the order of the entries and of `want`.  After every st
 requests hold at any time, each request's count rounded up to a multiple of 64;
 every layer group's pool is made for that many, so pages are used again.
 
-Further options: `--page-size P` (tokens in a page, default 16; pools of pages that do
+Further options: `--requests N` (state slots, i.e. requests live at a time, default 4); `--page-size P` (tokens in a page, default 16; pools of pages that do
 not divide 64 get one more page per live request, since a request's last page may be
 partly filled beyond its multiple of 64); `--pages all=N,8192=M` sets the pools' sizes in
 pages outright, by the group's window (`all`: the group that keeps every key);
@@ -167,6 +167,7 @@ def main(argv: Optional[List[str]] = None) -> int:
     parser.add_argument("--max-tokens", type=int, required=True)
     parser.add_argument("--device", default="cuda:0")
     parser.add_argument("--page-size", type=int, default=REPLAY_PAGE_SIZE, help="tokens in a page")
+    parser.add_argument("--requests", type=int, default=REPLAY_MAX_LIVE, help="state slots: the most requests live at a time")
     parser.add_argument("--pages", default="", help="pool sizes in pages by group, e.g. all=40,8192=12 (default: from --max-tokens)")
     parser.add_argument("--random-config", help="a config.json to run with random weights instead of --model")
     parser.add_argument("--seed", type=int, default=0, help="seed of those random weights")
@@ -189,7 +190,7 @@ def main(argv: Optional[List[str]] = None) -> int:
 
     os.makedirs(args.out, exist_ok=True)
     replayer = Replayer(
-        args.model, args.dtype, args.max_tokens, device=args.device, page_size=args.page_size, pages=pages,
+        args.model, args.dtype, args.max_tokens, device=args.device, page_size=args.page_size, max_requests=args.requests, pages=pages,
         random_config=random_config, seed=args.seed, std=args.std, page_log=args.page_log, num_graphs=args.graphs,
     )
     for line in sys.stdin:

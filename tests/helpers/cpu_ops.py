@@ -103,7 +103,7 @@ def qkv_rope_write(x, weight, bias, n_q_heads, n_kv_heads, head_dim, positions, 
     return qkv
 
 
-def paged_attention(q, cache, block_table, batch, window, scale, sink=None, softcap=None, chunk=None):
+def paged_attention(q, cache, block_table, batch, window, scale, sink=None, softcap=None, chunk=None, distance_bias=None):
     n_tokens, n_q, hd = q.shape
     n_kv = cache.shape[2]
     page_size = cache.shape[3] // hd
@@ -130,6 +130,9 @@ def paged_attention(q, cache, block_table, batch, window, scale, sink=None, soft
             s = (kk[g] @ q[t, h].float()) * scale
             if softcap is not None:
                 s = softcap * torch.tanh(s / softcap)
+            if distance_bias is not None:
+                slope, rate = (float(t[h]) for t in distance_bias)
+                s = s - slope * torch.log1p(rate * (p - torch.arange(lo, p + 1)).float())
             if sink is not None:  # one more term of the denominator, without a key or a value
                 w = torch.softmax(torch.cat([s, sink[h].float().reshape(1)]), -1)[:-1]
             else:
@@ -343,6 +346,10 @@ def act_rows(x, kind, out_dtype):
         z = torch.relu(z)
     elif kind == "gelu_tanh":
         z = torch.nn.functional.gelu(z, approximate="tanh")
+    elif kind == "gelu_erf":
+        z = torch.nn.functional.gelu(z)
+    elif kind == "tanh":
+        z = torch.tanh(z)
     else:
         z = z * torch.sigmoid(z)
     return z.to(out_dtype)
@@ -513,7 +520,7 @@ def add_layernorm(h, delta, weight, bias, eps, out_dtype, rows=None, weight2=Non
 
 
 def head_norm_rope_write(qkv, n_q_heads, n_kv_heads, qk_dim, v_dim, head_dim, bias, q_weight, k_weight, eps, positions, inv_freq, out_dtype,
-                         cache=None, block_table=None, seq_of_token=None, v_other=None, v_mix=None, keep_values=False):
+                         cache=None, block_table=None, seq_of_token=None, v_other=None, v_mix=None, keep_values=False, temperature=None):
     if qkv.dim() == 3:
         qkv = qkv.sum(0)
     n = qkv.shape[0]
@@ -526,6 +533,9 @@ def head_norm_rope_write(qkv, n_q_heads, n_kv_heads, qk_dim, v_dim, head_dim, bi
         q = q * torch.rsqrt((q * q).mean(-1, keepdim=True) + eps) * q_weight.float()
     if k_weight is not None:
         k = k * torch.rsqrt((k * k).mean(-1, keepdim=True) + eps) * k_weight.float()
+    if temperature is not None:
+        coef, every = temperature
+        q = q * (1.0 + coef * torch.log(((positions + 1) // every + 1).float()))[:, None, None]
     if v_other is not None:
         lam = float(v_mix.reshape(-1)[0])
         v = (1.0 - lam) * v + lam * v_other.float()
@@ -574,7 +584,70 @@ def matrix_memory(proj, gates, weight, state, batch, heads, dim, vdim, cap, eps,
     return (y.reshape(n, heads * vdim) * weight.float() * torch.sigmoid(g.reshape(n, heads * vdim))).to(proj.dtype)
 
 
+def embedding_sinusoid(tokens, table, positions, turns, scale=1.0):
+    out = table[tokens.long()].float() * scale
+    angle = 2.0 * math.pi * positions.double()[:, None] * turns[None]
+    out[:, 0::2] += torch.sin(angle).float()
+    out[:, 1::2] += torch.cos(angle).float()[:, : out.shape[1] // 2]
+    return out
+
+
+def add_normed_rmsnorm(h, delta, weight, eps, out_dtype, rows=None):
+    total = torch.zeros_like(h)
+    for t, w, c in delta.terms:
+        y = t.float().sum(0) if t.dim() == 3 else t.float()
+        total += c * y * torch.rsqrt((y * y).mean(-1, keepdim=True) + delta.eps) * w.float()
+    return add_rmsnorm(h, total, weight, eps, out_dtype, rows)
+
+
+def token_mixes(x, mu, state, state_offset, batch):
+    xf = x.float()
+    before = torch.cat([xf[:1], xf[:-1]])
+    for b in range(batch.n_seqs):
+        row = state[int(batch.state_slots[b])]
+        before[int(batch.cu_q[b])] = row[state_offset : state_offset + x.shape[1]]
+        row[state_offset : state_offset + x.shape[1]] = xf[int(batch.cu_q[b + 1]) - 1]
+    return (xf[None] + (before - xf)[None] * mu[:, None]).to(x.dtype)
+
+
+def min_gru(proj, z_bias, x_bias, state, batch, out_dtype):
+    width = z_bias.numel()
+    p = (proj.sum(0) if proj.dim() == 3 else proj).float()
+    z = torch.sigmoid(p[:, :width] + z_bias)
+    u = p[:, width : 2 * width] + x_bias
+    c = torch.where(u >= 0, u + 0.5, torch.sigmoid(u))
+    g = p[:, 2 * width : 3 * width]
+    y = torch.zeros_like(z)
+    for b in range(batch.n_seqs):
+        row = state[int(batch.state_slots[b])]
+        for t in range(int(batch.cu_q[b]), int(batch.cu_q[b + 1])):
+            row[:width] = (1.0 - z[t]) * row[:width] + z[t] * c[t]
+            y[t] = row[:width]
+    return (y * g * torch.sigmoid(g)).to(out_dtype)
+
+
+def wkv(r, k, v, gate, decay_logits, bonus, weight, state, batch, heads, dim, vdim, eps):
+    """The state's layout is the stand-in's own: per head the matrix [dim, vdim]."""
+    n = r.shape[0]
+    q, k = r.float().reshape(n, heads, dim), k.float().reshape(n, heads, dim)
+    v, g = v.float().reshape(n, heads, vdim), gate.float().reshape(n, heads, vdim)
+    alpha = torch.exp(-torch.exp(decay_logits.float())).reshape(n, heads, dim)
+    u = bonus.reshape(heads, dim)
+    y = torch.zeros((n, heads, vdim))
+    for b in range(batch.n_seqs):
+        row = state[int(batch.state_slots[b])]
+        S = row[: heads * dim * vdim].reshape(heads, dim, vdim).clone()
+        for t in range(int(batch.cu_q[b]), int(batch.cu_q[b + 1])):
+            kv = k[t][:, :, None] * v[t][:, None, :]
+            y[t] = torch.einsum("hde,hd->he", S + u[:, :, None] * kv, q[t])
+            S = alpha[t][:, :, None] * S + kv
+        row[: heads * dim * vdim] = S.reshape(-1)
+    y = y * torch.rsqrt((y * y).mean(-1, keepdim=True) + eps) * weight.float().reshape(heads, vdim)
+    return (y * (g * torch.sigmoid(g))).reshape(n, heads * vdim).to(r.dtype)
+
+
 STAND_INS = (
+    "embedding_sinusoid", "add_normed_rmsnorm", "token_mixes", "min_gru", "wkv",
     "talking_attention", "gated_linear_attention", "short_conv", "token_side", "gated_act_rows",
     "add_layernorm", "head_norm_rope_write", "matrix_memory",
     "embedding_streams", "stream_mix_norm", "act_rows", "qk_norm_rope_write",

@@ -2,7 +2,7 @@
 
     python bench.py [--gpus 1] [--steps K] [--warmup W] [--layers L] [--dtype bf16|fp32]
     python bench.py --shape llama8b --serve 64     (requests through the scheduler instead)
-    python bench.py --compare lapevik|segedra|dogotar|digasun   (another design beside the dense decoder of equal size instead)
+    python bench.py --compare lapevik|segedra|dogotar|digasun|sunusun   (another design beside the dense decoder of equal size instead)
 
 Default run: the layer sizes of the CWM-32B shape with random weights, a batch of 8
 requests at a context of 32,768 tokens each; a step is one decode step of the whole
@@ -419,9 +419,30 @@ DIGASUN_SIZES = {
     "w4096": (dict(width=4096, layers=8, heads=32, kv_heads=8, window=8192, linear_heads=32, ff_dense=7680, ff=1536, experts=32, top=4, shared=1536, taps=4, side=64), 7680),
 }
 
+
+def sunusun_config(width, layers, heads, kv_heads, recurrent, wkv_heads, ff, vocab=32768):
+    """A Sunusun model of `layers` layers in the order parallel, wkv, wkv, parallel: attention heads of 128 beside a gated
+    recurrence of `recurrent` elements, wkv heads of 64, a dense feed-forward in every layer, no shared tensors."""
+    left = {"heads": heads, "kv_heads": kv_heads, "dim": 128, "vdim": 128, "scale": 128 ** -0.5, "q_temp": {"coef": 0.1, "every": 4096}}
+    parallel = {"type": "parallel", "mixer": {"left": left, "right": {"width": recurrent}}}
+    wkv = {"type": "wkv", "mixer": {"heads": wkv_heads, "dim": 64}}
+    mlp = {"kind": "dense", "ff": ff}
+    return {
+        "architecture": "Sunusun", "vocab": vocab, "width": width, "norm": {"eps": 1e-5}, "logit_scale": 1.0,
+        "layers": [dict(parallel if i % 4 in (0, 3) else wkv, mlp=mlp) for i in range(layers)],
+    }
+
+
+# the same two widths; beside it also the Dogotar model of the same width, whose layers are the most alike
+SUNUSUN_SIZES = {
+    "w2048": (dict(width=2048, layers=8, heads=16, kv_heads=8, recurrent=2048, wkv_heads=32, ff=6144), 4096),
+    "w4096": (dict(width=4096, layers=8, heads=32, kv_heads=8, recurrent=4096, wkv_heads=64, ff=9216), 6144),
+}
+
+# design -> (sizes, maker of its configuration, other designs measured beside it at the size of the same name)
 COMPARISONS = {
-    "lapevik": (LAPEVIK_SIZES, lapevik_config), "segedra": (SEGEDRA_SIZES, segedra_config), "dogotar": (DOGOTAR_SIZES, dogotar_config),
-    "digasun": (DIGASUN_SIZES, digasun_config),
+    "lapevik": (LAPEVIK_SIZES, lapevik_config, ()), "segedra": (SEGEDRA_SIZES, segedra_config, ()), "dogotar": (DOGOTAR_SIZES, dogotar_config, ()),
+    "digasun": (DIGASUN_SIZES, digasun_config, ()), "sunusun": (SUNUSUN_SIZES, sunusun_config, ("dogotar",)),
 }
 
 
@@ -429,12 +450,13 @@ def compare_designs(args, device):
     """Prefill and decode of another design at sizes like a real model's layers, beside the dense decoder of equal
     width, depth and active feed-forward width: one JSON line."""
     out = {"compare": args.compare, "dtype": args.dtype, "batch": args.batch, "context": args.context, "prefill_tokens": args.prefill_tokens, "sizes": {}}
-    all_sizes, make_config = COMPARISONS[args.compare]
+    all_sizes, make_config, others = COMPARISONS[args.compare]
     names = [args.size] if args.size else list(all_sizes)
     for name in names:
         sizes, hidden = all_sizes[name]
         row = {}
-        for label, config in ((args.compare, make_config(**sizes)), ("llama3_dense", dense_like(sizes["width"], sizes["layers"], hidden))):
+        beside = [(other, COMPARISONS[other][1](**COMPARISONS[other][0][name][0])) for other in others]
+        for label, config in ((args.compare, make_config(**sizes)), *beside, ("llama3_dense", dense_like(sizes["width"], sizes["layers"], hidden))):
             if args.only and label != args.only:
                 continue
             bench = ShapeBench(f"{label} {name}", config, None, args.dtype, args.page, args.graphs, device)
@@ -484,7 +506,7 @@ def main() -> int:
     ap.add_argument("--new", type=int, default=512, help="tokens generated per request with --serve")
     ap.add_argument("--compare", default=None, choices=sorted(COMPARISONS), help="instead of the step benchmark: prefill and decode of another design beside the dense decoder of equal size")
     ap.add_argument("--size", default=None, choices=sorted(LAPEVIK_SIZES), help="with --compare: one size only")
-    ap.add_argument("--only", default=None, choices=sorted(COMPARISONS) + ["llama3_dense"], help="with --compare: one of the two models only")
+    ap.add_argument("--only", default=None, choices=sorted(COMPARISONS) + ["llama3_dense"], help="with --compare: one of the models only")
     args = ap.parse_args()
     if args.gpus != 1:
         print(f"bench.py: this engine runs on one GPU; --gpus {args.gpus} is not supported")

@@ -11,19 +11,32 @@
 //   S_t     = diag(alpha_t) S_(t-1) + k_t v_t^T
 //   out_t   as above, with a weight of heads x vdim values
 //
-// `gla_walk_kernel`: a block a (tile of value columns, head, sequence) walks the sequence's tokens of the step one by
-// one, from the state that the step before left in the sequence's slot, and leaves the new state there.  A thread
-// holds up to 32 rows of one column of S in registers; `split` neighbouring lanes share a column (a run of consecutive
-// rows each, a multiple of four, read from LDS sixteen bytes at a time) and add their parts of o_t by shuffles.  q, k, the decays and v of 16 (or 8) tokens are staged in LDS at a time,
-// in float32, the decays computed once a (token, channel).  The same tokens give the same bits however they are cut
-// into steps.  The state of a (head, tile) lies in memory in the order its threads hold it (row r of thread i at
-// [r][i]), so it is read and written in whole lines; only this kernel looks inside.
-// A step with a portion of more than a segment of tokens runs all its portions in segments side by side, in three
-// launches: every segment but a sequence's last from a zero state, leaving its own sum and the product of its decays
-// (MODE 1); `gla_carry_kernel`, which carries the states across a sequence's segments, start_(s+1) = decay_s *
-// start_s + sum_s; and every segment from its true start with its results (MODE 2).  That differs from the walk by
-// float32 rounding only.
-// `gla_out_kernel`: the norm of every head's o_t, its weight and the gate, a wavefront a (token, head).
+// Three ways through a step's tokens:
+//
+// `gla_walk_kernel`, MODE 0: a block a (tile of value columns, head, sequence) walks the sequence's tokens one by one,
+// from the state that the step before left in the sequence's slot, and leaves the new state there.  A thread holds up
+// to 32 rows of one column of S in registers; `split` neighbouring lanes share a column (a run of consecutive rows each,
+// a multiple of four, read from LDS sixteen bytes at a time) and add their parts of o_t by shuffles.  q, k, the decays
+// and v of 16 (or 8) tokens are staged in LDS at a time, in float32, the decays computed once a (token, channel).  The
+// same tokens give the same bits however they are cut into steps.  The state of a (head, tile) lies in memory in the
+// order its threads hold it (row r of thread i at [r][i]), so it is read and written in whole lines.
+//
+// Segments side by side: a step with long portions cuts them into segments and runs three launches: every segment but a
+// sequence's last from a zero state, leaving its own sum and the product of its decays (MODE 1); `gla_carry_kernel`,
+// which carries the states across a sequence's segments, start_(s+1) = decay_s * start_s + sum_s; and every segment from
+// its true start with its results (MODE 2).  That differs from the walk by float32 rounding only.
+//
+// `gla_block_kernel` is MODE 1 and MODE 2 on the matrix cores (float32 operands and sums), 16 tokens at a time: with
+// w the decays, P_t their products from the block's first token to t, and Q_s those after s to the block's last,
+//   o_t  = (q_t P)^T S + sum_(s <= t) a_ts v_s,     a_ts = sum_d q_t[d] k_s[d] w_(s+1)[d] .. w_t[d]
+//   S   <- diag(w_1 .. w_16) S + sum_s (k_s Q_s) v_s^T
+// (KIND_WKV: products up to t - 1, and a_tt = sum_d q_t u k_t).  Every factor is a product of decays, at most one: no
+// logarithm and no quotient of decays, which might overflow, is formed.  The state stays in the accumulators of the matrix
+// instruction (16 columns a wavefront, or 32), in the order that makes it the next product's operand as it is.
+// `gla_walk_kernel` has these two modes as well, for heads of more than GLA_BLOCK_DIM rows.
+//
+// The norm of every head's o_t, its weight and the gate are done where a block holds a head's columns of a token together;
+// else by `gla_out_kernel`, a wavefront a (token, head).
 #include "common.h"
 
 CWM_DEFINE_ERROR_API
@@ -35,25 +48,42 @@ CWM_DEFINE_ERROR_API
 
 extern "C" int cwm_gla_max_dim() { return GLA_MAX_DIM; }
 
-// lanes that share a column of the state: the fewest (1, 2, 4, 8) that leave a lane at most GLA_ROWS rows
-static inline int gla_split(int dim) {
+#define GLA_BLOCK_DIM 128  // rows of a head that gla_block_kernel takes at most
+
+extern "C" int cwm_gla_block_dim() { return GLA_BLOCK_DIM; }
+
+// lanes that share a column of the state: the fewest (1, 2, 4, 8) that leave a lane at most GLA_ROWS rows, and more of
+// them where a block would otherwise have twice the columns that a head has
+static inline int gla_split(int dim, int vdim) {
   int split = 1;
-  while (split < 8 && (dim + split - 1) / split > GLA_ROWS) split *= 2;
+  while (split < 8 && ((dim + split - 1) / split > GLA_ROWS || GLA_THREADS / split / 2 >= vdim)) split *= 2;
   return split;
 }
 // rows of a column that a lane holds: a multiple of 4
-static inline int gla_rows(int dim, int split) { return ((dim + split - 1) / split + 3) / 4 * 4; }
-extern "C" int cwm_gla_split(int dim) { return gla_split(dim); }
+__host__ __device__ static inline int gla_rows(int dim, int split) { return ((dim + split - 1) / split + 3) / 4 * 4; }
+extern "C" int cwm_gla_split(int dim, int vdim) { return gla_split(dim, vdim); }
 // float32 elements of a request's state
 extern "C" long cwm_gla_state_elems(int heads, int dim, int vdim) {
-  const int split = gla_split(dim), rows = gla_rows(dim, split), cols = GLA_THREADS / split;
+  const int split = gla_split(dim, vdim), rows = gla_rows(dim, split), cols = GLA_THREADS / split;
   return (long)heads * ((vdim + cols - 1) / cols) * rows * GLA_THREADS;
 }
 
-__device__ __forceinline__ int gla_rows_device(int dim, int split) { return ((dim + split - 1) / split + 3) / 4 * 4; }
-
 #define KIND_GLA 0
 #define KIND_WKV 1
+
+// One head's results of one token by one wavefront: o over its root mean square, times weight, times silu(gate).
+template <typename T>
+__device__ __forceinline__ void gla_finish(const float* o, const T* __restrict__ gate, const float* __restrict__ weight,
+                                           T* __restrict__ out, int vdim, float eps) {
+  const int lane = threadIdx.x & (CWM_WAVE - 1);
+  float sq = 0.f;
+  for (int e = lane; e < vdim; e += CWM_WAVE) sq += o[e] * o[e];
+  const float rstd = 1.0f / sqrtf(wave_sum(sq) / (float)vdim + eps);
+  for (int e = lane; e < vdim; e += CWM_WAVE) {
+    const float g = Elem<T>::load(gate + e);
+    Elem<T>::store(out + e, o[e] * rstd * weight[e] * (g / (1.0f + expf(-g))));
+  }
+}
 
 template <int KIND>
 __device__ __forceinline__ float gla_decay(float z, float inv_tau) {
@@ -70,7 +100,8 @@ __device__ __forceinline__ float gla_decay(float z, float inv_tau) {
 // MODE 2: a block a (tile, head, segment) walks from seg_start with results; a sequence's last segment writes the slot.
 template <typename T, int MODE, int KIND>
 __global__ void __launch_bounds__(GLA_THREADS)
-gla_walk_kernel(const T* __restrict__ q, const T* __restrict__ k, const T* __restrict__ v_in, long proj_ld,
+gla_walk_kernel(const T* __restrict__ q, const T* __restrict__ k, const T* __restrict__ v_in, const T* __restrict__ gate,
+                long proj_ld, const float* __restrict__ weight, int weight_stride, T* __restrict__ out, float eps,
                 const float* __restrict__ bonus, const float* __restrict__ z, long z_ld, float* __restrict__ o_raw,
                 float* __restrict__ state, long state_ld, const int* __restrict__ slots, const int* __restrict__ cu_q,
                 int n_slots, int heads, int dim, int vdim, int split, int chunk, float inv_tau, float q_scale,
@@ -78,7 +109,7 @@ gla_walk_kernel(const T* __restrict__ q, const T* __restrict__ k, const T* __res
                 const float* __restrict__ seg_start, long seg_ld) {
   extern __shared__ __attribute__((aligned(16))) float lds[];
   const int vt = blockIdx.x, h = blockIdx.y;
-  const int cols = GLA_THREADS / split, rows = gla_rows_device(dim, split), dpad = split * rows;
+  const int cols = GLA_THREADS / split, rows = gla_rows(dim, split), dpad = split * rows;
   const int col = threadIdx.x / split, part = threadIdx.x % split;
   const int e = vt * cols + col;  // this thread's value column
   const bool live = e < vdim;
@@ -87,6 +118,7 @@ gla_walk_kernel(const T* __restrict__ q, const T* __restrict__ k, const T* __res
   float* as = ks + chunk * dpad;    // [chunk][dpad]
   float* vs = as + chunk * dpad;    // [chunk][cols]
   float* cs = vs + chunk * cols;    // [chunk]: the share of a token's own value (KIND_WKV)
+  float* os = cs + chunk;           // [chunk][cols]: the results, where one tile holds all of a head's columns
   int b, t0, t1, seg = 0;
   bool last = true;
   if constexpr (MODE == 0) {
@@ -163,7 +195,20 @@ gla_walk_kernel(const T* __restrict__ q, const T* __restrict__ k, const T* __res
       }
       if constexpr (MODE != 1) {
         for (int off = 1; off < split; off *= 2) o += __shfl_xor(o, off, CWM_WAVE);
-        if (part == 0 && live) o_raw[(size_t)(c0 + tt) * heads * vdim + h * vdim + e] = o;
+        if (part == 0 && live) {
+          if (n_vt == 1)
+            os[tt * cols + col] = o;
+          else
+            o_raw[(size_t)(c0 + tt) * heads * vdim + h * vdim + e] = o;
+        }
+      }
+    }
+    if constexpr (MODE != 1) {
+      if (n_vt == 1) {
+        __syncthreads();
+        for (int tt = threadIdx.x / CWM_WAVE; tt < n; tt += GLA_THREADS / CWM_WAVE)
+          gla_finish(os + tt * cols, gate + (size_t)(c0 + tt) * proj_ld + h * vdim, weight + h * weight_stride,
+                     out + ((size_t)(c0 + tt) * heads + h) * vdim, vdim, eps);
       }
     }
   }
@@ -172,30 +217,329 @@ gla_walk_kernel(const T* __restrict__ q, const T* __restrict__ k, const T* __res
     if (r >= rows) continue;
     if constexpr (MODE == 1) {
       seg_local[(size_t)seg * seg_ld + tile_at + (size_t)r * GLA_THREADS] = S[r];
-      seg_decay[(size_t)seg * seg_ld + tile_at + (size_t)r * GLA_THREADS] = P[r];
+      if (vt == 0 && col == 0 && part * rows + r < dim) seg_decay[(size_t)seg * heads * dim + h * dim + part * rows + r] = P[r];
     } else {
       if (last) st[(size_t)r * GLA_THREADS] = S[r];
     }
   }
 }
 
-// The states at the segments' starts: a thread an element of the state walks the step's segments in their order.
+// sum over the 16 lanes of a row of the wavefront, in every one of them (row rotations of the vector unit's operands)
+__device__ __forceinline__ float row16_sum(float x) {
+  x += __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(x), 0x128, 0xf, 0xf, false));  // row_ror:8
+  x += __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(x), 0x124, 0xf, 0xf, false));  // row_ror:4
+  x += __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(x), 0x122, 0xf, 0xf, false));  // row_ror:2
+  x += __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(x), 0x121, 0xf, 0xf, false));  // row_ror:1
+  return x;
+}
+
+// four consecutive bfloat16 values of a row, zeros from `limit` on
+__device__ __forceinline__ uint2 load4_bf16(const bf16_t* row, int at, int limit, bool vec) {
+  uint2 x = make_uint2(0u, 0u);
+  if (vec) {
+    if (at < limit) x = *(const uint2*)(row + at);
+  } else {
+    uint32_t h[4];
+#pragma unroll
+    for (int i = 0; i < 4; ++i) h[i] = at + i < limit ? row[at + i] : 0u;
+    x.x = h[0] | (h[1] << 16), x.y = h[2] | (h[3] << 16);
+  }
+  return x;
+}
+
+__device__ __forceinline__ void unpack4_bf16(uint2 x, float (&v)[4]) {
+  v[0] = __uint_as_float(x.x << 16), v[1] = __uint_as_float(x.x & 0xffff0000u);
+  v[2] = __uint_as_float(x.y << 16), v[3] = __uint_as_float(x.y & 0xffff0000u);
+}
+
+// A block of four wavefronts a (64 * EC value columns, head, segment); wavefront w owns columns 16 EC w .. of them.
+// CS: channels of a token that a thread stages (16 threads a token): heads of up to 16 CS rows.  `segments` as above.
+// Matrix-core layout (v_mfma_f32_16x16x4_f32, lane = 16 g + m): A holds element [m][k = g], B [k = g][m], the result
+// rows 4 g + i (i = 0 .. 3) of column m.  Which four of the summed-over indices an instruction takes as its k is free as
+// long as A and B agree: with k = 4 g + i the accumulator register i of a tile of S is B as it stands.
+template <int MODE, int KIND, int CS, int EC>
 __global__ void __launch_bounds__(GLA_THREADS)
-gla_carry_kernel(const int* __restrict__ segments, int n_segments, const float* __restrict__ state, long state_ld,
-                 const int* __restrict__ slots, int n_slots, const float* __restrict__ seg_local,
+gla_block_kernel(const bf16_t* __restrict__ q, const bf16_t* __restrict__ k, const bf16_t* __restrict__ v,
+                 const bf16_t* __restrict__ gate, long proj_ld, const float* __restrict__ bonus, const float* __restrict__ z,
+                 long z_ld, const float* __restrict__ weight, int weight_stride, float eps, float* __restrict__ o_raw,
+                 bf16_t* __restrict__ out, float* __restrict__ state, long state_ld, const int* __restrict__ slots, int n_slots,
+                 int heads, int dim, int vdim, int split, float inv_tau, float q_scale, bool vec, const int* __restrict__ segments,
+                 float* __restrict__ seg_local, float* __restrict__ seg_decay, const float* __restrict__ seg_start, long seg_ld) {
+  constexpr int DP = 16 * CS, LD = DP + 4, DT = DP / 16, VC = 64 * EC, VLD = VC + 4;
+  __shared__ __attribute__((aligned(16))) float Qs[MODE == 2 ? 16 : 1][LD], Ks[16][LD], Ws[16][LD];
+  __shared__ __attribute__((aligned(16))) float Qp[MODE == 2 ? 16 : 1][LD], Kq[16][LD], dec[DP];
+  __shared__ __attribute__((aligned(16))) float Vs[16][VLD], As[MODE == 2 ? 16 : 1][20];
+  __shared__ float sq_part[MODE == 2 ? 4 : 1][16];
+  const int tid = threadIdx.x, lane = tid & 63, m = lane & 15, g = lane >> 4;
+  const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+  const int h = blockIdx.y, e0 = blockIdx.x * VC;
+  const bool whole_head = gridDim.x == 1;
+  const int* sg = segments + 6 * blockIdx.z;
+  const int b = sg[0], t0 = sg[1], t1 = sg[2], seg = sg[4] + sg[3];
+  const bool last = sg[3] == sg[5] - 1, alone = sg[5] == 1;
+  if (MODE == 1 && last) return;  // nothing comes after it
+  const int slot = slots[b];
+  if (slot < 0 || slot >= n_slots) return;
+
+  // the state's place in memory (the walking kernel's order)
+  const int cols = GLA_THREADS / split, rows = gla_rows(dim, split), n_vt = (vdim + cols - 1) / cols;
+  auto state_at = [&](int d, int e) -> long {  // -1: a row or column that the state does not have
+    if (d >= split * rows || e >= n_vt * cols) return -1;
+    const int vt = e / cols, col = e - vt * cols, part = d / rows, r = d - part * rows;
+    return (((long)h * n_vt + vt) * rows + r) * GLA_THREADS + col * split + part;
+  };
+  float* home = state + (size_t)slot * state_ld;
+  float4v S[DT][EC];
+#pragma unroll
+  for (int dt = 0; dt < DT; ++dt)
+#pragma unroll
+    for (int ec = 0; ec < EC; ++ec)
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        S[dt][ec][i] = 0.f;
+        if constexpr (MODE == 2) {
+          const long at = state_at(16 * dt + 4 * g + i, e0 + 16 * (EC * wave + ec) + m);
+          if (at >= 0) S[dt][ec][i] = alone ? home[at] : seg_start[(size_t)seg * seg_ld + at];
+        }
+      }
+  // the upper triangle of the block's scores is zero and stays so
+  if constexpr (MODE == 2) As[tid >> 4][tid & 15] = 0.f;
+
+  // staging: thread (token ts, slice sl) takes CS channels and 4 EC value columns of its token
+  const int ts = tid >> 4, sl = tid & 15;
+  uint2 rq[CS / 4], rk[CS / 4], rv[EC];
+  float rz[CS];
+  float u[CS];
+#pragma unroll
+  for (int i = 0; i < CS; ++i) u[i] = (KIND == KIND_WKV && MODE == 2 && sl * CS + i < dim) ? bonus[h * dim + sl * CS + i] : 1.f;
+  auto fetch = [&](int c0) {
+    const bool there = c0 + ts < t1;
+    const size_t row = (size_t)(there ? c0 + ts : t0) * proj_ld;
+    const float* zr = z + (size_t)(there ? c0 + ts : t0) * z_ld + h * dim;
+#pragma unroll
+    for (int i = 0; i < CS / 4; ++i) {
+      const int c = sl * CS + 4 * i, limit = there ? dim : 0;
+      if constexpr (MODE == 2) rq[i] = load4_bf16(q + row + h * dim, c, limit, vec);
+      rk[i] = load4_bf16(k + row + h * dim, c, limit, vec);
+#pragma unroll
+      for (int x = 0; x < 4; ++x) rz[4 * i + x] = c + x < limit ? zr[c + x] : 0.f;
+    }
+#pragma unroll
+    for (int i = 0; i < EC; ++i) rv[i] = load4_bf16(v + row + h * vdim, e0 + 4 * (EC * sl + i), there ? vdim : 0, vec);
+  };
+  float product = 1.f;  // MODE 1: of the segment's decays, in the thread that forms a channel's products
+  fetch(t0);
+  for (int c0 = t0; c0 < t1; c0 += 16) {
+    const int n = min(16, t1 - c0);
+    __syncthreads();  // the block of tokens before is done with
+#pragma unroll
+    for (int i = 0; i < CS / 4; ++i) {
+      float kk[4], ww[4];
+      const int c = sl * CS + 4 * i;
+      unpack4_bf16(rk[i], kk);
+#pragma unroll
+      for (int x = 0; x < 4; ++x) ww[x] = (ts < n && c + x < dim) ? gla_decay<KIND>(rz[4 * i + x], inv_tau) : 1.f;
+      *(float4*)&Ks[ts][c] = make_float4(kk[0], kk[1], kk[2], kk[3]);
+      *(float4*)&Ws[ts][c] = make_float4(ww[0], ww[1], ww[2], ww[3]);
+      if constexpr (MODE == 2) {
+        float qq[4];
+        unpack4_bf16(rq[i], qq);
+        *(float4*)&Qs[ts][c] = make_float4(qq[0] * q_scale, qq[1] * q_scale, qq[2] * q_scale, qq[3] * q_scale);
+      }
+    }
+#pragma unroll
+    for (int i = 0; i < EC; ++i) {
+      float vv[4];
+      unpack4_bf16(rv[i], vv);
+      *(float4*)&Vs[ts][4 * (EC * sl + i)] = make_float4(vv[0], vv[1], vv[2], vv[3]);
+    }
+    __syncthreads();
+    if (c0 + 16 < t1) fetch(c0 + 16);  // in flight while this block of tokens is worked on
+    bf16_t gt[4][EC];
+    if constexpr (MODE == 2) {
+#pragma unroll
+      for (int i = 0; i < 4; ++i)
+#pragma unroll
+        for (int ec = 0; ec < EC; ++ec) {
+          const int t = 4 * g + i, e = e0 + 16 * (EC * wave + ec) + m;
+          gt[i][ec] = (whole_head && t < n && e < vdim) ? gate[(size_t)(c0 + t) * proj_ld + h * vdim + e] : (bf16_t)0;
+        }
+    }
+    // ---- products of decays: queries from the block's start (threads of the last wavefronts), keys to its end ------- //
+    for (int job = GLA_THREADS - 1 - tid; job < 2 * DP; job += GLA_THREADS) {
+      const int c = job & (DP - 1);
+      float w[16], x[16];
+      if (job < DP) {
+#pragma unroll
+        for (int t = 0; t < 16; ++t) w[t] = Ws[t][c], x[t] = Ks[t][c];
+        float p = 1.f;
+#pragma unroll
+        for (int t = 15; t >= 0; --t) {
+          Kq[t][c] = x[t] * p;
+          p *= w[t];
+        }
+        dec[c] = p;
+        if constexpr (MODE == 1) product *= p;
+      } else if constexpr (MODE == 2) {
+#pragma unroll
+        for (int t = 0; t < 16; ++t) w[t] = Ws[t][c], x[t] = Qs[t][c];
+        float p = 1.f;
+#pragma unroll
+        for (int t = 0; t < 16; ++t) {
+          if constexpr (KIND == KIND_GLA) p *= w[t];
+          Qp[t][c] = x[t] * p;
+          if constexpr (KIND == KIND_WKV) p *= w[t];
+        }
+      }
+    }
+    // ---- scores within the block: key ts against the queries from its own token on, CS channels a lane ------------- //
+    if constexpr (MODE == 2) {
+      float p[CS];
+      float own = 0.f;
+#pragma unroll
+      for (int i = 0; i < CS; i += 4) {
+        const float4 kk = *(const float4*)&Ks[ts][sl * CS + i], qq = *(const float4*)&Qs[ts][sl * CS + i];
+        p[i] = kk.x, p[i + 1] = kk.y, p[i + 2] = kk.z, p[i + 3] = kk.w;
+        own = fmaf(qq.x * kk.x, u[i], own), own = fmaf(qq.y * kk.y, u[i + 1], own);
+        own = fmaf(qq.z * kk.z, u[i + 2], own), own = fmaf(qq.w * kk.w, u[i + 3], own);
+      }
+      own = row16_sum(own);
+      if (sl == 0) As[ts][ts] = own;
+      const int most = 15 - 4 * wave;  // the wavefront's first key has the most queries after it
+      for (int after = 1; after <= most; ++after) {
+        const int t = ts + after, tr = min(t, 15);
+        float dot = 0.f;
+#pragma unroll
+        for (int i = 0; i < CS; i += 4) {
+          const float4 w = *(const float4*)&Ws[tr][sl * CS + i], qq = *(const float4*)&Qs[tr][sl * CS + i];
+          if constexpr (KIND == KIND_GLA) p[i] *= w.x, p[i + 1] *= w.y, p[i + 2] *= w.z, p[i + 3] *= w.w;
+          dot = fmaf(qq.x, p[i], dot), dot = fmaf(qq.y, p[i + 1], dot), dot = fmaf(qq.z, p[i + 2], dot), dot = fmaf(qq.w, p[i + 3], dot);
+          if constexpr (KIND == KIND_WKV) p[i] *= w.x, p[i + 1] *= w.y, p[i + 2] *= w.z, p[i + 3] *= w.w;
+        }
+        dot = row16_sum(dot);
+        if (sl == 0 && t < 16) As[t][ts] = dot;
+      }
+    }
+    __syncthreads();
+    // ---- results from the state and from the block's own tokens, then the state -------------------------------------- //
+    float vb[EC][4];
+#pragma unroll
+    for (int ec = 0; ec < EC; ++ec)
+#pragma unroll
+      for (int i = 0; i < 4; ++i) vb[ec][i] = Vs[4 * g + i][16 * (EC * wave + ec) + m];
+    float4v o[EC];
+    if constexpr (MODE == 2) {
+#pragma unroll
+      for (int ec = 0; ec < EC; ++ec) o[ec] = (float4v){0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+      for (int dt = 0; dt < DT; ++dt) {
+        const float4v a = *(const float4v*)&Qp[m][16 * dt + 4 * g];
+#pragma unroll
+        for (int i = 0; i < 4; ++i)
+#pragma unroll
+          for (int ec = 0; ec < EC; ++ec) o[ec] = __builtin_amdgcn_mfma_f32_16x16x4f32(a[i], S[dt][ec][i], o[ec], 0, 0, 0);
+      }
+      const float4v a = *(const float4v*)&As[m][4 * g];
+#pragma unroll
+      for (int i = 0; i < 4; ++i)
+#pragma unroll
+        for (int ec = 0; ec < EC; ++ec) o[ec] = __builtin_amdgcn_mfma_f32_16x16x4f32(a[i], vb[ec][i], o[ec], 0, 0, 0);
+    }
+#pragma unroll
+    for (int dt = 0; dt < DT; ++dt) {
+      const float4v f = *(const float4v*)&dec[16 * dt + 4 * g];
+#pragma unroll
+      for (int ec = 0; ec < EC; ++ec)
+#pragma unroll
+        for (int i = 0; i < 4; ++i) S[dt][ec][i] *= f[i];
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        const float a = Kq[4 * g + i][16 * dt + m];
+#pragma unroll
+        for (int ec = 0; ec < EC; ++ec) S[dt][ec] = __builtin_amdgcn_mfma_f32_16x16x4f32(a, vb[ec][i], S[dt][ec], 0, 0, 0);
+      }
+    }
+    if constexpr (MODE == 2) {
+      if (whole_head) {
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+          float sq = 0.f;
+#pragma unroll
+          for (int ec = 0; ec < EC; ++ec) sq = fmaf(o[ec][i], o[ec][i], sq);  // columns past the head's are zero
+          sq = row16_sum(sq);
+          if (m == 0) sq_part[wave][4 * g + i] = sq;
+        }
+        __syncthreads();
+      }
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        const int t = 4 * g + i;
+        const float sq = whole_head ? (sq_part[0][t] + sq_part[1][t]) + (sq_part[2][t] + sq_part[3][t]) : 0.f;
+        const float rstd = 1.0f / sqrtf(sq / (float)vdim + eps);
+#pragma unroll
+        for (int ec = 0; ec < EC; ++ec) {
+          const int e = e0 + 16 * (EC * wave + ec) + m;
+          if (t < n && e < vdim) {
+            const size_t at = ((size_t)(c0 + t) * heads + h) * vdim + e;
+            if (whole_head) {
+              const float gv = bf16_to_f32(gt[i][ec]);
+              out[at] = f32_to_bf16(o[ec][i] * rstd * weight[h * weight_stride + e] * (gv / (1.0f + expf(-gv))));
+            } else {
+              o_raw[at] = o[ec][i];
+            }
+          }
+        }
+      }
+    }
+  }
+  if (MODE == 1 || last) {
+#pragma unroll
+    for (int dt = 0; dt < DT; ++dt)
+#pragma unroll
+      for (int ec = 0; ec < EC; ++ec)
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+          const long at = state_at(16 * dt + 4 * g + i, e0 + 16 * (EC * wave + ec) + m);
+          if (at < 0) continue;
+          if constexpr (MODE == 1)
+            seg_local[(size_t)seg * seg_ld + at] = S[dt][ec][i];
+          else
+            home[at] = S[dt][ec][i];
+        }
+  }
+  if constexpr (MODE == 1) {
+    const int c = GLA_THREADS - 1 - tid;
+    if (blockIdx.x == 0 && c < dim) seg_decay[(size_t)seg * heads * dim + h * dim + c] = product;
+  }
+}
+
+// The states at the segments' starts: a thread an element of a sequence's state walks the sequence's segments in order.
+__global__ void __launch_bounds__(GLA_THREADS)
+gla_carry_kernel(const int* __restrict__ segments, const float* __restrict__ state, long state_ld, const int* __restrict__ slots,
+                 int n_slots, int heads, int dim, int split, int n_vt, const float* __restrict__ seg_local,
                  const float* __restrict__ seg_decay, float* __restrict__ seg_start, long seg_ld, long elems) {
+  const int* sg = segments + 6 * blockIdx.y;
+  if (sg[3] != 0) return;  // the sequence's first segment stands for all of them
   const long i = (long)blockIdx.x * GLA_THREADS + threadIdx.x;
   if (i >= elems) return;
-  float cur = 0.f;
-  for (int s = 0; s < n_segments; ++s) {
-    const int* sg = segments + 6 * s;
-    const int seg = sg[4] + sg[3];
-    if (sg[3] == 0) {
-      const int slot = slots[sg[0]];
-      cur = (slot >= 0 && slot < n_slots) ? state[(size_t)slot * state_ld + i] : 0.f;
+  const int rows = gla_rows(dim, split);
+  const long line = i / GLA_THREADS;  // [head][tile][row]
+  const int h = (int)(line / (n_vt * rows)), d = ((int)(i % GLA_THREADS) % split) * rows + (int)(line % rows);
+  const float* dp = seg_decay + h * dim + min(d, dim - 1);  // rows past the head's hold zeros, which stay
+  const int slot = slots[sg[0]], first = sg[4], count = sg[5];
+  float cur = (slot >= 0 && slot < n_slots) ? state[(size_t)slot * state_ld + i] : 0.f;
+  for (int s = 0; s < count; s += 8) {
+    float add[8], keep[8];
+#pragma unroll
+    for (int a = 0; a < 8; ++a) {  // the last segment has neither sum nor decays: what lies past the others is not used
+      const size_t seg = first + min(s + a, max(count - 2, 0));
+      add[a] = seg_local[seg * seg_ld + i], keep[a] = dp[seg * heads * dim];
     }
-    seg_start[(size_t)seg * seg_ld + i] = cur;
-    if (sg[3] < sg[5] - 1) cur = fmaf(seg_decay[(size_t)seg * seg_ld + i], cur, seg_local[(size_t)seg * seg_ld + i]);
+#pragma unroll
+    for (int a = 0; a < 8; ++a) {
+      if (s + a < count) seg_start[(size_t)(first + s + a) * seg_ld + i] = cur;
+      cur = fmaf(keep[a], cur, add[a]);
+    }
   }
 }
 
@@ -204,15 +548,8 @@ __global__ void __launch_bounds__(CWM_WAVE)
 gla_out_kernel(const float* __restrict__ o_raw, const T* __restrict__ gate, long gate_ld, const float* __restrict__ weight,
                int weight_stride, T* __restrict__ out, int heads, int vdim, float eps) {
   const int t = blockIdx.x / heads, h = blockIdx.x - t * heads;
-  const float* o = o_raw + ((size_t)t * heads + h) * vdim;
-  float sq = 0.f;
-  for (int e = threadIdx.x; e < vdim; e += CWM_WAVE) sq += o[e] * o[e];
-  const float rstd = 1.0f / sqrtf(wave_sum(sq) / (float)vdim + eps);
-  for (int e = threadIdx.x; e < vdim; e += CWM_WAVE) {
-    const float g = Elem<T>::load(gate + (size_t)t * gate_ld + h * vdim + e);
-    const float y = o[e] * rstd * weight[h * weight_stride + e] * (g / (1.0f + expf(-g)));
-    Elem<T>::store(out + ((size_t)t * heads + h) * vdim + e, y);
-  }
+  gla_finish(o_raw + ((size_t)t * heads + h) * vdim, gate + (size_t)t * gate_ld + h * vdim, weight + h * weight_stride,
+             out + ((size_t)t * heads + h) * vdim, vdim, eps);
 }
 
 // q, k ([T][heads * dim]) and v, gate ([T][heads * vdim]) of `dtype`, rows proj_ld elements apart.  bonus: null
@@ -221,7 +558,9 @@ gla_out_kernel(const float* __restrict__ o_raw, const T* __restrict__ gate, long
 // [n_slots, state_ld] with cwm_gla_state_elems(...) <= state_ld elements a request; slots: int32 [n_seqs]; cu_q: int32
 // [n_seqs + 1].  o_raw: float32 [T, heads * vdim] scratch.  out: [T, heads * vdim] of `dtype`.  segments (or null: every
 // sequence is walked by one block a tile): int32 [n_segments][6] as above, all segments of the step in the order of the
-// sequences; seg_local, seg_decay, seg_start: float32 [n_segments][seg_ld] scratch.
+// sequences; seg_local, seg_start: float32 [n_segments][seg_ld] scratch, seg_decay: float32 [n_segments][heads * dim]
+// (all three null where every sequence is one segment).  Segments with bfloat16 and heads of up to GLA_BLOCK_DIM rows run
+// on the matrix cores.
 extern "C" int cwm_gated_linear_attention(const void* q, const void* k, const void* v, const void* gate, long proj_ld, int dtype,
                                           const float* bonus, const float* z, long z_ld, const float* weight,
                                           int weight_stride, float* o_raw, void* out, float* state, long state_ld,
@@ -235,35 +574,85 @@ extern "C" int cwm_gated_linear_attention(const void* q, const void* k, const vo
   CWM_REQUIRE(q && k && v && gate && z && weight && o_raw && out && state && slots && cu_q, "gated_linear_attention: arguments missing");
   CWM_REQUIRE(state_ld >= cwm_gla_state_elems(heads, dim, vdim), "gated_linear_attention: a state row of %ld elements is too short", state_ld);
   CWM_REQUIRE(n_seqs <= 65535 && heads <= 65535 && n_segments <= 65535, "gated_linear_attention: too many sequences, segments or heads for one launch");
-  CWM_REQUIRE(!segments || (n_segments >= 1 && seg_local && seg_decay && seg_start && seg_ld >= cwm_gla_state_elems(heads, dim, vdim)),
+  const bool several = seg_local != nullptr;
+  CWM_REQUIRE(!segments || n_segments >= 1, "gated_linear_attention: an empty list of segments");
+  CWM_REQUIRE(!several || (segments && seg_decay && seg_start && seg_ld >= cwm_gla_state_elems(heads, dim, vdim)),
               "gated_linear_attention: segments need their scratch states");
   if (n_tokens == 0 || n_seqs == 0) return 0;
-  const int split = gla_split(dim), cols = GLA_THREADS / split, n_vt = (vdim + cols - 1) / cols;
+  const int split = gla_split(dim, vdim), cols = GLA_THREADS / split, n_vt = (vdim + cols - 1) / cols;
   const int dpad = split * gla_rows(dim, split);
-  int chunk = GLA_CHUNK;
-  while (chunk > 1 && sizeof(float) * (size_t)chunk * (3 * dpad + cols + 1) > 49152) chunk /= 2;
-  const size_t lds = sizeof(float) * (size_t)chunk * (3 * dpad + cols + 1);
-  const dim3 grid(n_vt, heads, n_seqs), grid_seg(n_vt, heads, segments ? n_segments : 1);
   const long elems = cwm_gla_state_elems(heads, dim, vdim);
   const float inv_tau = bonus ? 1.0f : 1.0f / tau;
+  const bool on_matrix_cores = segments && dtype == CWM_BF16 && dim <= GLA_BLOCK_DIM;
+  CWM_REQUIRE(on_matrix_cores || !segments || several, "gated_linear_attention: segments need their scratch states");
+  auto carry = [&] {
+    hipLaunchKernelGGL(gla_carry_kernel, dim3((unsigned)((elems + GLA_THREADS - 1) / GLA_THREADS), n_segments), dim3(GLA_THREADS), 0,
+                       stream, segments, state, state_ld, slots, n_slots, heads, dim, split, n_vt, seg_local, seg_decay, seg_start,
+                       seg_ld, elems);
+  };
+  int tiles = n_vt;  // blocks that share a head's columns
+  if (on_matrix_cores) {
+    const int ec = vdim <= 64 ? 1 : 2;
+    tiles = (vdim + 64 * ec - 1) / (64 * ec);
+    const bool vec = dim % 4 == 0 && vdim % 4 == 0 && proj_ld % 4 == 0 &&
+                     (((uintptr_t)q | (uintptr_t)k | (uintptr_t)v) % 8) == 0;
+    const dim3 grid(tiles, heads, n_segments);
+#define CWM_GLA_BLOCK(MODE, KIND, CS, EC)                                                                                   \
+  hipLaunchKernelGGL((gla_block_kernel<MODE, KIND, CS, EC>), grid, dim3(GLA_THREADS), 0, stream, (const bf16_t*)q,            \
+                     (const bf16_t*)k, (const bf16_t*)v, (const bf16_t*)gate, proj_ld, bonus, z, z_ld, weight, weight_stride,  \
+                     eps, o_raw, (bf16_t*)out, state, state_ld, slots, n_slots, heads, dim, vdim, split, inv_tau, q_scale, vec, \
+                     segments, seg_local, seg_decay, seg_start, seg_ld)
+#define CWM_GLA_BLOCK_EC(MODE, KIND, CS)          \
+  do {                                            \
+    if (ec == 1)                                  \
+      CWM_GLA_BLOCK(MODE, KIND, CS, 1);           \
+    else                                          \
+      CWM_GLA_BLOCK(MODE, KIND, CS, 2);           \
+  } while (0)
+#define CWM_GLA_BLOCK_CS(MODE, KIND)              \
+  do {                                            \
+    if (dim <= 64)                                \
+      CWM_GLA_BLOCK_EC(MODE, KIND, 4);            \
+    else                                          \
+      CWM_GLA_BLOCK_EC(MODE, KIND, 8);            \
+  } while (0)
+#define CWM_GLA_BLOCK_KIND(MODE)                  \
+  do {                                            \
+    if (bonus)                                    \
+      CWM_GLA_BLOCK_CS(MODE, KIND_WKV);           \
+    else                                          \
+      CWM_GLA_BLOCK_CS(MODE, KIND_GLA);           \
+  } while (0)
+    if (several) {
+      CWM_GLA_BLOCK_KIND(1);
+      carry();
+    }
+    CWM_GLA_BLOCK_KIND(2);
+#undef CWM_GLA_BLOCK_KIND
+#undef CWM_GLA_BLOCK_CS
+#undef CWM_GLA_BLOCK_EC
+#undef CWM_GLA_BLOCK
+    const int status = cwm_launch_status("gated_linear_attention (blocks)");
+    if (status) return status;
+  } else {
+    int chunk = GLA_CHUNK;
+    while (chunk > 1 && sizeof(float) * (size_t)chunk * (3 * dpad + 2 * cols + 1) > 49152) chunk /= 2;
+    const size_t lds = sizeof(float) * (size_t)chunk * (3 * dpad + 2 * cols + 1);
+    const dim3 grid(n_vt, heads, n_seqs), grid_seg(n_vt, heads, segments ? n_segments : 1);
 #define CWM_GLA_WALK(T, MODE, KIND, GRID)                                                                                   \
   hipLaunchKernelGGL((gla_walk_kernel<T, MODE, KIND>), GRID, dim3(GLA_THREADS), lds, stream, (const T*)q, (const T*)k,         \
-                     (const T*)v, proj_ld, bonus, z, z_ld, o_raw,                                                              \
-                     state, state_ld, slots, cu_q, n_slots, heads, dim, vdim, split, chunk, inv_tau, q_scale, segments, seg_local, \
+                     (const T*)v, (const T*)gate, proj_ld, weight, weight_stride, (T*)out, eps, bonus, z, z_ld, o_raw, state,   \
+                     state_ld, slots, cu_q, n_slots, heads, dim, vdim, split, chunk, inv_tau, q_scale, segments, seg_local,     \
                      seg_decay, seg_start, seg_ld)
-#define CWM_GLA_KIND(T, KIND)                                                                                              \
-  do {                                                                                                                     \
-    if (segments) {                                                                                                        \
-      CWM_GLA_WALK(T, 1, KIND, grid_seg);                                                                                        \
-      hipLaunchKernelGGL(gla_carry_kernel, dim3((unsigned)((elems + GLA_THREADS - 1) / GLA_THREADS)), dim3(GLA_THREADS), 0,  \
-                         stream, segments, n_segments, state, state_ld, slots, n_slots, seg_local, seg_decay, seg_start,     \
-                         seg_ld, elems);                                                                                     \
-      CWM_GLA_WALK(T, 2, KIND, grid_seg);                                                                                        \
-    } else {                                                                                                               \
-      CWM_GLA_WALK(T, 0, KIND, grid);                                                                                            \
-    }                                                                                                                      \
-    hipLaunchKernelGGL((gla_out_kernel<T>), dim3(n_tokens * heads), dim3(CWM_WAVE), 0, stream, o_raw,                        \
-                       (const T*)gate, proj_ld, weight, weight_stride, (T*)out, heads, vdim, eps);                           \
+#define CWM_GLA_KIND(T, KIND)                     \
+  do {                                            \
+    if (segments) {                               \
+      CWM_GLA_WALK(T, 1, KIND, grid_seg);         \
+      carry();                                    \
+      CWM_GLA_WALK(T, 2, KIND, grid_seg);         \
+    } else {                                      \
+      CWM_GLA_WALK(T, 0, KIND, grid);             \
+    }                                             \
   } while (0)
 #define CWM_GLA(T)                  \
   do {                              \
@@ -272,11 +661,22 @@ extern "C" int cwm_gated_linear_attention(const void* q, const void* k, const vo
     else                            \
       CWM_GLA_KIND(T, KIND_GLA);    \
   } while (0)
-  if (dtype == CWM_F32) CWM_GLA(float);
-  else if (dtype == CWM_BF16) CWM_GLA(bf16_t);
-  else return cwm_fail("gated_linear_attention: unknown element type %d", dtype);
+    if (dtype == CWM_F32) CWM_GLA(float);
+    else if (dtype == CWM_BF16) CWM_GLA(bf16_t);
+    else return cwm_fail("gated_linear_attention: unknown element type %d", dtype);
 #undef CWM_GLA
 #undef CWM_GLA_KIND
 #undef CWM_GLA_WALK
-  return cwm_launch_status("gated_linear_attention");
+    const int status = cwm_launch_status("gated_linear_attention");
+    if (status) return status;
+  }
+  if (tiles > 1) {
+    if (dtype == CWM_F32)
+      hipLaunchKernelGGL((gla_out_kernel<float>), dim3(n_tokens * heads), dim3(CWM_WAVE), 0, stream, o_raw, (const float*)gate,
+                         proj_ld, weight, weight_stride, (float*)out, heads, vdim, eps);
+    else
+      hipLaunchKernelGGL((gla_out_kernel<bf16_t>), dim3(n_tokens * heads), dim3(CWM_WAVE), 0, stream, o_raw, (const bf16_t*)gate,
+                         proj_ld, weight, weight_stride, (bf16_t*)out, heads, vdim, eps);
+  }
+  return cwm_launch_status("gated_linear_attention (results)");
 }

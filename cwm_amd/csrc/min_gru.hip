@@ -1,4 +1,4 @@
-// A gated recurrence whose gates read the current token only, an element of the state at a time (minGRU):
+// minGRU: every element of a state is an average over time whose weight depends on the token alone, not on the state:
 //
 //   z_t = sigmoid(a_t + b_z),   c_t = g(u_t + b_x)        a, u: projections of the token;  g(u) = u + 1/2 for u >= 0,
 //   S_t = (1 - z_t) S_(t-1) + z_t c_t                     sigmoid(u) for u < 0
@@ -21,7 +21,6 @@
 CWM_DEFINE_ERROR_API
 
 #define MGRU_THREADS 128
-#define MGRU_AHEAD 4  // tokens whose loads are in flight together
 
 template <typename T, int CH> struct Cols;
 template <typename T> struct Cols<T, 1> {
@@ -43,16 +42,29 @@ template <> struct Cols<bf16_t, 2> {
   static __device__ __forceinline__ void store(bf16_t* p, const float (&v)[2]) { *(uint32_t*)p = pack2_bf16(v[0], v[1]); }
 };
 
+// FAST: the hardware's exponential and reciprocal, each within a unit in the last place of float32 or so (results that
+// are stored in bfloat16); else the library's.
+template <bool FAST>
+__device__ __forceinline__ float exp_of(float x) {
+  return FAST ? __builtin_amdgcn_exp2f(x * 1.4426950408889634f) : expf(x);
+}
+template <bool FAST>
+__device__ __forceinline__ float inverse_of(float x) {
+  return FAST ? __builtin_amdgcn_rcpf(x) : 1.0f / x;
+}
+
 // sigmoid(v) and 1 - sigmoid(v)
+template <bool FAST>
 __device__ __forceinline__ void gate_pair(float v, float& open, float& keep) {
-  const float e = expf(-fabsf(v));
-  const float inv = 1.0f / (1.0f + e);
+  const float e = exp_of<FAST>(-fabsf(v));
+  const float inv = inverse_of<FAST>(1.0f + e);
   open = v >= 0.f ? inv : e * inv;
   keep = v >= 0.f ? e * inv : inv;
 }
 
+template <bool FAST>
 __device__ __forceinline__ float candidate_of(float u) {
-  return u >= 0.f ? u + 0.5f : 1.0f / (1.0f + expf(-u));
+  return u >= 0.f ? u + 0.5f : inverse_of<FAST>(1.0f + exp_of<FAST>(-u));
 }
 
 // segments: int32 [n][6]: sequence, first token, end token, number of the segment in its sequence, the sequence's first
@@ -63,6 +75,8 @@ min_gru_walk_kernel(const TS* __restrict__ proj, long ld, int n_partials, long p
                     const float* __restrict__ x_bias, TO* __restrict__ out, float* __restrict__ state, long state_ld,
                     const int* __restrict__ slots, const int* __restrict__ cu_q, int n_slots, int width,
                     const int* __restrict__ segments, float* __restrict__ seg_sum, float* __restrict__ seg_keep) {
+  constexpr bool FAST = sizeof(TO) == 2;
+  constexpr int AHEAD = MODE == 0 ? 2 : 8;  // tokens whose loads are in flight together, while those before are worked on
   const int c0 = CH * (blockIdx.x * MGRU_THREADS + threadIdx.x);
   if (c0 >= width) return;
   int b, t0, t1, number = 0, base = 0;
@@ -93,10 +107,18 @@ min_gru_walk_kernel(const TS* __restrict__ proj, long ld, int n_partials, long p
     const size_t held = (size_t)(base + segments[6 * blockIdx.y + 5] - 1) * width + c0;
 #pragma unroll
     for (int i = 0; i < CH; ++i) S[i] = seg_sum[held + i];
-    for (int s = 0; s < number; ++s) {
-      const size_t at = (size_t)(base + s) * width + c0;
+    for (int s = 0; s < number; s += 16) {  // sixteen segments' loads in flight
+      float keep[16][CH], add[16][CH];
 #pragma unroll
-      for (int i = 0; i < CH; ++i) S[i] = fmaf(seg_keep[at + i], S[i], seg_sum[at + i]);
+      for (int a = 0; a < 16; ++a) {
+        const size_t at = (size_t)(base + min(s + a, number - 1)) * width + c0;
+        Cols<float, CH>::load(seg_keep + at, keep[a]);
+        Cols<float, CH>::load(seg_sum + at, add[a]);
+      }
+#pragma unroll
+      for (int a = 0; a < 16; ++a)
+#pragma unroll
+        for (int i = 0; i < CH; ++i) S[i] = s + a < number ? fmaf(keep[a][i], S[i], add[a][i]) : S[i];
     }
   }
   auto fetch = [&](int t, int part, float (&v)[CH]) {
@@ -109,26 +131,39 @@ min_gru_walk_kernel(const TS* __restrict__ proj, long ld, int n_partials, long p
       for (int i = 0; i < CH; ++i) v[i] += more[i];
     }
   };
-  for (int t = t0; t < t1; t += MGRU_AHEAD) {
-    float z[MGRU_AHEAD][CH], x[MGRU_AHEAD][CH], y[MGRU_AHEAD][CH];
+  float z[AHEAD][CH], x[AHEAD][CH], y[AHEAD][CH];
+  auto fetch_from = [&](int t) {
 #pragma unroll
-    for (int a = 0; a < MGRU_AHEAD; ++a) {
+    for (int a = 0; a < AHEAD; ++a) {
       const int tt = min(t + a, t1 - 1);  // past the last token: that one again, not used
       fetch(tt, 0, z[a]);
       fetch(tt, 1, x[a]);
       if constexpr (MODE != 1) fetch(tt, 2, y[a]);
     }
+  };
+  fetch_from(t0);
+  for (int t = t0; t < t1; t += AHEAD) {
+    // what does not depend on the state, then the next tokens' loads, then the chain through the state
+    float keep[AHEAD][CH], add[AHEAD][CH], shown[AHEAD][CH];
 #pragma unroll
-    for (int a = 0; a < MGRU_AHEAD; ++a) {
+    for (int a = 0; a < AHEAD; ++a)
+#pragma unroll
+      for (int i = 0; i < CH; ++i) {
+        float open;
+        gate_pair<FAST>(z[a][i] + bz[i], open, keep[a][i]);
+        add[a][i] = open * candidate_of<FAST>(x[a][i] + bx[i]);
+        if constexpr (MODE != 1) shown[a][i] = y[a][i] * inverse_of<FAST>(1.0f + exp_of<FAST>(-y[a][i]));
+      }
+    if (t + AHEAD < t1) fetch_from(t + AHEAD);
+#pragma unroll
+    for (int a = 0; a < AHEAD; ++a) {
       if (t + a < t1) {
         float o[CH];
 #pragma unroll
         for (int i = 0; i < CH; ++i) {
-          float open, keep;
-          gate_pair(z[a][i] + bz[i], open, keep);
-          S[i] = fmaf(keep, S[i], open * candidate_of(x[a][i] + bx[i]));
-          if constexpr (MODE == 1) K[i] *= keep;
-          if constexpr (MODE != 1) o[i] = S[i] * (y[a][i] / (1.0f + expf(-y[a][i])));
+          S[i] = fmaf(keep[a][i], S[i], add[a][i]);
+          if constexpr (MODE == 1) K[i] *= keep[a][i];
+          if constexpr (MODE != 1) o[i] = S[i] * shown[a][i];
         }
         if constexpr (MODE != 1) Cols<TO, CH>::store(out + (size_t)(t + a) * width + c0, o);
       }

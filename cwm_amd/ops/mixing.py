@@ -160,31 +160,37 @@ GLA_THREADS = 256  # csrc/linear_attention.hip: threads of a walking block
 GLA_ROWS = 32  # and the rows of a column of the state that one of them holds at most
 
 
-def gla_split(dim: int) -> int:
-    """Lanes that share a column of a head's state: the fewest (1, 2, 4, 8) that leave a lane at most GLA_ROWS rows."""
+GLA_BLOCK_DIM = 128  # rows of a head that the kernel on the matrix cores takes at most
+GLA_WALK = 16  # tokens of the longest portion that a step still walks one by one
+GLA_SEGMENT = 128  # tokens of a segment on the matrix cores; half of it where that gives the chip too few blocks
+
+
+def gla_split(dim: int, vdim: int) -> int:
+    """Lanes that share a column of a head's state: the fewest (1, 2, 4, 8) that leave a lane at most GLA_ROWS rows and a
+    block no more than twice a head's columns."""
     split = 1
-    while split < 8 and -(-dim // split) > GLA_ROWS:
+    while split < 8 and (-(-dim // split) > GLA_ROWS or GLA_THREADS // split // 2 >= vdim):
         split *= 2
     return split
 
 
-def gla_rows(dim: int) -> int:
+def gla_rows(dim: int, vdim: int) -> int:
     """Rows of a column of a head's state that one lane holds: a multiple of 4."""
-    return -(-(-(-dim // gla_split(dim))) // 4) * 4
+    return -(-(-(-dim // gla_split(dim, vdim))) // 4) * 4
 
 
 def gla_state_elems(heads: int, dim: int, vdim: int) -> int:
     """float32 elements of one request's state of a gated linear attention, in the walking kernel's own order: per
     (head, tile of value columns) the rows a thread holds, [row][thread]."""
-    split = gla_split(dim)
-    rows, cols = gla_rows(dim), GLA_THREADS // split
+    split = gla_split(dim, vdim)
+    rows, cols = gla_rows(dim, vdim), GLA_THREADS // split
     return heads * -(-vdim // cols) * rows * GLA_THREADS
 
 
 def gla_state_unpack(flat: torch.Tensor, heads: int, dim: int, vdim: int) -> torch.Tensor:
     """S [heads, dim, vdim] of one request's state row (tests read states this way)."""
-    split = gla_split(dim)
-    rows, cols = gla_rows(dim), GLA_THREADS // split
+    split = gla_split(dim, vdim)
+    rows, cols = gla_rows(dim, vdim), GLA_THREADS // split
     n_vt = -(-vdim // cols)
     # [head][tile][row r][column][part]: element (d = part * rows + r, e = tile * cols + column)
     t = flat[: heads * n_vt * rows * GLA_THREADS].reshape(heads, n_vt, rows, cols, split)
@@ -202,9 +208,9 @@ def gated_linear_attention(
     float32 [vdim]; `state` float32 [slots, >= gla_state_elems], read and written at the sequences' slots.  Queries are
     multiplied by `q_scale` (default dim ** -0.5).  Returns [T, heads * vdim] in proj's type: every head's result over
     its root mean square, times weight, times silu(gate).  A step's portions are walked token by token, which gives the
-    same bits however a sequence is cut; in bfloat16 a step with a portion of more than `sequence.SCAN_SEGMENT` tokens
-    runs its portions in segments side by side, the state carried across them, which differs from the walk by float32
-    rounding."""
+    same bits however a sequence is cut; in bfloat16 a step with a portion of more than `GLA_WALK` tokens takes its
+    portions in blocks of 16 tokens on the matrix cores (float32 operands), long ones in segments side by side with the
+    state carried across them, which differs from the walk by float32 rounding."""
     KernelError = _base()[0]
     width = heads * (2 * dim + 2 * vdim)
     if proj.dim() != 2 or proj.stride(1) != 1 or proj.shape[1] < width:
@@ -258,13 +264,23 @@ def _linear_attention(
         raise KernelError(f"the state must be a contiguous float32 [slots, >= {need}] tensor")
     o_raw = torch.empty((n_tokens, heads * vdim), dtype=torch.float32, device=proj.device)
     out = torch.empty((n_tokens, heads * vdim), dtype=proj.dtype, device=proj.device)
-    # long portions in bfloat16 run in segments side by side (float32 keeps to the walk, whose bits no cut changes)
-    from .sequence import _scan_segments
+    # portions in bfloat16 go in blocks of tokens on the matrix cores, long ones in segments side by side (float32 keeps to
+    # the walk, whose bits no cut changes)
+    from .sequence import SCAN_SEGMENT, step_segments
 
-    segments = _scan_segments(batch, proj.device) if proj.dtype == torch.bfloat16 else None
+    segments, segment = None, SCAN_SEGMENT
+    if proj.dtype == torch.bfloat16 and dim <= GLA_BLOCK_DIM:
+        tiles = -(-vdim // (64 if vdim <= 64 else 128))
+        segment = GLA_SEGMENT if heads * tiles * -(-n_tokens // GLA_SEGMENT) >= 512 else GLA_SEGMENT // 2
+        segments = step_segments(batch, proj.device, GLA_WALK, segment)
+    elif proj.dtype == torch.bfloat16:
+        segments = step_segments(batch, proj.device, segment, segment)
+    if segments is not None and segments.shape[0] > 65535:
+        segments = None  # (more segments than one launch counts: the portions are walked whole)
     seg_local = seg_decay = seg_start = None
-    if segments is not None:
-        seg_local, seg_decay, seg_start = (torch.empty((segments.shape[0], need), dtype=torch.float32, device=proj.device) for _ in range(3))
+    if segments is not None and max(batch.q_lens) > segment:
+        seg_local, seg_start = (torch.empty((segments.shape[0], need), dtype=torch.float32, device=proj.device) for _ in range(2))
+        seg_decay = torch.empty((segments.shape[0], heads * dim), dtype=torch.float32, device=proj.device)
     lib = _build.load("linear_attention")
     _check(
         lib,

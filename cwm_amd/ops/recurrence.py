@@ -17,8 +17,8 @@ from .sequence import step_segments
 MAX_TOKEN_MIXES = 8  # csrc/token_mix.hip: TMIX_MAX
 MAX_NORMED_ADDENDS = 4  # csrc/normed_sum.hip: NSUM_MAX
 MIN_GRU_WALK = 32  # tokens of the longest portion that a step still walks as a whole; longer ones go in segments
-MIN_GRU_SEGMENT = 32  # tokens of a segment at least
-MIN_GRU_SEGMENTS = 64  # and segments of a portion at most
+MIN_GRU_SEGMENT = 16  # tokens of a segment at least
+MIN_GRU_SEGMENTS = 128  # and segments of a portion at most
 
 
 def _base():

@@ -433,7 +433,7 @@ class HeadNormAttention(Mixer):
         s_j <- s_j - r1_h ln(1 + r2_h (i - j))                   `distance_bias`: two stored numbers a query head
         softmax over the keys j <= i that the mask leaves: the last `window` keys (own included), or, with `chunk`, the keys
             of the query's own block of `chunk` positions counted from the start of the sequence; neither: all.
-            With `unit_sink` its denominator is 1 + sum_j exp(s_j): a sink whose score is always 0
+            With `unit_sink` its denominator is 1 + sum_j exp(s_j), as if a sink of score 0 were stored for every head
         out = W_o ([sum_j p_j v_j of every head] * sigmoid(W_g x))   the gate where `gate`, element by element
 
     Keys and values are cached with one head size, the larger of qk_dim and v_dim rounded up to a multiple of 16 (zeros

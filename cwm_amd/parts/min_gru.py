@@ -1,4 +1,4 @@
-"""A gated recurrence whose gates read the current token only, with a per-request state."""
+"""A recurrence over single elements, gated without looking at its own state (minGRU), with a per-request state."""
 
 from __future__ import annotations
 

@@ -13,8 +13,8 @@ from .linear import LinearWeights
 
 
 class WKV(Mixer):
-    """With x' the previous token's x (zeros for the first token), five blends x + (x' - x) * mu_s are read by r, k, v
-    (heads x head_dim each), by the output gate and by the decay:
+    """Five blends m_s = x_t + (x_(t-1) - x_t) * mu_s of neighbouring tokens (x_(-1) = 0) feed r, k, v (heads x head_dim
+    each), the output gate and the decay:
         r = W_r m_r,  k = W_k m_k,  v = W_v m_v,  g = W_g m_g,  alpha = exp(-exp(W_w2 tanh(W_w1 m_w) + w_0))
         o_t = (S_(t-1) + diag(u) k_t v_t^T)^T r_t,      S_t = diag(alpha_t) S_(t-1) + k_t v_t^T       per head
     with S zero at a request's start; then out = W_o (o / rms(o per head) * weight * silu(g)).  The low rank of the decay is

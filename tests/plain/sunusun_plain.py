@@ -56,16 +56,16 @@ def query_temperature(positions: torch.Tensor, coef: float, every: float) -> tor
     return 1.0 + coef * torch.log(torch.floor((positions.to(F) + 1.0) / every) + 1.0)
 
 
-def distance_bias(n: int, r1: torch.Tensor, r2: torch.Tensor) -> torch.Tensor:
-    """[H, n, n]: what comes off the score of query i and key j <= i (zero above the diagonal, which nothing reads)."""
-    d = (torch.arange(n)[:, None] - torch.arange(n)[None, :]).clamp(min=0).to(F)
+def distance_bias(queries: torch.Tensor, keys: torch.Tensor, r1: torch.Tensor, r2: torch.Tensor) -> torch.Tensor:
+    """[H, queries, keys]: what comes off the score of the query at one position and the key at another (zero where the key
+    comes after the query, which nothing reads)."""
+    d = (queries[:, None] - keys[None, :]).clamp(min=0).to(F)
     return r1[:, None, None] * torch.log(1.0 + r2[:, None, None] * d[None])
 
 
-def softmax_with_one(scores: torch.Tensor) -> torch.Tensor:
-    """scores [H, T, T] (causal) -> exp(s) / (1 + sum exp(s)) over the keys up to the query's own."""
-    n = scores.shape[-1]
-    s = scores.masked_fill(~torch.tril(torch.ones(n, n, dtype=torch.bool))[None], float("-inf"))
+def softmax_with_one(scores: torch.Tensor, visible: torch.Tensor) -> torch.Tensor:
+    """scores [H, queries, keys] -> exp(s) / (1 + sum exp(s)) over the visible keys of each query."""
+    s = scores.masked_fill(~visible[None], float("-inf"))
     m = s.max(dim=-1, keepdim=True).values.clamp(min=0.0)
     e = torch.exp(s - m)
     return e / (torch.exp(-m) + e.sum(dim=-1, keepdim=True))
@@ -82,8 +82,9 @@ def attention(w: Dict[str, torch.Tensor], p: str, m: dict, h: torch.Tensor, eps:
     q = rd(q)
     per = heads // groups
     k, v = k.repeat_interleave(per, dim=1), v.repeat_interleave(per, dim=1)
-    scores = torch.einsum("ihd,jhd->hij", q, k) * m["scale"] - distance_bias(n, w[p + "r1"], w[p + "r2"])
-    out = torch.einsum("hij,jhd->ihd", rd(softmax_with_one(scores)), v).reshape(n, heads * vdim)
+    at = torch.arange(n)
+    scores = torch.einsum("ihd,jhd->hij", q, k) * m["scale"] - distance_bias(at, at, w[p + "r1"], w[p + "r2"])
+    out = torch.einsum("hij,jhd->ihd", rd(softmax_with_one(scores, at[None, :] <= at[:, None])), v).reshape(n, heads * vdim)
     return rd(out) @ w[p + "o"].T
 
 

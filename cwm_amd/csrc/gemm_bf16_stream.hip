@@ -23,6 +23,9 @@
 // steps of K per wavefront in registers (M <= 16, K up to 6144 without a split), and
 // four tiles of A with 4 steps of K per wavefront (M <= 64, K up to 2048 per split).
 //
+// Several inputs: the rows of W may belong to several A's of one size, `tiles_per_input` tiles of 16 rows each (the last
+// may have fewer): blocks are dealt out by input, so a block still holds one slice of one A.
+//
 // Replaces torch.nn.functional.linear at cwm/fastgen/forward.py:593-606,763,776-782,
 // 820 for decode batches.  Needs K % 8 == 0 and 16-byte aligned rows; any N; M <= 64.
 #include "common.h"
@@ -76,15 +79,25 @@ template <typename TC, bool ROPE, bool GLU, int MT, int ST_WAVES, int ST_HALF, b
 __global__ void __launch_bounds__(ST_WAVES * 64)
 gemm_stream_kernel(const bf16_t* __restrict__ A, long lda, const bf16_t* __restrict__ W, long ldw, TC* __restrict__ C,
                    long ldc, long split_stride, const void* __restrict__ bias, int bias_dtype, int M, int N, int K,
-                   int steps_per_wave, int n_tiles, int k_split, RopeKv rk) {
+                   int steps_per_wave, int n_tiles, int k_split, RopeKv rk, long input_stride, int tiles_per_input,
+                   int blocks_per_input) {
   __shared__ float red[2][ST_WAVES][MT * 256];
   const int lane = threadIdx.x & 63;
   const int wave = threadIdx.x >> 6;
   const int r = lane & 15;
   const int j = lane >> 4;
   const int ks = blockIdx.x % k_split;
-  const int tile_first = blockIdx.x / k_split;
-  const int tile_stride = gridDim.x / k_split;
+  int tile_first = blockIdx.x / k_split;
+  int tile_stride = gridDim.x / k_split;
+  int tile_end = n_tiles;
+  if (tiles_per_input > 0) {
+    const int final_input = (n_tiles - 1) / tiles_per_input;
+    const int input = min(tile_first / blocks_per_input, final_input);
+    tile_first += input * (tiles_per_input - blocks_per_input);
+    tile_stride = input < final_input ? blocks_per_input : tile_stride - final_input * blocks_per_input;
+    tile_end = min(n_tiles, (input + 1) * tiles_per_input);
+    A += (size_t)input * input_stride;
+  }
 
   // this wavefront's steps of 32 along K, and its slice of A in registers
   const int s0 = (ks * ST_WAVES + wave) * steps_per_wave;
@@ -106,11 +119,11 @@ gemm_stream_kernel(const bf16_t* __restrict__ A, long lda, const bf16_t* __restr
   auto load_half = [&](Frag8 (&buf)[ST_HALF], int tile, int half) {
     if (TILED) {
       // ldw: values of one tile (16 rows of all steps)
-      const u32x4* wtile = (const u32x4*)(W + (size_t)min(tile, n_tiles - 1) * ldw) + (size_t)s0 * 64 + lane;
+      const u32x4* wtile = (const u32x4*)(W + (size_t)min(tile, tile_end - 1) * ldw) + (size_t)s0 * 64 + lane;
 #pragma unroll
       for (int i = 0; i < ST_HALF; ++i) {
         const int step = half * ST_HALF + i;
-        const bool ok = tile < n_tiles && step < steps_per_wave && s0 + step < steps_total;
+        const bool ok = tile < tile_end && step < steps_per_wave && s0 + step < steps_total;
         buf[i].w = ok ? __builtin_nontemporal_load(wtile + (size_t)step * 64) : u32x4{0, 0, 0, 0};
       }
       return;
@@ -120,7 +133,7 @@ gemm_stream_kernel(const bf16_t* __restrict__ A, long lda, const bf16_t* __restr
     for (int i = 0; i < ST_HALF; ++i) {
       const int step = half * ST_HALF + i;
       const int k = koff + 32 * step;
-      const bool ok = tile < n_tiles && step < steps_per_wave && k + 8 <= K;
+      const bool ok = tile < tile_end && step < steps_per_wave && k + 8 <= K;
       buf[i].u = ok ? *(const uint4*)(wrow + k) : make_uint4(0, 0, 0, 0);
     }
   };
@@ -129,7 +142,7 @@ gemm_stream_kernel(const bf16_t* __restrict__ A, long lda, const bf16_t* __restr
   int tile = tile_first;
   load_half(wa, tile, 0);
   int parity = 0;
-  for (; tile < n_tiles; tile += tile_stride) {
+  for (; tile < tile_end; tile += tile_stride) {
     load_half(wb, tile, 1);
     float4v acc[MT];
 #pragma unroll
@@ -255,7 +268,10 @@ extern "C" int cwm_gemm_bf16_stream(const void* A, long lda, const void* W, long
                                     const int* rope_seq_of_token, const float* rope_inv_freq, void* rope_cache,
                                     const int* rope_block_table, int rope_table_width, int rope_page_size,
                                     int rope_num_pages, int rope_n_q_heads, int rope_n_kv_heads, int rope_head_dim,
-                                    int glu, int tiled, hipStream_t stream) {
+                                    int glu, int tiled, long input_stride, int tiles_per_input, int blocks_per_input,
+                                    hipStream_t stream) {
+  // tiles_per_input > 0: W's tiles belong to several inputs of M rows, input_stride elements apart, that many each;
+  // blocks_per_input blocks (times k_split) take each input's tiles, what is left of n_blocks the last one's
   // tiled != 0: W is the streaming copy (see the kernel; `cwm_gemm_bf16_stream_tiled_values` gives its size) and ldw
   // the values of one of its tiles
   // glu != 0: W holds gate and up rows in alternating groups of 8 and C [M, N / 2] receives
@@ -299,12 +315,19 @@ extern "C" int cwm_gemm_bf16_stream(const void* A, long lda, const void* W, long
   CWM_REQUIRE(n_blocks >= k_split && n_blocks % k_split == 0, "gemm_bf16_stream: %d blocks do not divide into %d splits",
               n_blocks, k_split);
   CWM_REQUIRE(n_blocks / k_split <= n_tiles, "gemm_bf16_stream: more blocks than tiles");
+  if (tiles_per_input > 0) {
+    const int final_input = (n_tiles - 1) / tiles_per_input, rest = n_blocks / k_split - final_input * blocks_per_input;
+    CWM_REQUIRE(!rope && !glu, "gemm_bf16_stream: the fused epilogues take one input");
+    CWM_REQUIRE(input_stride % 8 == 0 && blocks_per_input >= 1 && blocks_per_input <= tiles_per_input && rest >= 1 &&
+                    rest <= n_tiles - final_input * tiles_per_input,
+                "gemm_bf16_stream: %d blocks do not serve %d tiles of %d an input", n_blocks / k_split, n_tiles, tiles_per_input);
+  }
   dim3 grid(n_blocks);
   dim3 block(ST_WAVES * 64);
 #define CWM_LAUNCH_STREAM_AS(TC, ROPE, GLU, MT, WAVES, HALF, TILED)                                                            \
   hipLaunchKernelGGL((gemm_stream_kernel<TC, ROPE, GLU, MT, WAVES, HALF, TILED>), grid, block, 0, stream, (const bf16_t*)A, lda, \
                      (const bf16_t*)W, ldw, (TC*)C, ldc, split_stride, bias, bias_dtype, M, N, K, steps_per_wave,                 \
-                     n_tiles, k_split, rk)
+                     n_tiles, k_split, rk, input_stride, tiles_per_input, blocks_per_input)
 #define CWM_LAUNCH_STREAM(TC, ROPE, GLU, MT, WAVES, HALF)           \
   do {                                                              \
     if (tiled)                                                      \

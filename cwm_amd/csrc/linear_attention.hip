@@ -680,3 +680,142 @@ extern "C" int cwm_gated_linear_attention(const void* q, const void* k, const vo
   }
   return cwm_launch_status("gated_linear_attention (results)");
 }
+
+// ---- a decode step of the form with a bonus, from the projections' sums to the gated result -------------------------- //
+// One token a sequence; a block a (head, sequence).  sums: the product's float32 partial sums, a row [r | k | v | g | low],
+// heads * dim values of the first four and `rank` of the last.  The decay's logits are z = w2 tanh(low) + w0, its second
+// matrix (bfloat16) read beside the state; then the recurrence as in the walk (the state lies as the walk keeps it), the
+// norm of the head's result, its weight and the gate.  All sums float32.
+__device__ __forceinline__ float partial_sum(const float* p, int n_partials, long stride) {
+  if (n_partials == 1) return *p;
+  float total = 0.f;
+  for (int q = 0; q < n_partials; q += 4) {  // four in flight, added in their order; past the last: that one times zero
+    float x[4];
+#pragma unroll
+    for (int u = 0; u < 4; ++u) x[u] = p[(size_t)min(q + u, n_partials - 1) * stride];
+#pragma unroll
+    for (int u = 0; u < 4; ++u) total = fmaf(q + u < n_partials ? 1.0f : 0.0f, x[u], total);
+  }
+  return total;
+}
+
+__global__ void __launch_bounds__(GLA_THREADS)
+wkv_token_kernel(const float* __restrict__ sums, long ld, int n_partials, long partial_stride, const bf16_t* __restrict__ w2,
+                 int rank, const float* __restrict__ w0, const float* __restrict__ bonus, const float* __restrict__ weight,
+                 float eps, bf16_t* __restrict__ out, float* __restrict__ state, long state_ld, const int* __restrict__ slots,
+                 int n_slots, int heads, int dim, int split) {
+  __shared__ __attribute__((aligned(16))) float qs[GLA_MAX_DIM], ks[GLA_MAX_DIM], uk[GLA_MAX_DIM], as[GLA_MAX_DIM];
+  __shared__ float vs[GLA_MAX_DIM], gs[GLA_MAX_DIM], os[GLA_MAX_DIM];
+  extern __shared__ float low[];  // [rank]
+  const int h = blockIdx.x, t = blockIdx.y, tid = threadIdx.x;
+  const int cols = GLA_THREADS / split, rows = gla_rows(dim, split), dpad = split * rows, n_vt = (dim + cols - 1) / cols;
+  const int col = tid / split, part = tid % split;
+  const int inner = heads * dim;
+  const int slot = slots[t];
+  if (slot < 0 || slot >= n_slots) return;
+  float* st = state + (size_t)slot * state_ld + (size_t)h * n_vt * rows * GLA_THREADS + tid;
+  // the first tile's state and the thread's share of w2 are in flight while the projections are added up
+  float S[GLA_ROWS];
+#pragma unroll
+  for (int r = 0; r < GLA_ROWS; ++r) S[r] = r < rows ? st[(size_t)r * GLA_THREADS] : 0.f;
+  int lanes = 1;  // threads that share a channel's logit
+  while (lanes < 8 && 2 * lanes * dim <= GLA_THREADS) lanes *= 2;
+  const int share = rank / lanes, chan = tid / lanes, piece = tid - chan * lanes;
+  const bool vec = share * lanes == rank && share % 8 == 0 && share <= 32 && ((uintptr_t)w2 % 16) == 0;
+  uint4 w2r[4];
+#pragma unroll
+  for (int i = 0; i < 4; ++i)
+    w2r[i] = (vec && chan < dim && 8 * i < share) ? *(const uint4*)(w2 + (size_t)(h * dim + chan) * rank + piece * share + 8 * i) : make_uint4(0, 0, 0, 0);
+  const float* row = sums + (size_t)t * ld;
+  for (int d = tid; d < dpad; d += GLA_THREADS) {
+    const bool real = d < dim;
+    const int c = h * dim + d;
+    const float kk = real ? partial_sum(row + inner + c, n_partials, partial_stride) : 0.f;
+    qs[d] = real ? partial_sum(row + c, n_partials, partial_stride) : 0.f;
+    ks[d] = kk;
+    uk[d] = real ? kk * bonus[c] : 0.f;
+    as[d] = 0.f;
+    if (real) {
+      vs[d] = partial_sum(row + 2 * inner + c, n_partials, partial_stride);
+      gs[d] = partial_sum(row + 3 * inner + c, n_partials, partial_stride);
+    }
+  }
+  for (int j = tid; j < rank; j += GLA_THREADS) low[j] = tanhf(partial_sum(row + 4 * inner + j, n_partials, partial_stride));
+  __syncthreads();
+  for (int c = chan; c < dim; c += GLA_THREADS / lanes) {
+    float z = 0.f;
+    if (vec) {
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        if (8 * i < share) {
+          const uint4 w = c == chan ? w2r[i] : *(const uint4*)(w2 + (size_t)(h * dim + c) * rank + piece * share + 8 * i);
+          const uint32_t ws[4] = {w.x, w.y, w.z, w.w};
+          const float* l = low + piece * share + 8 * i;
+#pragma unroll
+          for (int x = 0; x < 4; ++x) {
+            z = fmaf(__uint_as_float(ws[x] << 16), l[2 * x], z);
+            z = fmaf(__uint_as_float(ws[x] & 0xffff0000u), l[2 * x + 1], z);
+          }
+        }
+      }
+    } else {
+      for (int j = piece; j < rank; j += lanes) z = fmaf(bf16_to_f32(w2[(size_t)(h * dim + c) * rank + j]), low[j], z);
+    }
+    for (int off = 1; off < lanes; off *= 2) z += __shfl_xor(z, off, CWM_WAVE);
+    if (piece == 0) as[c] = gla_decay<KIND_WKV>(z + w0[h * dim + c], 1.0f);
+  }
+  __syncthreads();
+  const int d0 = part * rows;
+  for (int vt = 0; vt < n_vt; ++vt) {
+    float* tile = st + (size_t)vt * rows * GLA_THREADS;
+    if (vt > 0) {
+#pragma unroll
+      for (int r = 0; r < GLA_ROWS; ++r) S[r] = r < rows ? tile[(size_t)r * GLA_THREADS] : 0.f;
+    }
+    const int e = vt * cols + col;
+    const float v = e < dim ? vs[e] : 0.f;
+    float o = 0.f;
+#pragma unroll
+    for (int r = 0; r < GLA_ROWS; r += 4) {
+      if (r < rows) {
+        const float4 q4 = *(const float4*)(qs + d0 + r), k4 = *(const float4*)(ks + d0 + r);
+        const float4 u4 = *(const float4*)(uk + d0 + r), a4 = *(const float4*)(as + d0 + r);
+        o = fmaf(fmaf(u4.x, v, S[r]), q4.x, o), o = fmaf(fmaf(u4.y, v, S[r + 1]), q4.y, o);
+        o = fmaf(fmaf(u4.z, v, S[r + 2]), q4.z, o), o = fmaf(fmaf(u4.w, v, S[r + 3]), q4.w, o);
+        tile[(size_t)r * GLA_THREADS] = fmaf(a4.x, S[r], k4.x * v);
+        tile[(size_t)(r + 1) * GLA_THREADS] = fmaf(a4.y, S[r + 1], k4.y * v);
+        tile[(size_t)(r + 2) * GLA_THREADS] = fmaf(a4.z, S[r + 2], k4.z * v);
+        tile[(size_t)(r + 3) * GLA_THREADS] = fmaf(a4.w, S[r + 3], k4.w * v);
+      }
+    }
+    for (int off = 1; off < split; off *= 2) o += __shfl_xor(o, off, CWM_WAVE);
+    if (part == 0 && e < dim) os[e] = o;
+  }
+  __syncthreads();
+  if (tid >= CWM_WAVE) return;
+  float sq = 0.f;
+  for (int e = tid; e < dim; e += CWM_WAVE) sq += os[e] * os[e];
+  const float rstd = 1.0f / sqrtf(wave_sum(sq) / (float)dim + eps);
+  for (int e = tid; e < dim; e += CWM_WAVE) {
+    const float g = gs[e];
+    out[(size_t)t * inner + h * dim + e] = f32_to_bf16(os[e] * rstd * weight[h * dim + e] * (g / (1.0f + expf(-g))));
+  }
+}
+
+// sums: float32 [n_partials][n_tokens][ld], partial_stride elements between partial sums.  w2: bfloat16 [heads * dim][rank];
+// w0, bonus, weight: float32 [heads * dim].  out: bfloat16 [n_tokens][heads * dim].  Token t belongs to sequence t.
+extern "C" int cwm_wkv_token(const float* sums, long ld, int n_partials, long partial_stride, const void* w2, int rank,
+                             const float* w0, const float* bonus, const float* weight, float eps, void* out, float* state,
+                             long state_ld, const int* slots, int n_slots, int n_tokens, int heads, int dim, hipStream_t stream) {
+  CWM_REQUIRE(n_tokens >= 0 && n_tokens <= 65535 && heads >= 1 && n_partials >= 1, "wkv_token: bad sizes");
+  CWM_REQUIRE(dim >= 1 && dim <= GLA_MAX_DIM, "wkv_token: heads of %d rows are outside 1..%d", dim, GLA_MAX_DIM);
+  CWM_REQUIRE(rank >= 1 && rank <= 4096, "wkv_token: a rank of %d is outside 1..4096", rank);
+  CWM_REQUIRE(ld >= 4L * heads * dim + rank && eps > 0.f, "wkv_token: rows of %ld values are too short", ld);
+  CWM_REQUIRE(sums && w2 && w0 && bonus && weight && out && state && slots, "wkv_token: arguments missing");
+  CWM_REQUIRE(state_ld >= cwm_gla_state_elems(heads, dim, dim), "wkv_token: a state row of %ld elements is too short", state_ld);
+  if (n_tokens == 0) return 0;
+  hipLaunchKernelGGL(wkv_token_kernel, dim3(heads, n_tokens), dim3(GLA_THREADS), sizeof(float) * rank, stream, sums, ld, n_partials,
+                     partial_stride, (const bf16_t*)w2, rank, w0, bonus, weight, eps, (bf16_t*)out, state, state_ld, slots, n_slots,
+                     heads, dim, gla_split(dim, dim));
+  return cwm_launch_status("wkv_token");
+}

@@ -377,6 +377,7 @@ def gemm_bf16_stream(
     rope: Optional[tuple] = None,
     glu: bool = False,
     streamed: Optional[torch.Tensor] = None,
+    rows_per_input: Optional[int] = None,
 ) -> torch.Tensor:
     """bfloat16 x [M <= 64, K] @ weight[N, K]^T with persistent blocks that keep x in
     registers and stream the weight once.  `streamed` is the matrix's streaming copy
@@ -388,8 +389,19 @@ def gemm_bf16_stream(
     head_dim) makes the epilogue rotate the q and k columns and write k and v into the
     paged cache (see `qkv_rope_write`).  `glu`: the weight's rows are gate and up rows in
     alternating groups of 8 and the result is silu(gate) * up, [M, N / 2] (see
-    `gate_up_silu`)."""
+    `gate_up_silu`).  `rows_per_input` (a multiple of 16): x is [G, M, K], and the weight's rows belong to its G inputs in
+    turn, that many each (the last one's may be fewer): column n of the result is row n of the weight times input
+    n // rows_per_input."""
     _need_gpu(x, weight, bias)
+    inputs = 1
+    if rows_per_input is not None:
+        inputs = x.shape[0]
+        if (
+            x.dim() != 3 or rows_per_input < 16 or rows_per_input % 16 != 0 or rope is not None or glu or x.stride(0) % 8 != 0
+            or not (inputs - 1) * rows_per_input < weight.shape[0] <= inputs * rows_per_input
+        ):
+            raise KernelError(f"{weight.shape[0]} rows of a weight do not belong to {inputs} inputs in runs of {rows_per_input} (a multiple of 16)")
+        input_stride, x = x.stride(0), x[0]
     if x.dtype != torch.bfloat16 or weight.dtype != torch.bfloat16:
         raise KernelError("the streaming product takes bfloat16 operands")
     if x.dim() != 2 or weight.dim() != 2 or x.shape[1] != weight.shape[1]:
@@ -415,6 +427,17 @@ def gemm_bf16_stream(
         while n_tiles * k_split < 2 * cus and k_split < 8 and steps >= 2 * k_split * waves:
             k_split *= 2  # too few tiles to fill the chip
     blocks = max(k_split, min(cus, n_tiles * k_split) // k_split * k_split)
+    input_args = (ctypes.c_long(0), ctypes.c_int(0), ctypes.c_int(0))
+    if inputs > 1:
+        per, most = rows_per_input // 16, max(1, cus // k_split)
+        tiles_a_block = -(-n_tiles // most)
+        while True:  # as few tiles a block as leave one round of blocks
+            a_input, rest = -(-per // tiles_a_block), -(-(n_tiles - (inputs - 1) * per) // tiles_a_block)
+            if (inputs - 1) * a_input + rest <= most or tiles_a_block >= per:
+                break
+            tiles_a_block += 1
+        blocks = k_split * ((inputs - 1) * a_input + rest)
+        input_args = (ctypes.c_long(input_stride), ctypes.c_int(per), ctypes.c_int(a_input))
     if k_split == 1:
         out = torch.empty((m, n // 2 if glu else n), dtype=out_dtype, device=x.device)
     else:
@@ -432,12 +455,27 @@ def gemm_bf16_stream(
             _ptr(out), ctypes.c_int(_code(out.dtype)), ctypes.c_long(out.shape[-1]), ctypes.c_long(m * n),
             _ptr(bias), ctypes.c_int(_code(bias.dtype) if bias is not None else F32),
             ctypes.c_int(m), ctypes.c_int(n), ctypes.c_int(k), ctypes.c_int(k_split), ctypes.c_int(blocks),
-            *_rope_args(rope), ctypes.c_int(int(glu)), ctypes.c_int(int(streamed is not None)), _stream(),
+            *_rope_args(rope), ctypes.c_int(int(glu)), ctypes.c_int(int(streamed is not None)), *input_args, _stream(),
         ),
     )
     if k_split > 1 and not partials_ok:
         return sum_partials(out, out_dtype)
     return out
+
+
+def linear_inputs_takes(x: torch.Tensor, weight: torch.Tensor, rows_per_input: int) -> bool:
+    """Whether the product of a few rows of several inputs is one launch (`linear_inputs`)."""
+    return (
+        x.is_cuda and x.dtype == torch.bfloat16 and weight.dtype == torch.bfloat16 and x.dim() == 3 and x.shape[1] <= STREAM_EPILOGUE_ROWS
+        and rows_per_input % 16 == 0 and x.is_contiguous() and x.shape[1] * x.shape[2] % 8 == 0 and _stream_takes(x[0], weight)
+    )
+
+
+def linear_inputs(x: torch.Tensor, weight: torch.Tensor, rows_per_input: int, streamed: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """Several inputs x [G, M <= 16, K] times the rows of one joined weight that belong to each (`rows_per_input` rows an
+    input, the last one's may be fewer), side by side: float32 partial sums [P, M, N] for the caller to add."""
+    out = gemm_bf16_stream(x, weight, None, torch.float32, partials_ok=True, streamed=streamed, rows_per_input=rows_per_input)
+    return out if out.dim() == 3 else out.unsqueeze(0)
 
 
 _NO_ROPE_ARGS = [ctypes.c_void_p(0)] * 5 + [ctypes.c_int(0)] * 6
@@ -1182,6 +1220,8 @@ __all__ = [
     "gemm_f32_stream",
     "gemm_bf16",
     "gemm_bf16_stream",
+    "linear_inputs",
+    "linear_inputs_takes",
     "sum_partials",
     "linear",
     "rope_kv_write",
@@ -1260,7 +1300,7 @@ from .streams import (  # noqa: E402
 )
 from .mixing import (  # noqa: E402
     MAX_GLA_DIM, MAX_SHORT_CONV_TAPS, MAX_SIDE_ADDENDS, MAX_SIDE_DIM, MAX_TALK_HEADS, gated_act_rows, gated_linear_attention, gla_state_elems,
-    gla_state_unpack, short_conv, talking_attention, token_side, wkv,
+    gla_state_unpack, short_conv, talking_attention, token_side, wkv, wkv_token,
 )
 from .recurrence import (  # noqa: E402
     MAX_NORMED_ADDENDS, MAX_TOKEN_MIXES, NormedSum, add_normed_rmsnorm, embedding_sinusoid, min_gru, token_mixes,

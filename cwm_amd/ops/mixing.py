@@ -11,6 +11,7 @@ from typing import Any, Optional, Sequence, Tuple
 import torch
 
 from . import build as _build
+from .sequence import SCAN_SEGMENT, step_segments
 
 MAX_TALK_HEADS = 64  # csrc/attention_talk.hip: TALK_MAX_HEADS
 TALK_SPLIT = 128  # csrc/attention_talk.hip: columns of a block's range of the score table
@@ -161,7 +162,7 @@ GLA_ROWS = 32  # and the rows of a column of the state that one of them holds at
 
 
 GLA_BLOCK_DIM = 128  # rows of a head that the kernel on the matrix cores takes at most
-GLA_WALK = 16  # tokens of the longest portion that a step still walks one by one
+WKV_WALK = 16  # tokens of the longest portion that `wkv` still walks one by one
 GLA_SEGMENT = 128  # tokens of a segment on the matrix cores; half of it where that gives the chip too few blocks
 
 
@@ -208,7 +209,7 @@ def gated_linear_attention(
     float32 [vdim]; `state` float32 [slots, >= gla_state_elems], read and written at the sequences' slots.  Queries are
     multiplied by `q_scale` (default dim ** -0.5).  Returns [T, heads * vdim] in proj's type: every head's result over
     its root mean square, times weight, times silu(gate).  A step's portions are walked token by token, which gives the
-    same bits however a sequence is cut; in bfloat16 a step with a portion of more than `GLA_WALK` tokens takes its
+    same bits however a sequence is cut; in bfloat16 a step with a portion of more than `SCAN_SEGMENT` tokens takes its
     portions in blocks of 16 tokens on the matrix cores (float32 operands), long ones in segments side by side with the
     state carried across them, which differs from the walk by float32 rounding."""
     KernelError = _base()[0]
@@ -219,7 +220,9 @@ def gated_linear_attention(
         raise KernelError(f"the weight must be a contiguous float32 [{vdim}]")
     qk, vv = heads * dim, heads * vdim
     parts = torch.split(proj[:, :width], (qk, qk, vv, vv), dim=1)
-    return _linear_attention(parts, None, decay_logits, weight, 0, state, batch, heads, dim, vdim, tau, eps, dim ** -0.5 if q_scale is None else q_scale)
+    return _linear_attention(
+        parts, None, decay_logits, weight, 0, state, batch, heads, dim, vdim, tau, eps, dim ** -0.5 if q_scale is None else q_scale, SCAN_SEGMENT,
+    )
 
 
 def wkv(
@@ -231,21 +234,62 @@ def wkv(
     equally far in all four); `decay_logits` float32 [T, heads * dim]: a key channel decays by exp(-exp(logit)); `bonus`
     float32 [heads * dim]; `weight` float32 [heads * vdim]; `state` float32 [slots, >= gla_state_elems], read and written
     at the sequences' slots.  Returns [T, heads * vdim] in r's type: every head's result over its root mean square,
-    times weight, times silu(gate).  Portions are walked or cut into segments as in `gated_linear_attention`."""
+    times weight, times silu(gate).  Portions are walked or go in blocks and segments as in `gated_linear_attention`, in
+    blocks from `WKV_WALK` tokens on."""
     KernelError, _check, _code, _i32, _need_gpu, _ptr, _stream = _base()
     _need_gpu(bonus)
     if bonus.dtype != torch.float32 or bonus.numel() != heads * dim or not bonus.is_contiguous():
         raise KernelError(f"the bonus must be a contiguous float32 tensor of {heads * dim} values")
     if weight.shape != (heads * vdim,):
         raise KernelError(f"the weight must be a contiguous float32 [{heads * vdim}]")
-    return _linear_attention((r, k, v, gate), bonus, decay_logits, weight, vdim, state, batch, heads, dim, vdim, 1.0, eps, 1.0)
+    return _linear_attention((r, k, v, gate), bonus, decay_logits, weight, vdim, state, batch, heads, dim, vdim, 1.0, eps, 1.0, WKV_WALK)
+
+
+def wkv_token(
+    sums: torch.Tensor, w2: torch.Tensor, w0: torch.Tensor, bonus: torch.Tensor, weight: torch.Tensor, state: torch.Tensor, batch: Any,
+    heads: int, dim: int, eps: float, out_dtype: torch.dtype,
+) -> torch.Tensor:
+    """`wkv` for a step of one token a sequence, from the projections' float32 partial sums [P, T, 4 * heads * dim + rank]
+    (r, k, v, the output gate, and the low rank of the decay), which are added up first: the decay's logits are
+    w2 tanh(low) + w0 with `w2` [heads * dim, rank] in bfloat16 and `w0` float32.  Returns [T, heads * dim] of
+    `out_dtype` (bfloat16)."""
+    KernelError, _check, _code, _i32, _need_gpu, _ptr, _stream = _base()
+    _need_gpu(sums, w2, w0, bonus, weight, state)
+    inner, rank = heads * dim, w2.shape[1]
+    if sums.dtype != torch.float32 or sums.dim() != 3 or not sums.is_contiguous() or tuple(sums.shape[1:]) != (batch.n_tokens, 4 * inner + rank):
+        raise KernelError(f"the projections' sums {tuple(sums.shape)} must be contiguous float32 [P, {batch.n_tokens}, {4 * inner + rank}]")
+    if batch.n_tokens != batch.n_seqs or max(batch.q_lens) != 1:
+        raise KernelError("one token a sequence is needed")
+    if w2.dtype != torch.bfloat16 or w2.shape[0] != inner or not w2.is_contiguous() or out_dtype != torch.bfloat16:
+        raise KernelError(f"the decay's second matrix must be a contiguous bfloat16 [{inner}, rank], the results bfloat16")
+    for what, t in (("the decay's bias", w0), ("the bonus", bonus), ("the weight", weight)):
+        if t.dtype != torch.float32 or t.numel() != inner or not t.is_contiguous():
+            raise KernelError(f"{what} must be a contiguous float32 tensor of {inner} values")
+    if dim > MAX_GLA_DIM:
+        raise KernelError(f"heads of {dim} rows: the kernel takes up to {MAX_GLA_DIM}")
+    need = gla_state_elems(heads, dim, dim)
+    if state.dtype != torch.float32 or state.dim() != 2 or state.shape[1] < need or not state.is_contiguous():
+        raise KernelError(f"the state must be a contiguous float32 [slots, >= {need}] tensor")
+    n_partials, n_tokens, ld = sums.shape
+    out = torch.empty((n_tokens, inner), dtype=out_dtype, device=sums.device)
+    lib = _build.load("linear_attention")
+    _check(
+        lib,
+        lib.cwm_wkv_token(
+            _ptr(sums), ctypes.c_long(ld), ctypes.c_int(n_partials), ctypes.c_long(n_tokens * ld), _ptr(w2), ctypes.c_int(rank), _ptr(w0), _ptr(bonus),
+            _ptr(weight), ctypes.c_float(eps), _ptr(out), _ptr(state), ctypes.c_long(state.shape[1]), _ptr(batch.state_slots),
+            ctypes.c_int(state.shape[0]), ctypes.c_int(n_tokens), ctypes.c_int(heads), ctypes.c_int(dim), _stream(),
+        ),
+    )
+    return out
 
 
 def _linear_attention(
     parts: Sequence[torch.Tensor], bonus: Optional[torch.Tensor], decay_logits: torch.Tensor, weight: torch.Tensor, weight_stride: int,
-    state: torch.Tensor, batch: Any, heads: int, dim: int, vdim: int, tau: float, eps: float, q_scale: float,
+    state: torch.Tensor, batch: Any, heads: int, dim: int, vdim: int, tau: float, eps: float, q_scale: float, walk: int,
 ) -> torch.Tensor:
-    """The launch that both forms share: `parts` are queries, keys, values and the output gate's projection."""
+    """The launch that both forms share: `parts` are queries, keys, values and the output gate's projection; a bfloat16
+    step whose portions all have up to `walk` tokens is walked."""
     KernelError, _check, _code, _i32, _need_gpu, _ptr, _stream = _base()
     proj = parts[0]
     _need_gpu(*parts, decay_logits, weight, state)
@@ -266,13 +310,11 @@ def _linear_attention(
     out = torch.empty((n_tokens, heads * vdim), dtype=proj.dtype, device=proj.device)
     # portions in bfloat16 go in blocks of tokens on the matrix cores, long ones in segments side by side (float32 keeps to
     # the walk, whose bits no cut changes)
-    from .sequence import SCAN_SEGMENT, step_segments
-
     segments, segment = None, SCAN_SEGMENT
     if proj.dtype == torch.bfloat16 and dim <= GLA_BLOCK_DIM:
         tiles = -(-vdim // (64 if vdim <= 64 else 128))
         segment = GLA_SEGMENT if heads * tiles * -(-n_tokens // GLA_SEGMENT) >= 512 else GLA_SEGMENT // 2
-        segments = step_segments(batch, proj.device, GLA_WALK, segment)
+        segments = step_segments(batch, proj.device, walk, segment)
     elif proj.dtype == torch.bfloat16:
         segments = step_segments(batch, proj.device, segment, segment)
     if segments is not None and segments.shape[0] > 65535:

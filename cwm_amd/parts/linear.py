@@ -49,6 +49,14 @@ class LinearWeights:
             bias = torch.stack([c.reshape(-1, group) for c in columns], dim=1).reshape(-1) if columns else None
         return cls(weight, bias, stream_copy)
 
+    def rows(self, start: int, stop: int) -> "LinearWeights":
+        """The rows start .. stop - 1 of a joined matrix as a matrix of their own that shares its memory (its streaming
+        copy only where both ends fall on a tile of 16 rows or the matrix's end)."""
+        part = LinearWeights(self.weight[start:stop], self.bias[start:stop] if self.bias is not None else None)
+        if self.streamed is not None and start % 16 == 0 and (stop % 16 == 0 or stop == self.weight.shape[0]):
+            part.streamed = self.streamed[start // 16 : -(-stop // 16)]
+        return part
+
     def __call__(self, x: torch.Tensor, out_dtype: Optional[torch.dtype] = None, partials_ok: bool = False) -> torch.Tensor:
         """With `partials_ok` the result may be float32 partial sums [P, M, N] (a
         product whose K was split) for a consumer that adds them, as the norms do."""

@@ -61,8 +61,10 @@ class WKV(Mixer):
         if tensors[n["w1"]].shape[0] != tensors[n["w2"]].shape[1]:
             raise ValueError(f"the decay's two projections do not meet: {tuple(tensors[n['w1']].shape)} and {tuple(tensors[n['w2']].shape)}")
         self.mu = torch.stack([tensors[n[f"mu_{s}"]].float() for s in "rkvgw"]).contiguous()
-        self.proj = [LinearWeights(tensors[n[s]], stream_copy=runtime.stream_copies) for s in "rkvg"]
-        self.decay_down = LinearWeights(tensors[n["w1"]], stream_copy=runtime.stream_copies)
+        # one matrix whose rows meet five inputs: a decode step's product; the others take its rows apart
+        self.joined = LinearWeights.joined([tensors[n[s]] for s in ("r", "k", "v", "g", "w1")], [None] * 5, stream_copy=runtime.stream_copies)
+        self.proj = [self.joined.rows(i * self.inner, (i + 1) * self.inner) for i in range(4)]
+        self.decay_down = self.joined.rows(4 * self.inner, self.joined.weight.shape[0])
         self.decay_up = LinearWeights(tensors[n["w2"]], tensors[n["w0"]].float())
         self.bonus = tensors[n["u"]].float().reshape(-1).contiguous()
         self.weight = tensors[n["norm"]].float().contiguous()
@@ -72,6 +74,13 @@ class WKV(Mixer):
         if not write_cache:
             raise ValueError("this mixer cannot read another layer's state")
         mixes = ops.token_mixes(x, self.mu, cache.state, self.matrix_elems, batch)
+        if max(batch.q_lens) == 1 and self.decay_down.weight.shape[0] <= self.inner and ops.linear_inputs_takes(mixes, self.joined.weight, self.inner):
+            # a decode step: one product for the five inputs, one kernel from its sums to the gated result
+            sums = ops.linear_inputs(mixes, self.joined.weight, self.inner, streamed=self.joined.streamed)
+            y = ops.wkv_token(
+                sums, self.decay_up.weight, self.decay_up.bias, self.bonus, self.weight, cache.state, batch, self.heads, self.head_dim, self.eps, x.dtype,
+            )
+            return self.w_out(y, partials_ok=True)
         r, k, v, g = (weights(mix) for weights, mix in zip(self.proj, mixes))
         low = ops.act_rows(self.decay_down(mixes[4], out_dtype=torch.float32, partials_ok=True), "tanh", torch.float32)
         logits = ops.gemm_f32(low, self.decay_up.weight, self.decay_up.bias, torch.float32)

@@ -330,6 +330,41 @@ def test_linear_attention_with_slow_with_fast_and_with_total_decays(dtype, shift
         assert torch.isfinite(state).all()
 
 
+@pytest.mark.parametrize("heads,dim,rank,width,batch", [(2, 16, 8, 64, 3), (4, 64, 64, 256, 8), (3, 48, 5, 200, 16), (1, 128, 32, 128, 1), (2, 176, 40, 512, 5), (5, 80, 100, 2048, 8)])
+def test_a_decode_step_in_two_kernels(heads, dim, rank, width, batch):
+    """The product of five inputs with one joined matrix against five products, with and without the matrix's streaming
+    copy; then the kernel from its sums to the gated result against the plain recurrence, over several steps, with
+    states in slots of any order."""
+    from cwm_amd import ops
+
+    inner, steps, slots = heads * dim, 4, list(range(batch))[::-1]
+    w = rnd((4 * inner + rank, width), 1, width ** -0.5).bfloat16()
+    w2, w0 = rnd((inner, rank), 2, rank ** -0.5).bfloat16(), rnd((inner,), 3, 2.0) - 1.0
+    bonus, weight = rnd((inner,), 4), rnd((inner,), 5).abs() + 0.5
+    state = torch.zeros((batch + 1, ops.gla_state_elems(heads, dim, dim) + width), dtype=torch.float32, device=DEV)
+    b = step_batch([7] * batch, [1] * batch, slots)
+    rows, got = [], []
+    for i in range(steps):
+        x = rnd((5, batch, width), 10 + i).bfloat16()
+        assert ops.linear_inputs_takes(x.to(DEV), w.to(DEV), inner)
+        sums = ops.linear_inputs(x.to(DEV), w.to(DEV), inner)
+        ends = [0, inner, 2 * inner, 3 * inner, 4 * inner, 4 * inner + rank]
+        want = torch.cat([x[j].double() @ w[ends[j] : ends[j + 1]].double().T for j in range(5)], dim=1)
+        torch.testing.assert_close(sums.sum(0).cpu().double(), want, rtol=1e-4, atol=1e-4)
+        streamed = ops.linear_inputs(x.to(DEV), w.to(DEV), inner, streamed=ops.stream_layout(w.to(DEV)))
+        torch.testing.assert_close(streamed, sums, rtol=1e-5, atol=1e-5)
+        got.append(ops.wkv_token(sums, w2.to(DEV), w0.to(DEV), bonus.to(DEV), weight.to(DEV), state, b, heads, dim, 1e-5, torch.bfloat16).cpu())
+        rows.append(want)
+    rows = torch.stack(rows)  # [steps, batch, 4 inner + rank]
+    for s in range(batch):
+        r, k, v, g = (rows[:, s, j * inner : (j + 1) * inner].reshape(steps, heads, dim) for j in range(4))
+        decay = torch.exp(-torch.exp(torch.tanh(rows[:, s, 4 * inner :]) @ w2.double().T + w0.double())).reshape(steps, heads, dim)
+        o = sp.wkv_scan(r, k, v, decay, bonus.double().reshape(heads, dim))
+        want = sp.unit_rms(o, 1e-5).reshape(steps, -1) * weight.double() * sp.silu(g).reshape(steps, -1)
+        torch.testing.assert_close(torch.stack([y[s] for y in got]).double(), want, rtol=1e-2, atol=2e-3)
+    assert torch.count_nonzero(state[batch]) == 0, "a slot that no sequence of the steps names was written"
+
+
 # ---- results that are normalised first, positions, activations -------------------------------------------------------- #
 @pytest.mark.parametrize("dtype", DTYPES)
 @pytest.mark.parametrize("dim,addends", [(40, 2), (192, 1), (1024, 2), (2048, 2), (4096, 2), (7, 2), (100, 3), (9000, 2)])

@@ -726,6 +726,14 @@ wkv_token_kernel(const float* __restrict__ sums, long ld, int n_partials, long p
 #pragma unroll
   for (int i = 0; i < 4; ++i)
     w2r[i] = (vec && chan < dim && 8 * i < share) ? *(const uint4*)(w2 + (size_t)(h * dim + chan) * rank + piece * share + 8 * i) : make_uint4(0, 0, 0, 0);
+  // and so are what the later stages read of the weights: no stage then waits for memory of its own
+  const float w0r = chan < dim ? w0[h * dim + chan] : 0.f;
+  float wr[GLA_MAX_DIM / CWM_WAVE];
+#pragma unroll
+  for (int i = 0; i < GLA_MAX_DIM / CWM_WAVE; ++i) {
+    const int e = tid + CWM_WAVE * i;
+    wr[i] = (tid < CWM_WAVE && e < dim) ? weight[h * dim + e] : 0.f;
+  }
   const float* row = sums + (size_t)t * ld;
   for (int d = tid; d < dpad; d += GLA_THREADS) {
     const bool real = d < dim;
@@ -762,7 +770,7 @@ wkv_token_kernel(const float* __restrict__ sums, long ld, int n_partials, long p
       for (int j = piece; j < rank; j += lanes) z = fmaf(bf16_to_f32(w2[(size_t)(h * dim + c) * rank + j]), low[j], z);
     }
     for (int off = 1; off < lanes; off *= 2) z += __shfl_xor(z, off, CWM_WAVE);
-    if (piece == 0) as[c] = gla_decay<KIND_WKV>(z + w0[h * dim + c], 1.0f);
+    if (piece == 0) as[c] = gla_decay<KIND_WKV>(z + (c == chan ? w0r : w0[h * dim + c]), 1.0f);
   }
   __syncthreads();
   const int d0 = part * rows;
@@ -796,9 +804,13 @@ wkv_token_kernel(const float* __restrict__ sums, long ld, int n_partials, long p
   float sq = 0.f;
   for (int e = tid; e < dim; e += CWM_WAVE) sq += os[e] * os[e];
   const float rstd = 1.0f / sqrtf(wave_sum(sq) / (float)dim + eps);
-  for (int e = tid; e < dim; e += CWM_WAVE) {
-    const float g = gs[e];
-    out[(size_t)t * inner + h * dim + e] = f32_to_bf16(os[e] * rstd * weight[h * dim + e] * (g / (1.0f + expf(-g))));
+#pragma unroll
+  for (int i = 0; i < GLA_MAX_DIM / CWM_WAVE; ++i) {
+    const int e = tid + CWM_WAVE * i;
+    if (e < dim) {
+      const float g = gs[e];
+      out[(size_t)t * inner + h * dim + e] = f32_to_bf16(os[e] * rstd * wr[i] * (g / (1.0f + expf(-g))));
+    }
   }
 }
 

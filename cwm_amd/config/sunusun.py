@@ -2,8 +2,8 @@
 
 config.json names the vocabulary, the width, one eps for every norm, a factor on the logits and a list of layers.  Every
 layer names its mixer (`type`: "parallel" or "wkv"), the mixer's sizes (`mixer`) and its feed-forward (`mlp`, null for
-none).  A layer with `weights_of` has no tensors of its own: it uses another layer's, and the rest of its entry repeats
-that layer's.  Strict as every configuration: an unknown key is an error that names it.
+none).  `weights_of` makes a layer run on the tensors of another one, whose mixer and feed-forward it must repeat; caches
+and states are not shared.  Strict as every configuration: an unknown key is an error that names it.
 """
 
 from __future__ import annotations

@@ -4,7 +4,7 @@
 //   S_t = (1 - z_t) S_(t-1) + z_t c_t                     sigmoid(u) for u < 0
 //   out_t = S_t * silu(y_t)                               y: a third projection
 //
-// S is float32, `width` values a sequence, carried from token to token in the sequence's slot.  z and 1 - z are both
+// S is float32, `width` values in the sequence's slot from one step to the next.  z and 1 - z are both
 // formed from exp(-|.|), so neither loses digits where the gate is nearly shut or nearly open.
 //
 // `min_gru_walk_kernel`: a thread owns CH neighbouring elements and walks tokens one by one.

@@ -93,6 +93,23 @@ __device__ __forceinline__ float tanh_of(float x) {
 #define BIAS_TILE(SLOPE_RAW, RATE, DIST)
 #endif
 
+// A library built with -DKEPT_KEYS=1 also lets every query read the sequence's first `keep_first` keys, however far back
+// they lie: key j is read if j <= p and (p - j <= window_left or j < keep_first).  The item that starts at the first key of
+// its rows' windows takes the kept keys that lie before it as tiles of their own, ahead of its range; kept keys inside the
+// range are left in by its masks.
+#ifdef KEPT_KEYS
+#define KEPT_PARAMS , int keep_first
+#define KEPT_RANGE(FIRST_ROW)                                                                                \
+    const int item_lo = window_left >= 0 ? max(0, n_old + (FIRST_ROW) / group - window_left) : 0;            \
+    const int kept_end = key_begin == item_lo ? min(keep_first, key_begin) : 0;                              \
+    const int kept_tiles = (kept_end + 31) >> 5;
+#define IS_KEPT(key) ((key) < keep_first)
+#else
+#define KEPT_PARAMS
+#define KEPT_RANGE(FIRST_ROW) constexpr int kept_end = 0, kept_tiles = 0;
+#define IS_KEPT(key) false
+#endif
+
 #define MAXIMUM(a, b) __builtin_elementwise_maximum(a, b)
 #define SOFTMAX_TILE(VOTE, ST0, ST1, NEED_MASK, OK_EXPR, M_RUN, NEG_MC, L_RUN, ALPHA, PF, SLOPE_RAW, RATE, DIST) \
   {                                                                                                          \
@@ -179,7 +196,7 @@ attention_mfma_kernel(const bf16_t* __restrict__ q, long q_stride, bf16_t* __res
                       const int* __restrict__ cu_q, const int* __restrict__ kv_len, const int* __restrict__ work,
                       int n_work, float* __restrict__ partial, int n_q_heads, int n_kv_heads, int page_size,
                       int page_shift, int num_pages, int window_left, int chunk, float scale_log2e, float cap_raw,
-                      const float* __restrict__ sink BIAS_PARAMS) {
+                      const float* __restrict__ sink, const float* __restrict__ out_scale BIAS_PARAMS KEPT_PARAMS) {
   const int lane = threadIdx.x & 63;
   const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
   const int id = blockIdx.x;  // (item, key/value head): the same for the whole block
@@ -199,6 +216,7 @@ attention_mfma_kernel(const bf16_t* __restrict__ q, long q_stride, bf16_t* __res
   const int n_new = cu_q[b + 1] - q0;
   const int n_old = kv_len[b] - n_new;
   const int n_rows = n_new * group;
+  KEPT_RANGE(row0)
 
   const int n = lane & 15;  // row of the tile (B operands, results), key or dim of the tile (A operands)
   const int j = lane >> 4;
@@ -259,7 +277,8 @@ attention_mfma_kernel(const bf16_t* __restrict__ q, long q_stride, bf16_t* __res
   const bf16_t* vbase = cache + plane + (size_t)g * page_size * HEAD_DIM;
   // a key that some row reads must have a page: if its table entry is -1 or out of range the rows'
   // results are made NaN (the loads below then read page 0, so nothing faults)
-  const bool page_missing = span_lacks_page(table, table_width, num_pages, page_size, page_shift, lo_any, hi_any, lane);
+  const bool page_missing = span_lacks_page(table, table_width, num_pages, page_size, page_shift, lo_any, hi_any, lane) ||
+                            (kept_end > 0 && span_lacks_page(table, table_width, num_pages, page_size, page_shift, 0, kept_end - 1, lane));
 
   // page of a key; keys outside [0, key_end) and slots without a page read page 0 and are masked
   auto page_of = [&](int key, int& slot_in_page) -> int {
@@ -322,17 +341,18 @@ attention_mfma_kernel(const bf16_t* __restrict__ q, long q_stride, bf16_t* __res
     }
   };
   // masks, softmax and the value product of the tile from `kt` on
-  auto finish = [&](float4v (&st)[2], Frag8 (&VF)[D_TILES], int kt) {
-    const bool need_mask = kt < lo_all || kt + 31 > hi_all;
+  auto finish = [&](float4v (&st)[2], Frag8 (&VF)[D_TILES], int kt, bool kept) {
+    const bool need_mask = kept || kt < lo_all || kt + 31 > hi_all;
+    const int lo_used = kept ? 0 : lo_any, hi_used = kept ? kept_end - 1 : hi_any;
     // ---- values outside the span that any row reads are zeroed ---------------------------------- //
     const int vkey = kt + 8 * j;
-    const bool boundary = (kt < lo_any) || (kt + 31 > hi_any);
+    const bool boundary = (kt < lo_used) || (kt + 31 > hi_used);
     if (boundary) {
       uint32_t keep[4] = {0xffffffffu, 0xffffffffu, 0xffffffffu, 0xffffffffu};
 #pragma unroll
       for (int e = 0; e < 8; ++e) {
         const int key = vkey + e;
-        if (key < lo_any || key > hi_any) keep[e >> 1] &= (e & 1) ? 0x0000ffffu : 0xffff0000u;
+        if (key < lo_used || key > hi_used) keep[e >> 1] &= (e & 1) ? 0x0000ffffu : 0xffff0000u;
       }
 #pragma unroll
       for (int dt = 0; dt < D_TILES; ++dt) {
@@ -345,7 +365,8 @@ attention_mfma_kernel(const bf16_t* __restrict__ q, long q_stride, bf16_t* __res
     // ---- mask, running maximum, probabilities --------------------------------------------------- //
     float alpha;
     Frag8 pf;
-    SOFTMAX_TILE(false, st[0], st[1], need_mask, row_valid && key >= row_start && key <= row_end && key >= key_begin && key < key_end,
+    SOFTMAX_TILE(false, st[0], st[1], need_mask,
+                 row_valid && key <= row_end && (kept ? key < kept_end : (key >= row_start || IS_KEPT(key)) && key >= key_begin && key < key_end),
                  m_run, neg_mc_run, l_run, alpha, pf, slope_raw, rate, row_end - (kt + 8 * j))
     if (__any(alpha != 1.0f)) {  // seldom after the first tiles
       asm volatile("" ::: "memory");  // keeps this a branch: unconditional, it is 4 multiplications per output tile
@@ -357,24 +378,27 @@ attention_mfma_kernel(const bf16_t* __restrict__ q, long q_stride, bf16_t* __res
     for (int dt = 0; dt < D_TILES; ++dt) acc[dt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(VF[dt].v, pf.v, acc[dt], 0, 0, 0);
   };
 
-  // wavefront w starts at the item's tile w and goes on in steps of TEAM tiles
-  const int kt_step = 32 * TEAM;
-  const int kt_first = (key_begin & ~31) + 32 * wave;
+  // wavefront w starts at the item's tile w and goes on in steps of TEAM tiles (kept keys' tiles come first)
+  const int range_tile0 = key_begin >> 5;
+  const int n_tiles = kept_tiles + ((key_end + 31) >> 5) - range_tile0;
+  auto first_key = [&](int tile) { return 32 * (tile < kept_tiles ? tile : range_tile0 + tile - kept_tiles); };
   Frag8 kf[2][K32_STEPS], vf[D_TILES];
-  if (kt_first < key_end) {
-    issue_keys(kf, kt_first);
-    int kt = kt_first;
-    for (; kt + kt_step < key_end; kt += kt_step) {
+  if (wave < n_tiles) {
+    issue_keys(kf, first_key(wave));
+    int tile = wave;
+    for (; tile + TEAM < n_tiles; tile += TEAM) {
       float4v st[2];
+      const int kt = first_key(tile);
       issue_values(vf, kt);
       scores(kf, st);
-      issue_keys(kf, kt + kt_step);  // the next tile's keys: in flight during the softmax and the value product
-      finish(st, vf, kt);
+      issue_keys(kf, first_key(tile + TEAM));  // the next tile's keys: in flight during the softmax and the value product
+      finish(st, vf, kt, tile < kept_tiles);
     }
     float4v st[2];
+    const int kt = first_key(tile);
     issue_values(vf, kt);
     scores(kf, st);
-    finish(st, vf, kt);
+    finish(st, vf, kt, tile < kept_tiles);
   }
 
   // ---- the team's wavefronts combine: the largest reference maximum, every wavefront's sums and output
@@ -407,7 +431,8 @@ attention_mfma_kernel(const bf16_t* __restrict__ q, long q_stride, bf16_t* __res
   // a sink: one more term of the denominator, exp(sink) of the query head (not scaled, no key, no value).  It
   // counts once a row: a block that leaves a partial result leaves it to the merge kernel
   if (sink && slot < 0) l_all += __builtin_amdgcn_exp2f(sink[hq] * 1.4426950408889634f - m_all * scale_log2e);
-  const float inv = page_missing ? not_a_number() : 1.0f / l_all;
+  float inv = page_missing ? not_a_number() : 1.0f / l_all;
+  if (out_scale && slot < 0) inv *= out_scale[(size_t)(q0 + ti) * n_q_heads + hq];
   bf16_t* orow = out + (size_t)(q0 + ti) * out_stride + (size_t)hq * HEAD_DIM;
   float* prow = slot < 0 ? nullptr : partial + (((size_t)slot * n_kv_heads + g) * 16 + n) * PARTIAL_STRIDE;
   for (int dt = wave; dt < D_TILES; dt += TEAM) {
@@ -488,7 +513,7 @@ attention_lds_kernel(const bf16_t* __restrict__ q, long q_stride, bf16_t* __rest
                      const int* __restrict__ cu_q, const int* __restrict__ kv_len, const int* __restrict__ work,
                      float* __restrict__ partial, int n_kv_heads_grid, int n_q_heads, int n_kv_heads, int page_size,
                      int page_shift, int num_pages, int window_left, int chunk, float scale_log2e, float cap_raw,
-                      const float* __restrict__ sink BIAS_PARAMS) {
+                      const float* __restrict__ sink, const float* __restrict__ out_scale BIAS_PARAMS KEPT_PARAMS) {
   constexpr bool FAST = MODE != LDS_PLAIN;
   constexpr int DMA_AHEAD = DMA_BUFFERS - 1;
   __shared__ __attribute__((aligned(16))) bf16_t lds_k[MODE == LDS_DMA ? 1 : 2][MODE == LDS_DMA ? 8 : 32 * LDS_K_STRIDE];
@@ -513,6 +538,7 @@ attention_lds_kernel(const bf16_t* __restrict__ q, long q_stride, bf16_t* __rest
   const int n_new = cu_q[b + 1] - q0;
   const int n_old = kv_len[b] - n_new;
   const int n_rows = n_new * group;
+  KEPT_RANGE(w[1])
 
   const int n = lane & 15;
   const int j = lane >> 4;
@@ -578,7 +604,10 @@ attention_lds_kernel(const bf16_t* __restrict__ q, long q_stride, bf16_t* __rest
   struct Staged {
     uint4 k[LDS_K_PER_THREAD], v[LDS_V_PER_THREAD];
   };
-  auto fetch = [&](Staged& st, int kt, int page) {
+  // the keys that count in a tile: the kept keys before the block's span, or the span itself
+  auto tile_lo = [&](bool kept) { return kept ? 0 : key_begin; };
+  auto tile_hi = [&](bool kept) { return kept ? kept_end : key_end; };
+  auto fetch = [&](Staged& st, int kt, bool kept, int page) {
     if constexpr (FAST) {
       const int lp = page_shift >= 0 ? (kt >> page_shift) : (kt / page_size);
       const int slot0 = kt - lp * page_size;  // the tile's first slot in its page
@@ -603,7 +632,7 @@ attention_lds_kernel(const bf16_t* __restrict__ q, long q_stride, bf16_t* __rest
         if (c < LDS_K_CHUNKS) {
           const int key = kt + c / (HEAD_DIM / 8);
           const int dp = c % (HEAD_DIM / 8);
-          if (key >= key_begin && key < key_end) {
+          if (key >= tile_lo(kept) && key < tile_hi(kept)) {
             int ks;
             const int pg = page_of(key, ks);
             st.k[i] = *(const uint4*)(kbase + (size_t)pg * 2 * plane + (size_t)ks * HEAD_DIM + 8 * dp);
@@ -618,7 +647,7 @@ attention_lds_kernel(const bf16_t* __restrict__ q, long q_stride, bf16_t* __rest
           const int kb = c / HEAD_DIM;
           const int d = c - kb * HEAD_DIM;
           const int key = kt + 8 * kb;
-          if (key + 7 >= key_begin && key < key_end) {
+          if (key + 7 >= tile_lo(kept) && key < tile_hi(kept)) {
             int vs;
             const int pg = page_of(key, vs);
             st.v[i] = *(const uint4*)(vbase + (size_t)pg * 2 * plane + ((size_t)(vs >> 3) * HEAD_DIM + d) * 8);
@@ -628,8 +657,9 @@ attention_lds_kernel(const bf16_t* __restrict__ q, long q_stride, bf16_t* __rest
     }
   };
   // writes a fetched tile to LDS, with zeros for the keys outside the block's span
-  auto stash = [&](const Staged& st, int kt, int buf) {
-    const bool whole = kt >= key_begin && kt + 32 <= key_end;  // all but a span's first and last tiles
+  auto stash = [&](const Staged& st, int kt, bool kept, int buf) {
+    const int k_lo = tile_lo(kept), k_hi = tile_hi(kept);
+    const bool whole = kt >= k_lo && kt + 32 <= k_hi;  // all but a span's first and last tiles
     if (FAST && whole) {  // nothing to zero: the registers go to LDS as they are
 #pragma unroll
       for (int i = 0; i < LDS_K_PER_THREAD; ++i) {
@@ -651,7 +681,7 @@ attention_lds_kernel(const bf16_t* __restrict__ q, long q_stride, bf16_t* __rest
         const int t = (kk >> 2) & 1;
         const int m = 4 * (kk >> 3) + (kk & 3);
         const int key = kt + kk;
-        const bool inside = whole || (key >= key_begin && key < key_end);
+        const bool inside = whole || (key >= k_lo && key < k_hi);
         *(uint4*)(&lds_k[buf][(t * 16 + m) * LDS_K_STRIDE + 8 * dp]) = inside ? st.k[i] : make_uint4(0, 0, 0, 0);
       }
     }
@@ -662,13 +692,13 @@ attention_lds_kernel(const bf16_t* __restrict__ q, long q_stride, bf16_t* __rest
         const int key = kt + 8 * (c / HEAD_DIM);
         uint4 v = st.v[i];
         if (whole) {
-        } else if (key + 7 < key_begin || key >= key_end) {
+        } else if (key + 7 < k_lo || key >= k_hi) {
           v = make_uint4(0, 0, 0, 0);
-        } else if (key < key_begin || key + 7 >= key_end) {  // the span's first or last keys: zero what lies outside
+        } else if (key < k_lo || key + 7 >= k_hi) {  // the span's first or last keys: zero what lies outside
           uint32_t keep[4] = {0xffffffffu, 0xffffffffu, 0xffffffffu, 0xffffffffu};
 #pragma unroll
           for (int e = 0; e < 8; ++e)
-            if (key + e < key_begin || key + e >= key_end) keep[e >> 1] &= (e & 1) ? 0x0000ffffu : 0xffff0000u;
+            if (key + e < k_lo || key + e >= k_hi) keep[e >> 1] &= (e & 1) ? 0x0000ffffu : 0xffff0000u;
           v.x &= keep[0];
           v.y &= keep[1];
           v.z &= keep[2];
@@ -701,12 +731,13 @@ attention_lds_kernel(const bf16_t* __restrict__ q, long q_stride, bf16_t* __rest
 
   // a key that a row of this wavefront reads must have a page, or the wavefront's rows become NaN
   const bool page_missing =
-      span_lacks_page(table, table_width, num_pages, page_size, page_shift, max(lo_w, key_begin), min(hi_w, key_end - 1), lane);
+      span_lacks_page(table, table_width, num_pages, page_size, page_shift, max(lo_w, key_begin), min(hi_w, key_end - 1), lane) ||
+      (kept_end > 0 && hi_w >= 0 && span_lacks_page(table, table_width, num_pages, page_size, page_shift, 0, kept_end - 1, lane));
 
   // one 32-key tile from LDS buffer `buf`: scores, running softmax, weighted values
-  auto compute = [&](int kt, const bf16_t* kbuf, const bf16_t* vbuf) {
+  auto compute = [&](int kt, bool kept, const bf16_t* kbuf, const bf16_t* vbuf) {
     // a wavefront whose rows all end before this tile, or start after it, has nothing to add
-    if (!(kt <= hi_w && kt + 31 >= lo_w)) return;
+    if (!(kt <= hi_w && (kt + 31 >= lo_w || IS_KEPT(kt)))) return;
     // ---- S^T = K Q^T ------------------------------------------------------------------ //
     float4v st[LDS_RT][2];
 #pragma unroll
@@ -728,13 +759,14 @@ attention_lds_kernel(const bf16_t* __restrict__ q, long q_stride, bf16_t* __rest
       }
     }
     // ---- mask, running maximum, probabilities ------------------------------------------------ //
-    const bool need_mask = kt < lo_all || kt + 31 > hi_all;
+    const bool need_mask = kept || kt < lo_all || kt + 31 > hi_all;
     float alpha[LDS_RT];
     Frag8 pf[LDS_RT];
     bool moved = false;
 #pragma unroll
     for (int rt = 0; rt < LDS_RT; ++rt) {
-      SOFTMAX_TILE(true, st[rt][0], st[rt][1], need_mask, row_valid[rt] && key >= row_start[rt] && key <= row_end[rt], m_run[rt],
+      SOFTMAX_TILE(true, st[rt][0], st[rt][1], need_mask,
+                   row_valid[rt] && key <= row_end[rt] && (kept ? key < kept_end : key >= row_start[rt] || (IS_KEPT(key) && key >= key_begin)), m_run[rt],
                    neg_mc_run[rt], l_run[rt], alpha[rt], pf[rt], slope_raw[rt], rate[rt], row_end[rt] - (kt + 8 * j))
       moved = moved || alpha[rt] != 1.0f;
     }
@@ -764,7 +796,8 @@ attention_lds_kernel(const bf16_t* __restrict__ q, long q_stride, bf16_t* __rest
   };
 
   const int kt_first = key_begin & ~31;
-  const int n_tiles = (key_end - kt_first + 31) / 32;
+  const int n_tiles = kept_tiles + (key_end - kt_first + 31) / 32;
+  auto first_key = [&](int tile) { return tile < kept_tiles ? 32 * tile : kt_first + 32 * (tile - kept_tiles); };
   if constexpr (MODE == LDS_DMA) {
     // tile t lies in buffer t % DMA_BUFFERS; its loads are issued DMA_AHEAD tiles ahead, after the
     // barrier that ends the use of that buffer by tile t - 1
@@ -795,9 +828,10 @@ attention_lds_kernel(const bf16_t* __restrict__ q, long q_stride, bf16_t* __rest
     for (int i = 0; i < VPT; ++i) v_off[i] = (uint32_t)(plane * 2) + (uint32_t)((4 * i + wave) * 64 + lane) * 16;
     // where the next tile to be loaded lies: its first key, its slot in its page, that page's keys
     // in the cache, and the table's entry for the page after it, read a page ahead; all uniform
-    int issue_kt = kt_first;
-    int issue_lp = page_shift >= 0 ? (kt_first >> page_shift) : (kt_first / page_size);
-    int issue_slot = kt_first - issue_lp * page_size;
+    int issue_kt = first_key(0);
+    int issue_lp = page_shift >= 0 ? (issue_kt >> page_shift) : (issue_kt / page_size);
+    int issue_slot = issue_kt - issue_lp * page_size;
+    int kept_left = kept_tiles;  // tiles of kept keys still to be issued; after the last one the range follows
     auto entry = [&](int lp) -> int { return lp < table_width ? table[lp] : 0; };
     auto page_keys = [&](int raw, int kt) -> const bf16_t* {
       const int page = (kt < key_end && raw >= 0 && raw < num_pages) ? raw : 0;  // past the span: any page, never used
@@ -814,7 +848,13 @@ attention_lds_kernel(const bf16_t* __restrict__ q, long q_stride, bf16_t* __rest
       for (int i = 0; i < VPT; ++i) dma16(src, v_off[i], dst + DMA_K_BYTES + i * 4096);
       issue_kt += 32;
       issue_slot += 32;
-      if (issue_slot == page_size) {
+      if (kept_tiles > 0 && --kept_left == 0) {
+        issue_kt = kt_first;
+        issue_lp = page_shift >= 0 ? (kt_first >> page_shift) : (kt_first / page_size);
+        issue_slot = kt_first - issue_lp * page_size;
+        issue_page = page_keys(entry(issue_lp), issue_kt);
+        entry_after = entry(issue_lp + 1);
+      } else if (issue_slot == page_size) {
         issue_slot = 0;
         ++issue_lp;
         issue_page = page_keys(entry_after, issue_kt);
@@ -823,17 +863,17 @@ attention_lds_kernel(const bf16_t* __restrict__ q, long q_stride, bf16_t* __rest
     };
     // zeros over the values of keys outside the block's span (their scores are masked, but what
     // lies there may be anything, also not a number)
-    auto zero_outside = [&](int kt, bf16_t* vbuf) {
+    auto zero_outside = [&](int kt, int k_lo, int k_hi, bf16_t* vbuf) {
 #pragma unroll
       for (int i = 0; i < VPT; ++i) {
         const int c = tid + 256 * i;
         const int key = kt + 8 * (c / HEAD_DIM);
-        if (key >= key_begin && key + 8 <= key_end) continue;
+        if (key >= k_lo && key + 8 <= k_hi) continue;
         uint4 v = *(uint4*)(vbuf + (size_t)c * 8);
         uint32_t keep[4] = {0xffffffffu, 0xffffffffu, 0xffffffffu, 0xffffffffu};
 #pragma unroll
         for (int e = 0; e < 8; ++e)
-          if (key + e < key_begin || key + e >= key_end) keep[e >> 1] &= (e & 1) ? 0x0000ffffu : 0xffff0000u;
+          if (key + e < k_lo || key + e >= k_hi) keep[e >> 1] &= (e & 1) ? 0x0000ffffu : 0xffff0000u;
         v.x &= keep[0];
         v.y &= keep[1];
         v.z &= keep[2];
@@ -846,7 +886,8 @@ attention_lds_kernel(const bf16_t* __restrict__ q, long q_stride, bf16_t* __rest
     for (int it = 0; it < n_tiles; it += DMA_BUFFERS) {
 #pragma unroll
       for (int u = 0; u < DMA_BUFFERS; ++u) {
-        const int kt = kt_first + 32 * (it + u);
+        const int kt = first_key(it + u);
+        const bool kept = it + u < kept_tiles;
         // this thread's loads of tile it + u have landed (those of the tiles after it may be in flight);
         // after the barrier so have everyone's, and everyone has left tile it + u - 1
         asm volatile("s_waitcnt vmcnt(%0)\n\ts_barrier" : : "n"((DMA_AHEAD - 1) * (KPT + VPT)) : "memory");
@@ -854,11 +895,11 @@ attention_lds_kernel(const bf16_t* __restrict__ q, long q_stride, bf16_t* __rest
         if (it + u < n_tiles) {
           bf16_t* kbuf = lds_dma + u * (DMA_TILE_BYTES / 2);
           bf16_t* vbuf = kbuf + DMA_K_BYTES / 2;
-          if (kt < key_begin || kt + 32 > key_end) {  // a span's first or last tile
-            zero_outside(kt, vbuf);
+          if (kt < tile_lo(kept) || kt + 32 > tile_hi(kept)) {  // a span's first or last tile
+            zero_outside(kt, tile_lo(kept), tile_hi(kept), vbuf);
             __syncthreads();
           }
-          compute(kt, kbuf, vbuf);
+          compute(kt, kept, kbuf, vbuf);
         }
       }
     }
@@ -867,40 +908,44 @@ attention_lds_kernel(const bf16_t* __restrict__ q, long q_stride, bf16_t* __rest
     // tile t waits in registers set t % 2 and is multiplied from LDS buffer t % 2; its fetch is
     // issued three tiles ahead of its use and has two iterations to arrive
     Staged sa, sb;
-    fetch(sa, kt_first, tile_page(kt_first));
-    fetch(sb, kt_first + 32, tile_page(kt_first + 32));
-    int page_next = tile_page(kt_first + 64);
-    stash(sa, kt_first, 0);
-    fetch(sa, kt_first + 64, page_next);
-    page_next = tile_page(kt_first + 96);
+    auto fetch_tile = [&](Staged& st, int tile, int page) { fetch(st, first_key(tile), tile < kept_tiles, page); };
+    auto stash_tile = [&](const Staged& st, int tile, int buf) { stash(st, first_key(tile), tile < kept_tiles, buf); };
+    auto compute_tile = [&](int tile, int buf) { compute(first_key(tile), tile < kept_tiles, lds_k[buf], lds_v[buf]); };
+    auto page_of_tile = [&](int tile) { return tile_page(first_key(tile)); };
+    fetch_tile(sa, 0, page_of_tile(0));
+    fetch_tile(sb, 1, page_of_tile(1));
+    int page_next = page_of_tile(2);
+    stash_tile(sa, 0, 0);
+    fetch_tile(sa, 2, page_next);
+    page_next = page_of_tile(3);
     __syncthreads();
     for (int it = 0; it < n_tiles; it += 2) {
-      const int kt = kt_first + 32 * it;
-      compute(kt, lds_k[0], lds_v[0]);
-      stash(sb, kt + 32, 1);
-      fetch(sb, kt + 96, page_next);
-      page_next = tile_page(kt + 128);
+      compute_tile(it, 0);
+      stash_tile(sb, it + 1, 1);
+      fetch_tile(sb, it + 3, page_next);
+      page_next = page_of_tile(it + 4);
       __syncthreads();
-      if (it + 1 < n_tiles) compute(kt + 32, lds_k[1], lds_v[1]);
-      stash(sa, kt + 64, 0);
-      fetch(sa, kt + 128, page_next);
-      page_next = tile_page(kt + 160);
+      if (it + 1 < n_tiles) compute_tile(it + 1, 1);
+      stash_tile(sa, it + 2, 0);
+      fetch_tile(sa, it + 4, page_next);
+      page_next = page_of_tile(it + 5);
       __syncthreads();
     }
   } else {
     Staged sa;
-    fetch(sa, kt_first, 0);
-    stash(sa, kt_first, 0);
-    if (n_tiles > 1) fetch(sa, kt_first + 32, 0);
+    auto fetch_tile = [&](int tile) { fetch(sa, first_key(tile), tile < kept_tiles, 0); };
+    auto stash_tile = [&](int tile, int buf) { stash(sa, first_key(tile), tile < kept_tiles, buf); };
+    fetch_tile(0);
+    stash_tile(0, 0);
+    if (n_tiles > 1) fetch_tile(1);
     __syncthreads();
     for (int it = 0; it < n_tiles; ++it) {
-      const int kt = kt_first + 32 * it;
       const int buf = it & 1;
-      compute(kt, lds_k[buf], lds_v[buf]);
+      compute(first_key(it), it < kept_tiles, lds_k[buf], lds_v[buf]);
       // tile it + 1 (fetched an iteration ago) goes into the other buffer, which every wavefront
       // left at the last barrier; then tile it + 2 is fetched
-      if (it + 1 < n_tiles) stash(sa, kt + 32, buf ^ 1);
-      if (it + 2 < n_tiles) fetch(sa, kt + 64, 0);
+      if (it + 1 < n_tiles) stash_tile(it + 1, buf ^ 1);
+      if (it + 2 < n_tiles) fetch_tile(it + 2);
       __syncthreads();
     }
   }
@@ -925,7 +970,8 @@ attention_lds_kernel(const bf16_t* __restrict__ q, long q_stride, bf16_t* __rest
       continue;
     }
     if (sink) l_row += __builtin_amdgcn_exp2f(sink[hq[rt]] * 1.4426950408889634f - m_run[rt] * scale_log2e);
-    const float inv = page_missing ? not_a_number() : 1.0f / l_row;
+    float inv = page_missing ? not_a_number() : 1.0f / l_row;
+    if (out_scale) inv *= out_scale[(size_t)(q0 + ti[rt]) * n_q_heads + hq[rt]];
     bf16_t* orow = out + (size_t)(q0 + ti[rt]) * out_stride + (size_t)hq[rt] * HEAD_DIM;
 #pragma unroll
     for (int dt = 0; dt < D_TILES; ++dt) {
@@ -947,7 +993,7 @@ template <int MERGE_WAVES>
 __global__ void __launch_bounds__(MERGE_WAVES * 64)
 attention_merge_kernel(bf16_t* __restrict__ out, long out_stride, const float* __restrict__ partial,
                        const int* __restrict__ cu_q, const int* __restrict__ merge, int n_q_heads, int n_kv_heads,
-                       const float* __restrict__ sink) {
+                       const float* __restrict__ sink, const float* __restrict__ out_scale) {
   __shared__ float red_max[MERGE_WAVES];
   __shared__ float red_l[MERGE_WAVES];
   __shared__ float red_o[MERGE_WAVES][HEAD_DIM];
@@ -1009,7 +1055,8 @@ attention_merge_kernel(bf16_t* __restrict__ out, long out_stride, const float* _
 #pragma unroll
   for (int w = 0; w < MERGE_WAVES; ++w) l_all += red_l[w];
   if (sink) l_all += exp2f(sink[hq] * 1.4426950408889634f - m_all);  // the maxima are kept in the scaled (log2) domain
-  const float inv = 1.0f / l_all;
+  float inv = 1.0f / l_all;
+  if (out_scale) inv *= out_scale[(size_t)(q0 + ti) * n_q_heads + hq];
   bf16_t* orow = out + (size_t)(q0 + ti) * out_stride + (size_t)hq * HEAD_DIM;
 #pragma unroll
   for (int i = 0; i < (HEAD_DIM + 63) / 64; ++i) {
@@ -1029,7 +1076,16 @@ extern "C" int cwm_attention_mfma(const void* q, long q_stride, void* out, long 
                                   int wide_three_blocks, const int* merge,
                                   int n_merge, int n_merge_mid, int n_merge_few, float* partial, int n_q_heads, int n_kv_heads, int head_dim,
                                   int page_size, int num_pages, int window_left, int chunk, float scale, float softcap,
-                                  const float* sink, const float* bias_slope, const float* bias_rate, hipStream_t stream) {
+                                  const float* sink, const float* bias_slope, const float* bias_rate, const float* out_scale, int keep_first,
+                                  hipStream_t stream) {
+  // `out_scale`: null, or float32 [tokens][n_q_heads], a factor on a head's finished row
+#ifdef KEPT_KEYS
+  CWM_REQUIRE(keep_first >= 0 && chunk == 0, "attention_mfma: kept first keys go with a window, not with blocks of keys");
+#define KEPT_ARGS , keep_first
+#else
+  CWM_REQUIRE(keep_first == 0, "attention_mfma: this library is built without kept first keys");
+#define KEPT_ARGS
+#endif
 #ifdef DISTANCE_BIAS
   CWM_REQUIRE(bias_slope && bias_rate, "attention_mfma: this library takes a distance bias off the scores, with a slope and a rate a head");
 #define BIAS_ARGS , bias_slope, bias_rate
@@ -1069,7 +1125,7 @@ extern "C" int cwm_attention_mfma(const void* q, long q_stride, void* out, long 
   hipLaunchKernelGGL((attention_mfma_kernel<PAGE32>), dim3((unsigned)blocks), dim3(256), 0, stream, (const bf16_t*)q,     \
                      q_stride, (bf16_t*)out, out_stride, (const bf16_t*)cache, block_table, table_width, cu_q, kv_len,   \
                      work, n_work, partial, n_q_heads, n_kv_heads, page_size, page_shift, num_pages, window_left,        \
-                     chunk, scale_log2e, cap_raw, sink BIAS_ARGS)
+                     chunk, scale_log2e, cap_raw, sink, out_scale BIAS_ARGS KEPT_ARGS)
     if (page_size % 32 == 0)
       CWM_LAUNCH_TEAM(true);
     else
@@ -1085,7 +1141,7 @@ extern "C" int cwm_attention_mfma(const void* q, long q_stride, void* out, long 
   hipLaunchKernelGGL((attention_lds_kernel<MODE, BUFFERS, MIN_BLOCKS>), dim3((unsigned)blocks), dim3(256), 0, stream,     \
                      (const bf16_t*)q, q_stride,                                                                          \
                      (bf16_t*)out, out_stride, (const bf16_t*)cache, block_table, table_width, cu_q, kv_len, work_wide,   \
-                     partial, n_kv_heads, n_q_heads, n_kv_heads, page_size, page_shift, num_pages, window_left, chunk, scale_log2e, cap_raw, sink BIAS_ARGS)
+                     partial, n_kv_heads, n_q_heads, n_kv_heads, page_size, page_shift, num_pages, window_left, chunk, scale_log2e, cap_raw, sink, out_scale BIAS_ARGS KEPT_ARGS)
     // tiles of 32 keys that never straddle a page, and shares of a tile that divide evenly over the block
     if (page_size % 32 == 0 && LDS_K_CHUNKS % 256 == 0 && LDS_V_CHUNKS % 256 == 0) {
 #if DMA_HEAD_DIM_OK
@@ -1115,7 +1171,7 @@ extern "C" int cwm_attention_mfma(const void* q, long q_stride, void* out, long 
 #define CWM_LAUNCH_MERGE(WAVES, COUNT, FIRST)                                                                              \
   if ((COUNT) > 0)                                                                                                        \
   hipLaunchKernelGGL(attention_merge_kernel<WAVES>, dim3(COUNT, n_kv_heads, 16), dim3(WAVES * 64), 0, stream, (bf16_t*)out, \
-                     out_stride, (const float*)partial, cu_q, merge + (size_t)(FIRST) * 4, n_q_heads, n_kv_heads, sink)
+                     out_stride, (const float*)partial, cu_q, merge + (size_t)(FIRST) * 4, n_q_heads, n_kv_heads, sink, out_scale)
     CWM_LAUNCH_MERGE(16, n_many, 0);
     CWM_LAUNCH_MERGE(4, n_merge_mid, n_many);
     CWM_LAUNCH_MERGE(1, n_merge_few, n_many + n_merge_mid);

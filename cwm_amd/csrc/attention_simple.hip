@@ -11,6 +11,9 @@
 // of that many positions counted from 0 (the query at p reads the keys of its own block up to p), and `softcap` > 0
 // caps the scaled score, s_j <- softcap * tanh(s_j / softcap), before the softmax.  A distance bias (`bias_slope`,
 // `bias_rate`: float32, one number a query head) then comes off it, s_j <- s_j - slope_h * ln(1 + rate_h * (p - j)).
+// With `keep_first` > 0 a query also reads the sequence's first `keep_first` keys, however far before its window they lie
+// (its first segment takes those that do, as chunks ahead of its own).  `out_scale` (float32 [tokens][n_q_heads], or null)
+// is a factor on a head's finished row.
 //
 // One block of four wavefronts per (token, key/value head, up to 8 of its query heads,
 // segment of the keys): a key and a value are loaded once and used for all the block's
@@ -77,7 +80,8 @@ attention_simple_kernel(const T* __restrict__ q, long q_stride, T* __restrict__ 
                         const int* __restrict__ positions, const int* __restrict__ seq_of_token, float* __restrict__ partial,
                         int n_q_heads, int n_kv_heads, int head_groups, int head_dim, int page_size, int num_pages,
                         int window_left, int chunk, float scale, float softcap, const float* __restrict__ sink,
-                        const float* __restrict__ bias_slope, const float* __restrict__ bias_rate) {
+                        const float* __restrict__ bias_slope, const float* __restrict__ bias_rate, int keep_first,
+                        const float* __restrict__ out_scale) {
   __shared__ __attribute__((aligned(16))) float qs[HEADS][D_REGS * CWM_WAVE];
   // probabilities of a chunk, key jj at [in0 + jj] (in0: the first key's place in its block of 8 values), so that the
   // eight of a block lie at a multiple of 8
@@ -139,11 +143,18 @@ attention_simple_kernel(const T* __restrict__ q, long q_stride, T* __restrict__ 
     for (int r = 0; r < D_REGS; ++r) o[h][r] = 0.f;
   }
 
-  // wavefront w takes the chunks of 64 keys w, w + SIMPLE_WAVES, ... of the segment
-  for (int base = k0 + wave * CWM_WAVE; base < k1; base += SIMPLE_WAVES * CWM_WAVE) {
+  // wavefront w takes the chunks of 64 keys w, w + SIMPLE_WAVES, ... of the segment; chunks of kept keys that lie before
+  // the window come first
+  const int kept_end = seg == 0 ? min(keep_first, start) : 0;
+  const int kept_chunks = (kept_end + CWM_WAVE - 1) / CWM_WAVE;
+  const int n_chunks = kept_chunks + (k1 - k0 + CWM_WAVE - 1) / CWM_WAVE;
+  for (int c = wave; c < n_chunks; c += SIMPLE_WAVES) {
+    const bool kept = c < kept_chunks;
+    const int base = kept ? c * CWM_WAVE : k0 + (c - kept_chunks) * CWM_WAVE;
+    const int end = kept ? kept_end : k1;
     const int j = base + lane;
-    const bool valid = j < k1;
-    const int n = min(CWM_WAVE, k1 - base);
+    const bool valid = j < end;
+    const int n = min(CWM_WAVE, end - base);
     const int in0 = base & 7;  // the first key's place in its block of 8 values
     float s[HEADS];
 #pragma unroll
@@ -334,6 +345,7 @@ attention_simple_kernel(const T* __restrict__ q, long q_stride, T* __restrict__ 
     // counts once for the token, so where the token has several segments the join kernel adds it
     if (sink && n_seg == 1) l_all += expf(sink[h0 + h] - m_all);
     T* orow = out + (size_t)t * out_stride + (size_t)(h0 + h) * head_dim;
+    const float factor = out_scale ? out_scale[(size_t)t * n_q_heads + h0 + h] : 1.f;
     float* prow = n_seg > 1 ? partial + (((size_t)t * n_q_heads + h0 + h) * SIMPLE_MAX_SEGMENTS + seg) * PARTIAL_STRIDE(head_dim) : nullptr;
 #pragma unroll
     for (int r = 0; r < D_REGS; ++r) {
@@ -345,7 +357,7 @@ attention_simple_kernel(const T* __restrict__ q, long q_stride, T* __restrict__ 
         if (n_seg > 1)
           prow[d] = sum;
         else
-          Elem<T>::store(orow + d, sum / l_all);
+          Elem<T>::store(orow + d, sum / l_all * factor);
       }
     }
     if (n_seg > 1 && lane == 0) {
@@ -361,7 +373,7 @@ template <typename T>
 __global__ void __launch_bounds__(CWM_WAVE)
 attention_simple_join_kernel(T* __restrict__ out, long out_stride, const float* __restrict__ partial,
                              const int* __restrict__ positions, int n_q_heads, int head_dim, int window_left, int chunk,
-                             int max_segments, const float* __restrict__ sink) {
+                             int max_segments, const float* __restrict__ sink, const float* __restrict__ out_scale) {
   const int t = blockIdx.x / n_q_heads;
   const int h = blockIdx.x - t * n_q_heads;
   const int lane = threadIdx.x;
@@ -390,16 +402,17 @@ attention_simple_join_kernel(T* __restrict__ out, long out_stride, const float* 
     }
   }
   if (sink) l_all += expf(sink[h] - m_all);
+  const float factor = out_scale ? out_scale[(size_t)t * n_q_heads + h] : 1.f;
   T* orow = out + (size_t)t * out_stride + (size_t)h * head_dim;
 #pragma unroll
   for (int r = 0; r < SIMPLE_D_REGS; ++r) {
     const int d = lane + r * CWM_WAVE;
-    if (d < head_dim) Elem<T>::store(orow + d, o[r] / l_all);
+    if (d < head_dim) Elem<T>::store(orow + d, o[r] / l_all * factor);
   }
 }
 
-// `max_keys`: the most keys that any token of the call reads (its position + 1, or the window if that
-// is less); `sink`: null, or float32 [n_q_heads], a term exp(sink) of every softmax denominator that has no key and
+// `max_keys`: the most keys, kept ones before the window apart, that any token of the call reads (its position + 1, or the
+// window if that is less); `sink`: null, or float32 [n_q_heads], a term exp(sink) of every softmax denominator that has no key and
 // no value (it is not scaled and counts once a token); `partial`: float32 scratch of n_tokens * n_q_heads * 16 * (head_dim + 2) values, needed
 // (and touched) only if max_keys exceeds 2,048.  A token that reads more keys than `max_keys` says has no
 // place for its segments' results: its rows of `out` are NaN and every kernel ends normally.
@@ -408,7 +421,8 @@ extern "C" int cwm_attention_simple(const void* q, long q_stride, void* out, lon
                                     const int* seq_of_token, int n_tokens, int n_q_heads, int n_kv_heads,
                                     int head_dim, int page_size, int num_pages, int window_left, int chunk, float scale,
                                     float softcap, int max_keys, float* partial, const float* sink, const float* bias_slope,
-                                    const float* bias_rate, hipStream_t stream) {
+                                    const float* bias_rate, int keep_first, const float* out_scale, hipStream_t stream) {
+  CWM_REQUIRE(keep_first >= 0 && (keep_first == 0 || chunk == 0), "attention: kept first keys go with a window, not with blocks of keys");
   CWM_REQUIRE((bias_slope == nullptr) == (bias_rate == nullptr), "attention: a distance bias has a slope and a rate a head");
   CWM_REQUIRE(chunk >= 0 && softcap >= 0.f, "attention: a block of keys and a cap on the scores cannot be negative");
   CWM_REQUIRE(n_tokens >= 0, "attention: negative token count");
@@ -438,7 +452,7 @@ extern "C" int cwm_attention_simple(const void* q, long q_stride, void* out, lon
   hipLaunchKernelGGL((attention_simple_kernel<float, HEADS, D_REGS>), grid, dim3(SIMPLE_WAVES * CWM_WAVE), 0, stream,     \
                      (const float*)q, q_stride, (float*)out, out_stride, (const float*)cache, block_table, table_width,   \
                      positions, seq_of_token, partial, n_q_heads, n_kv_heads, head_groups, head_dim, page_size, num_pages, \
-                     window_left, chunk, scale, softcap, sink, bias_slope, bias_rate)
+                     window_left, chunk, scale, softcap, sink, bias_slope, bias_rate, keep_first, out_scale)
 #define CWM_LAUNCH_SIMPLE_HEADS(D_REGS)   \
   do {                                    \
     if (heads <= 2)                       \
@@ -460,15 +474,15 @@ extern "C" int cwm_attention_simple(const void* q, long q_stride, void* out, lon
 #undef CWM_LAUNCH_SIMPLE
     if (max_segments > 1)
       hipLaunchKernelGGL(attention_simple_join_kernel<float>, dim3((unsigned)join_blocks), dim3(CWM_WAVE), 0, stream,
-                         (float*)out, out_stride, (const float*)partial, positions, n_q_heads, head_dim, window_left, chunk, max_segments, sink);
+                         (float*)out, out_stride, (const float*)partial, positions, n_q_heads, head_dim, window_left, chunk, max_segments, sink, out_scale);
   } else if (dtype == CWM_BF16) {
     hipLaunchKernelGGL((attention_simple_kernel<bf16_t, SIMPLE_HEADS, SIMPLE_D_REGS>), grid, dim3(SIMPLE_WAVES * CWM_WAVE), 0, stream, (const bf16_t*)q,
                        q_stride, (bf16_t*)out, out_stride, (const bf16_t*)cache, block_table, table_width, positions,
                        seq_of_token, partial, n_q_heads, n_kv_heads, head_groups, head_dim, page_size, num_pages, window_left,
-                       chunk, scale, softcap, sink, bias_slope, bias_rate);
+                       chunk, scale, softcap, sink, bias_slope, bias_rate, keep_first, out_scale);
     if (max_segments > 1)
       hipLaunchKernelGGL(attention_simple_join_kernel<bf16_t>, dim3((unsigned)join_blocks), dim3(CWM_WAVE), 0, stream,
-                         (bf16_t*)out, out_stride, (const float*)partial, positions, n_q_heads, head_dim, window_left, chunk, max_segments, sink);
+                         (bf16_t*)out, out_stride, (const float*)partial, positions, n_q_heads, head_dim, window_left, chunk, max_segments, sink, out_scale);
   } else {
     return cwm_fail("attention: unknown dtype %d", dtype);
   }

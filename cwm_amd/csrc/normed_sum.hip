@@ -4,8 +4,9 @@
 //   x   <- x + sum_a c_a y_a / sqrt(mean(y_a^2) + eps_a) * w_a        in the order of the addends
 //   out  = x / sqrt(mean(x^2) + eps) * w
 //
-// An addend y_a is a [T, D] tensor (rows may lie apart) or float32 partial sums [P, T, D] of a product whose K was
-// split, added in order.  float32 arithmetic.  One block a row.  With `rows` only those rows are read and the residual
+// An addend y_a is a [T, D] tensor (rows may lie apart), float32 partial sums [P, T, D] of a product whose K was
+// split, added in order, or a token's weighted sum of float32 rows, y_a[t] = sum_k c[t][k] rows[index[t][k]] in the order
+// of k (what routed experts leave: an index below 0 names no row).  float32 arithmetic.  One block a row.  With `rows` only those rows are read and the residual
 // is left as it was.  Rows of up to 8,192 elements (a multiple of 4) with up to two addends stay in registers; others
 // are read again for every pass.
 #include "common.h"
@@ -22,6 +23,8 @@ struct NsumAddend {
   int n_partials;
   int dtype;
   float scale;
+  const int* row_index;  // [T][n_partials]: the rows of a weighted sum; null for the other two kinds
+  const float* row_weight;
 };
 
 struct NsumAddends {
@@ -45,6 +48,13 @@ __device__ __forceinline__ void nsum_load4(const void* p, int dtype, size_t e, f
 
 __device__ __forceinline__ float nsum_value(const NsumAddend& ad, size_t t, int e) {
   float y = 0.f;
+  if (ad.row_index) {
+    for (int k = 0; k < ad.n_partials; ++k) {
+      const int row = ad.row_index[t * ad.n_partials + k];
+      if (row >= 0) y += ad.row_weight[t * ad.n_partials + k] * ((const float*)ad.ptr)[(size_t)row * ad.ld + e];
+    }
+    return y;
+  }
   for (int p = 0; p < ad.n_partials; ++p) {
     const size_t at = (size_t)p * ad.partial_stride + t * ad.ld + e;
     y += ad.dtype == CWM_F32 ? ((const float*)ad.ptr)[at] : bf16_to_f32(((const bf16_t*)ad.ptr)[at]);
@@ -92,7 +102,25 @@ __global__ void normed_sum_regs_kernel(float* __restrict__ h, NsumAddends ad, co
 #pragma unroll
       for (int i = 0; i < 4; ++i) y[a][c][i] = 0.f;
       if (chunk < n_chunks) {
-        if (ad.a[a].n_partials == 1) {
+        if (ad.a[a].row_index) {
+          // four rows in flight at a time; what lies past the last, or names no row, is some row times zero
+          const int top = ad.a[a].n_partials;
+          for (int k = 0; k < top; k += 4) {
+            float z[4][4], keep[4];
+#pragma unroll
+            for (int u = 0; u < 4; ++u) {
+              const size_t at = t * top + min(k + u, top - 1);
+              const int row = ad.a[a].row_index[at];
+              keep[u] = k + u < top && row >= 0 ? ad.a[a].row_weight[at] : 0.f;
+              nsum_load4(ad.a[a].ptr, CWM_F32, (size_t)max(row, 0) * ad.a[a].ld + 4 * chunk, z[u]);
+              if (keep[u] == 0.f) z[u][0] = z[u][1] = z[u][2] = z[u][3] = 0.f;
+            }
+#pragma unroll
+            for (int u = 0; u < 4; ++u)
+#pragma unroll
+              for (int i = 0; i < 4; ++i) y[a][c][i] = fmaf(keep[u], z[u][i], y[a][c][i]);
+          }
+        } else if (ad.a[a].n_partials == 1) {
           nsum_load4(ad.a[a].ptr, ad.a[a].dtype, t * ad.a[a].ld + 4 * chunk, y[a][c]);
         } else {
           // four partial sums in flight at a time; what lies past the last is the last again, times zero
@@ -195,12 +223,14 @@ __global__ void normed_sum_kernel(float* __restrict__ h, NsumAddends ad, const f
   for (int e = threadIdx.x; e < dim; e += blockDim.x) Elem<TO>::store(out + (size_t)r * dim + e, (rows ? summed(e) : hrow[e]) * rstd * weight[e]);
 }
 
+// row_index[a], row_weight[a]: null, or the addend is a weighted sum of rows of ptrs[a] (float32), n_partials[a] of them a token.
 // h: float32 [T, dim], changed in place unless `rows` chooses rows.  Addend a: ptrs[a] of dtypes[a], rows lds[a] elements
 // apart, n_partials[a] slabs partial_strides[a] elements apart, normalised with `addend_eps`, times weights[a] (float32
 // [dim]) and scales[a].  weight: float32 [dim]; out: [n_out, dim] of out_dtype.
 extern "C" int cwm_normed_sum(float* h, int n_addends, const void* const* ptrs, const int* dtypes, const long* lds,
                               const int* n_partials, const long* partial_strides, const float* scales, const void* const* weights,
-                              float addend_eps, const float* weight, float eps, void* out, int out_dtype, const int* rows,
+                              const void* const* row_index, const void* const* row_weight, float addend_eps, const float* weight,
+                              float eps, void* out, int out_dtype, const int* rows,
                               int n_out, int dim, hipStream_t stream) {
   CWM_REQUIRE(n_out >= 0 && dim >= 1, "normed_sum: bad sizes");
   CWM_REQUIRE(n_addends >= 1 && n_addends <= NSUM_MAX, "normed_sum: %d addends are outside 1..%d", n_addends, NSUM_MAX);
@@ -215,7 +245,10 @@ extern "C" int cwm_normed_sum(float* h, int n_addends, const void* const* ptrs, 
   for (int a = 0; a < n_addends; ++a) {
     CWM_REQUIRE(ptrs[a] && weights[a] && n_partials[a] >= 1, "normed_sum: addend %d is empty", a);
     CWM_REQUIRE(n_partials[a] == 1 || dtypes[a] == CWM_F32, "normed_sum: partial sums must be float32");
-    ad.a[a] = NsumAddend{ptrs[a], (const float*)weights[a], lds[a], partial_strides[a], n_partials[a], dtypes[a], scales[a]};
+    ad.a[a] = NsumAddend{ptrs[a], (const float*)weights[a], lds[a], partial_strides[a], n_partials[a], dtypes[a], scales[a],
+                         (const int*)row_index[a], (const float*)row_weight[a]};
+    CWM_REQUIRE((row_index[a] == nullptr) == (row_weight[a] == nullptr) && (!row_index[a] || dtypes[a] == CWM_F32),
+                "normed_sum: a weighted sum of rows has indices, weights and float32 rows");
     const int bytes = dtypes[a] == CWM_F32 ? 4 : 2;
     vec = vec && lds[a] % 4 == 0 && partial_strides[a] % 4 == 0 && ((uintptr_t)ptrs[a] % (4 * bytes)) == 0 && ((uintptr_t)weights[a] % 16) == 0;
   }

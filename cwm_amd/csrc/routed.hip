@@ -2,7 +2,8 @@
 //
 //   route_top        per token: the `top` largest of its router logits (the lower index wins a tie) and the softmax
 //                    over those alone, float32; or, mode 1, the softmax over all experts, a choice by score plus a
-//                    correction per expert, and weights that are the chosen scores times a scale.
+//                    correction per expert, and weights that are the chosen scores times a scale.  Experts may form
+//                    equal groups of neighbours, of which only those with the best members stay open to the choice.
 //   group_by_expert  the step's (token, choice) pairs grouped by expert, each group padded to whole tiles of 16
 //                    rows: row_token[row] (-1 in the padding), pair_row[pair], tile_expert[tile] (-1 beyond the
 //                    last tile).  One block; no count leaves the device.  The order of a group's rows is whatever
@@ -11,7 +12,7 @@
 //                    or, for a batch of independent products (one weight per head, say), from the block's z.
 //                    bfloat16 operands on v_mfma_f32_16x16x32_bf16, float32 operands on v_mfma_f32_16x16x4_f32
 //                    (exact products); float32 sums in the order of k either way, whatever else is in the step.
-//                    With two weights the epilogue forms silu(W0 a) * (W1 a), or the clamped form of `GateAct`.
+//                    With two weights the epilogue forms silu(W0 a) * (W1 a), or another form of `GateAct`.
 //   combine          out[t] = sum_k weight[t][k] * rows[pair_row[t][k]] in the order of k, float32.
 //
 // Matrix-core layout as in the other products of this package: operand A = the weight tile (lane 16 j + r: row
@@ -40,7 +41,8 @@ extern "C" int cwm_route_tile_rows() { return TILE_ROWS; }
 // and, if given, to chosen_lds.
 __device__ __forceinline__ void route_wave(float (&score)[ROUTE_MAX_EXPERTS / CWM_WAVE], int lane, int n_experts, int top, int mode,
                                            const float* __restrict__ correction, float scale, int renormalize,
-                                           int* __restrict__ chosen_out, float* __restrict__ weights_out, int* chosen_lds) {
+                                           int n_groups, int keep_groups, int* __restrict__ chosen_out, float* __restrict__ weights_out,
+                                              int* chosen_lds) {
   const float neg_inf = -__builtin_inff();
   float choice[ROUTE_PER_LANE];  // what an expert is chosen by; score: what a weight is made of
 #pragma unroll
@@ -63,6 +65,40 @@ __device__ __forceinline__ void route_wave(float (&score)[ROUTE_MAX_EXPERTS / CW
       score[i] *= inv;
       choice[i] = e < n_experts ? (correction ? score[i] + correction[e] : score[i]) : neg_inf;
     }
+  }
+  if (keep_groups < n_groups) {
+    // the groups with the best members stay open: `keep_groups` votes, each for the best expert of the groups that are not
+    // open yet (the lower index among equals), which opens its group; every other expert then leaves the choice
+    const int size = n_experts / n_groups;
+    bool open[ROUTE_PER_LANE];
+#pragma unroll
+    for (int i = 0; i < ROUTE_PER_LANE; ++i) open[i] = false;
+    for (int k = 0; k < keep_groups; ++k) {
+      float bv = neg_inf;
+      int be = 0x7fffffff;
+#pragma unroll
+      for (int i = 0; i < ROUTE_PER_LANE; ++i) {
+        const int e = lane + CWM_WAVE * i;
+        if (e < n_experts && !open[i] && (be == 0x7fffffff || choice[i] > bv)) {
+          bv = choice[i];
+          be = e;
+        }
+      }
+#pragma unroll
+      for (int off = CWM_WAVE / 2; off > 0; off >>= 1) {
+        const float ov = __shfl_xor(bv, off, CWM_WAVE);
+        const int oe = __shfl_xor(be, off, CWM_WAVE);
+        if (oe != 0x7fffffff && (be == 0x7fffffff || ov > bv || (ov == bv && oe < be))) {
+          bv = ov;
+          be = oe;
+        }
+      }
+#pragma unroll
+      for (int i = 0; i < ROUTE_PER_LANE; ++i) open[i] = open[i] || (lane + CWM_WAVE * i) / size == be / size;
+    }
+#pragma unroll
+    for (int i = 0; i < ROUTE_PER_LANE; ++i)
+      if (!open[i]) choice[i] = neg_inf;  // open experts are at least `top`, so the votes below end before these
   }
   int idx[ROUTE_MAX_TOP];
   float val[ROUTE_MAX_TOP];
@@ -133,7 +169,8 @@ __device__ __forceinline__ void route_wave(float (&score)[ROUTE_MAX_EXPERTS / CW
 
 __global__ void __launch_bounds__(256) route_top_kernel(const float* __restrict__ logits, int* __restrict__ chosen,
                                                         float* __restrict__ weights, int n_tokens, int n_experts, int top, int mode,
-                                                        const float* __restrict__ correction, float scale, int renormalize) {
+                                                        const float* __restrict__ correction, float scale, int renormalize,
+                                                        int n_groups, int keep_groups) {
   const int lane = threadIdx.x & (CWM_WAVE - 1);
   const int t = blockIdx.x * (blockDim.x / CWM_WAVE) + threadIdx.x / CWM_WAVE;
   if (t >= n_tokens) return;
@@ -144,19 +181,22 @@ __global__ void __launch_bounds__(256) route_top_kernel(const float* __restrict_
     const int e = lane + CWM_WAVE * i;
     score[i] = e < n_experts ? z[e] : -__builtin_inff();
   }
-  route_wave(score, lane, n_experts, top, mode, correction, scale, renormalize, chosen + (size_t)t * top, weights + (size_t)t * top, nullptr);
+  route_wave(score, lane, n_experts, top, mode, correction, scale, renormalize, n_groups, keep_groups, chosen + (size_t)t * top, weights + (size_t)t * top, nullptr);
 }
 
 extern "C" int cwm_route_top(const float* logits, int* chosen, float* weights, int n_tokens, int n_experts, int top, int mode,
-                             const float* correction, float scale, int renormalize, hipStream_t stream) {
+                             const float* correction, float scale, int renormalize, int n_groups, int keep_groups, hipStream_t stream) {
   CWM_REQUIRE(logits && chosen && weights, "route_top: arguments missing");
   CWM_REQUIRE(top >= 1 && top <= ROUTE_MAX_TOP && top <= n_experts, "route_top: %d of %d experts, the kernel takes up to %d", top, n_experts,
               ROUTE_MAX_TOP);
   CWM_REQUIRE(n_experts <= ROUTE_MAX_EXPERTS, "route_top: %d experts, the kernel takes up to %d", n_experts, ROUTE_MAX_EXPERTS);
   CWM_REQUIRE(mode == 0 || mode == 1, "route_top: unknown mode %d", mode);
+  CWM_REQUIRE(n_groups >= 1 && n_experts % n_groups == 0 && keep_groups >= 1 && keep_groups <= n_groups &&
+                  top <= keep_groups * (n_experts / n_groups),
+              "route_top: %d of %d groups of %d experts do not hold %d choices", keep_groups, n_groups, n_experts, top);
   if (n_tokens <= 0) return 0;
   hipLaunchKernelGGL(route_top_kernel, dim3((n_tokens + 3) / 4), dim3(256), 0, stream, logits, chosen, weights, n_tokens, n_experts, top,
-                     mode, correction, scale, renormalize);
+                     mode, correction, scale, renormalize, n_groups, keep_groups);
   return cwm_launch_status("route_top");
 }
 
@@ -225,6 +265,7 @@ extern "C" int cwm_group_by_expert(const int* chosen, int n_tokens, int top, int
 // What the epilogue of a product with two weights makes of g = W0 a and u = W1 a:
 //   kind 0: silu(g) * u
 //   kind 1: g' * sigmoid(alpha g') * (u' + 1) with g' = min(g, limit), u' = clamp(u, -limit, limit)
+//   kind 2: gelu(g) * u, the tanh form of gelu
 struct GateAct {
   int kind;
   float alpha, limit;
@@ -235,6 +276,7 @@ __device__ __forceinline__ float gated_value(float g, float u, const GateAct act
     u = fminf(fmaxf(u, -act.limit), act.limit);
     return g / (1.f + expf(-act.alpha * g)) * (u + 1.f);
   }
+  if (act.kind == 2) return 0.5f * g * (1.f + tanhf(0.7978845608028654f * (g + 0.044715f * g * g * g))) * u;
   return g / (1.f + expf(-g)) * u;
 }
 
@@ -665,7 +707,7 @@ extern "C" int cwm_grouped_product(const void* a, long a_ld, long a_batch, int d
                                    long out_batch, int n_rows, int N, int K, int tiles_a_block, int act_kind, float act_alpha,
                                    float act_limit, hipStream_t stream) {
   CWM_REQUIRE(a && w0 && out, "grouped_product: arguments missing");
-  CWM_REQUIRE(act_kind == 0 || act_kind == 1, "grouped_product: unknown gated activation %d", act_kind);
+  CWM_REQUIRE(act_kind >= 0 && act_kind <= 2, "grouped_product: unknown gated activation %d", act_kind);
   const GateAct act = {act_kind, act_alpha, act_limit};
   CWM_REQUIRE(N > 0 && K > 0 && a_ld >= K && out_ld >= 0, "grouped_product: bad sizes");
   CWM_REQUIRE(tile_expert ? (n_tiles >= 0 && n_batch == 1 && row_token) : (n_batch >= 1 && n_batch <= 65535), "grouped_product: give a tile list or a number of batches");

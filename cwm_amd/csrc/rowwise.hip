@@ -474,7 +474,7 @@ extern "C" int cwm_act_rows(void* out, int out_dtype, const void* x, int x_dtype
 // What a gated feed-forward makes of its joined gate/up product: `x` is [T, 2 F (+ extra)] of type TX, a row's gate
 // values first, then its up values (or n_partials float32 slabs that are added in order first); out [T, F].
 // kind 0: silu(g) * u.  kind 1: g' * sigmoid(alpha * g') * (u' + 1) with g' = min(g, limit), u' = clamp(u, -limit,
-// limit).  With `row_gate_col` >= 0 the row is also multiplied by the sigmoid of that column of x (one more output
+// limit).  kind 2: gelu(g) * u, the tanh form of gelu.  With `row_gate_col` >= 0 the row is also multiplied by the sigmoid of that column of x (one more output
 // of the same product: a gate on the whole row).  float32 arithmetic, rounded once.
 __device__ __forceinline__ float gated_pair(float g, float u, int kind, float alpha, float limit) {
   if (kind == 1) {
@@ -482,6 +482,7 @@ __device__ __forceinline__ float gated_pair(float g, float u, int kind, float al
     u = fminf(fmaxf(u, -limit), limit);
     return g / (1.f + expf(-alpha * g)) * (u + 1.f);
   }
+  if (kind == 2) return act_value(g, 2) * u;
   return g / (1.f + expf(-g)) * u;
 }
 
@@ -513,8 +514,8 @@ extern "C" int cwm_gated_act_rows(void* out, int out_dtype, const void* x, int x
                                   float limit, hipStream_t stream) {
   CWM_REQUIRE(n_partials >= 1 && n_rows >= 0 && hidden >= 1, "gated_act_rows: bad sizes");
   CWM_REQUIRE(n_partials == 1 || x_dtype == CWM_F32, "gated_act_rows: partial sums must be float32");
-  CWM_REQUIRE(kind == 0 || kind == 1, "gated_act_rows: unknown gated activation %d", kind);
-  CWM_REQUIRE(kind == 0 || limit > 0.f, "gated_act_rows: the clamped form needs a positive limit");
+  CWM_REQUIRE(kind >= 0 && kind <= 2, "gated_act_rows: unknown gated activation %d", kind);
+  CWM_REQUIRE(kind != 1 || limit > 0.f, "gated_act_rows: the clamped form needs a positive limit");
   if (n_rows == 0) return 0;
   long blocks = ((long)n_rows * hidden + 255) / 256;
   if (blocks > 8192) blocks = 8192;

@@ -864,6 +864,15 @@ def _check_mask(window: Optional[int], chunk: Optional[int], softcap: Optional[f
         raise KernelError("a cap on the scores must be positive")
 
 
+def _check_kept(q: torch.Tensor, window: Optional[int], chunk: Optional[int], keep_first: int, out_scale: Optional[torch.Tensor]) -> None:
+    if keep_first < 0 or (keep_first > 0 and (chunk is not None or window is None)):
+        raise KernelError("kept first keys go with a window")
+    if out_scale is not None and (
+        q.dim() != 3 or out_scale.dtype != torch.float32 or tuple(out_scale.shape) != tuple(q.shape[:2]) or not out_scale.is_contiguous()
+    ):
+        raise KernelError("out_scale must be contiguous float32 [T, Hq]")
+
+
 def paged_attention_simple(
     q: torch.Tensor,
     cache: torch.Tensor,
@@ -877,6 +886,8 @@ def paged_attention_simple(
     softcap: Optional[float] = None,
     chunk: Optional[int] = None,
     distance_bias: Optional[Tuple[torch.Tensor, torch.Tensor]] = None,
+    keep_first: int = 0,
+    out_scale: Optional[torch.Tensor] = None,
 ) -> torch.Tensor:
     """Causal attention of `q` [T, Hq, hd] over the paged cache by the plain kernel:
     float32 arithmetic, a key/value head's query heads sharing its keys and values, long
@@ -886,8 +897,11 @@ def paged_attention_simple(
     each head's softmax denominator holds beside its keys (no key, no value, not scaled).  `softcap`: scaled scores
     become softcap * tanh(score / softcap) before the softmax.  `chunk` (instead of a window): a query reads the keys of
     its own block of that many positions, counted from 0, up to itself.  `distance_bias` (slope, rate), float32 [Hq]
-    each: slope_h * ln(1 + rate_h * (query's position - key's)) comes off the score.  Returns [T, Hq * hd]."""
-    _need_gpu(q, cache, block_table, positions, seq_of_token, sink)
+    each: slope_h * ln(1 + rate_h * (query's position - key's)) comes off the score.  `keep_first` (with a window): a query
+    also reads the sequence's first so many keys, however far back.  `out_scale`: float32 [T, Hq], a factor on every
+    head's result.  Returns [T, Hq * hd]."""
+    _need_gpu(q, cache, block_table, positions, seq_of_token, sink, out_scale)
+    _check_kept(q, window, chunk, keep_first, out_scale)
     bias_slope, bias_rate = _check_bias(distance_bias, q.shape[1] if q.dim() == 3 else 0)
     _check_mask(window, chunk, softcap)
     _check_sink(sink, q.shape[1] if q.dim() == 3 else 0)
@@ -922,7 +936,8 @@ def paged_attention_simple(
             _ptr(positions), _ptr(seq_of_token), ctypes.c_int(n_tokens), ctypes.c_int(n_q), ctypes.c_int(n_kv),
             ctypes.c_int(hd), ctypes.c_int(cache.shape[3] // hd), ctypes.c_int(cache.shape[0]),
             ctypes.c_int(-1 if window is None else window - 1), ctypes.c_int(chunk or 0), ctypes.c_float(scale),
-            ctypes.c_float(softcap or 0.0), ctypes.c_int(max_keys), _ptr(partial), _ptr(sink), _ptr(bias_slope), _ptr(bias_rate), _stream(),
+            ctypes.c_float(softcap or 0.0), ctypes.c_int(max_keys), _ptr(partial), _ptr(sink), _ptr(bias_slope), _ptr(bias_rate),
+            ctypes.c_int(keep_first), _ptr(out_scale), _stream(),
         ),
     )
     return out
@@ -1062,12 +1077,16 @@ def paged_attention_mfma(
     softcap: Optional[float] = None,
     chunk: Optional[int] = None,
     distance_bias: Optional[Tuple[torch.Tensor, torch.Tensor]] = None,
+    keep_first: int = 0,
+    out_scale: Optional[torch.Tensor] = None,
 ) -> torch.Tensor:
     """Matrix-core attention (bfloat16): prompt portions and decoded tokens in one
-    launch, long key ranges of short sequences split and merged.  `sink`, `softcap`, `chunk`, `distance_bias`: as in
-    `paged_attention_simple`; the bias is a build of its own, so that the other models' kernel does without its instructions."""
+    launch, long key ranges of short sequences split and merged.  `sink`, `softcap`, `chunk`, `distance_bias`, `keep_first`,
+    `out_scale`: as in `paged_attention_simple`; the bias and the kept keys are builds of their own, so that the other
+    models' kernel does without their instructions."""
+    _check_kept(q, window, chunk, keep_first, out_scale)
     bias_slope, bias_rate = _check_bias(distance_bias, q.shape[1] if q.dim() == 3 else 0)
-    _need_gpu(q, cache, block_table, sink)
+    _need_gpu(q, cache, block_table, sink, out_scale)
     _check_mask(window, chunk, softcap)
     _check_sink(sink, q.shape[1] if q.dim() == 3 else 0)
     if q.dtype != torch.bfloat16 or cache.dtype != torch.bfloat16:
@@ -1093,7 +1112,12 @@ def paged_attention_mfma(
     partial = None
     if plan.n_partials:
         partial = torch.empty(plan.n_partials * n_kv * 16 * (hd + 4), dtype=torch.float32, device=q.device)
-    lib = _build.load("attention_mfma", {"HEAD_DIM": hd} if distance_bias is None else {"DISTANCE_BIAS": 1, "HEAD_DIM": hd})
+    defines = {"HEAD_DIM": hd}
+    if distance_bias is not None:
+        defines["DISTANCE_BIAS"] = 1
+    if keep_first > 0:
+        defines["KEPT_KEYS"] = 1
+    lib = _build.load("attention_mfma", defines)
     _check(
         lib,
         lib.cwm_attention_mfma(
@@ -1105,7 +1129,8 @@ def paged_attention_mfma(
             _ptr(plan.merge), ctypes.c_int(plan.n_merge), ctypes.c_int(plan.n_merge_mid), ctypes.c_int(plan.n_merge_wide), _ptr(partial),
             ctypes.c_int(n_q), ctypes.c_int(n_kv), ctypes.c_int(hd), ctypes.c_int(page_size),
             ctypes.c_int(cache.shape[0]), ctypes.c_int(-1 if window is None else window - 1), ctypes.c_int(chunk or 0),
-            ctypes.c_float(scale), ctypes.c_float(softcap or 0.0), _ptr(sink), _ptr(bias_slope), _ptr(bias_rate), _stream(),
+            ctypes.c_float(scale), ctypes.c_float(softcap or 0.0), _ptr(sink), _ptr(bias_slope), _ptr(bias_rate), _ptr(out_scale),
+            ctypes.c_int(keep_first), _stream(),
         ),
     )
     return out
@@ -1122,6 +1147,8 @@ def paged_attention(
     softcap: Optional[float] = None,
     chunk: Optional[int] = None,
     distance_bias: Optional[Tuple[torch.Tensor, torch.Tensor]] = None,
+    keep_first: int = 0,
+    out_scale: Optional[torch.Tensor] = None,
 ) -> torch.Tensor:
     """Attention of the step's tokens over the cache.  `batch` is the step's
     `StepBatch` (positions, sequence of each token and the per-sequence lengths).
@@ -1129,12 +1156,12 @@ def paged_attention(
     matrix cores; float32, and other sizes, on the plain kernel."""
     hd = q.shape[2]
     if q.is_cuda and mfma_attention_takes(q.dtype, hd, cache.shape[3] // hd):
-        return paged_attention_mfma(q, cache, block_table, batch, window, scale, sink, softcap, chunk, distance_bias)
+        return paged_attention_mfma(q, cache, block_table, batch, window, scale, sink, softcap, chunk, distance_bias, keep_first, out_scale)
     static = getattr(batch, "static", None)
     max_keys = batch.max_kv_len if static is None else static.max_keys
     return paged_attention_simple(
         q, cache, block_table, batch.positions, batch.seq_of_token, window, scale, max_keys=max_keys, sink=sink, softcap=softcap, chunk=chunk,
-        distance_bias=distance_bias,
+        distance_bias=distance_bias, keep_first=keep_first, out_scale=out_scale,
     )
 
 
@@ -1304,4 +1331,7 @@ from .mixing import (  # noqa: E402
 )
 from .recurrence import (  # noqa: E402
     MAX_NORMED_ADDENDS, MAX_TOKEN_MIXES, NormedSum, add_normed_rmsnorm, embedding_sinusoid, min_gru, token_mixes,
+)
+from .projected import (  # noqa: E402
+    MAX_CONV_QK_CHANNELS, MAX_CONV_QK_TAPS, conv_qk_rope_write, latent_rows,
 )

@@ -13,6 +13,7 @@ import torch
 
 from . import build as _build
 from .sequence import step_segments
+from .streams import RoutedSum
 
 MAX_TOKEN_MIXES = 8  # csrc/token_mix.hip: TMIX_MAX
 MAX_NORMED_ADDENDS = 4  # csrc/normed_sum.hip: NSUM_MAX
@@ -56,7 +57,7 @@ def embedding_sinusoid(tokens: torch.Tensor, table: torch.Tensor, positions: tor
 
 class NormedSum:
     """A sum that has not been done yet: `terms` is a list of (tensor, weight, factor), each tensor ([T, D], rows may lie
-    apart, or float32 partial sums [P, T, D]) divided by its rows' root mean square (`eps` inside the root) and multiplied
+    apart, float32 partial sums [P, T, D], or a `RoutedSum`) divided by its rows' root mean square (`eps` inside the root) and multiplied
     by its weight (float32 [D]) and its factor.  The norm that reads the residual next adds the terms up in their order,
     in float32 (`add_normed_rmsnorm`)."""
 
@@ -65,13 +66,27 @@ class NormedSum:
         self.eps = float(eps)
 
 
-def _addends(terms: Sequence[Tuple[torch.Tensor, float]], n_tokens: int, dim: int):
-    """ctypes arrays (pointers, types, row distances, numbers of partial sums, their distances, factors) of addends."""
+def _addends(terms: Sequence[Tuple[Any, float]], n_tokens: int, dim: int):
+    """ctypes arrays (pointers, types, row distances, numbers of partial sums or of rows in a weighted sum, the partial sums'
+    distances, factors, and for weighted sums the rows' places and weights) of addends."""
     KernelError, _check, _code, _i32, _need_gpu, _ptr, _stream = _base()
     n = len(terms)
     ptrs, dtypes, lds, partials = (ctypes.c_void_p * n)(), (ctypes.c_int * n)(), (ctypes.c_long * n)(), (ctypes.c_int * n)()
     strides, scales = (ctypes.c_long * n)(), (ctypes.c_float * n)()
+    row_index, row_weight = (ctypes.c_void_p * n)(), (ctypes.c_void_p * n)()
     for i, (t, c) in enumerate(terms):
+        if isinstance(t, RoutedSum):
+            top = t.groups.top
+            _need_gpu(t.rows, t.weights, t.groups.pair_row)
+            if t.rows.dtype != torch.float32 or t.rows.dim() != 2 or t.rows.shape[1] != dim or not t.rows.is_contiguous():
+                raise KernelError(f"the experts' rows must be a contiguous float32 [rows, {dim}] tensor")
+            if t.weights.dtype != torch.float32 or tuple(t.weights.shape) != (n_tokens, top) or not t.weights.is_contiguous():
+                raise KernelError(f"the weights of a weighted sum must be float32 [{n_tokens}, {top}]")
+            if t.groups.pair_row.numel() != n_tokens * top:
+                raise KernelError("the list of rows does not fit the tokens")
+            ptrs[i], dtypes[i], scales[i], lds[i], partials[i] = t.rows.data_ptr(), _code(torch.float32), c, dim, top
+            row_index[i], row_weight[i] = t.groups.pair_row.data_ptr(), t.weights.data_ptr()
+            continue
         _need_gpu(t)
         if t.dim() == 3:
             if t.dtype != torch.float32 or not t.is_contiguous() or tuple(t.shape[1:]) != (n_tokens, dim):
@@ -82,7 +97,7 @@ def _addends(terms: Sequence[Tuple[torch.Tensor, float]], n_tokens: int, dim: in
                 raise KernelError(f"an addend {tuple(t.shape)} does not match the residual stream [{n_tokens}, {dim}]")
             partials[i], strides[i], lds[i] = 1, 0, (t.stride(0) if n_tokens > 1 else dim)
         ptrs[i], dtypes[i], scales[i] = t.data_ptr(), _code(t.dtype), c
-    return ptrs, dtypes, lds, partials, strides, scales
+    return ptrs, dtypes, lds, partials, strides, scales, row_index, row_weight
 
 
 def add_normed_rmsnorm(
@@ -104,7 +119,7 @@ def add_normed_rmsnorm(
             raise KernelError(f"{what} must be a contiguous float32 [{dim}] tensor")
     if rows is not None:
         _i32(rows, "rows")
-    ptrs, dtypes, lds, partials, strides, scales = _addends([(t, c) for t, _, c in delta.terms], n_tokens, dim)
+    ptrs, dtypes, lds, partials, strides, scales, row_index, row_weight = _addends([(t, c) for t, _, c in delta.terms], n_tokens, dim)
     weights = (ctypes.c_void_p * len(delta.terms))(*[w.data_ptr() for _, w, _ in delta.terms])
     n_out = n_tokens if rows is None else rows.numel()
     out = torch.empty((n_out, dim), dtype=out_dtype, device=h.device)
@@ -112,7 +127,7 @@ def add_normed_rmsnorm(
     _check(
         lib,
         lib.cwm_normed_sum(
-            _ptr(h), ctypes.c_int(len(delta.terms)), ptrs, dtypes, lds, partials, strides, scales, weights, ctypes.c_float(delta.eps),
+            _ptr(h), ctypes.c_int(len(delta.terms)), ptrs, dtypes, lds, partials, strides, scales, weights, row_index, row_weight, ctypes.c_float(delta.eps),
             _ptr(weight), ctypes.c_float(eps), _ptr(out), ctypes.c_int(_code(out_dtype)), _ptr(rows), ctypes.c_int(n_out), ctypes.c_int(dim), _stream(),
         ),
     )

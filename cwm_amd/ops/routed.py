@@ -26,14 +26,15 @@ def _base():
 
 def route_top(
     logits: torch.Tensor, top: int, scores: str = "softmax_chosen", correction: Optional[torch.Tensor] = None, scale: float = 1.0,
-    renormalize: bool = False,
+    renormalize: bool = False, groups: Optional[Tuple[int, int]] = None,
 ) -> Tuple[torch.Tensor, torch.Tensor]:
     """float32 router logits [T, E] -> (chosen int32 [T, top], weights float32 [T, top]), the chosen in falling order
     of what they were chosen by (the lower index first among equals).
     `scores` "softmax_chosen": the `top` largest logits, weighted by the softmax over those alone.
     `scores` "softmax_all": s = softmax over all experts; the `top` largest of s + `correction` (float32 [E], None for
     none) are chosen; their weights are `scale` * s (the correction is no part of a weight), divided by the sum of
-    the chosen s first if `renormalize`."""
+    the chosen s first if `renormalize`.  `groups` (count, keep): the experts form `count` equal groups of neighbours, and
+    only those of the `keep` groups with the best members can be chosen."""
     KernelError, _check, _code, _i32, _need_gpu, _ptr, _stream = _base()
     _need_gpu(logits, correction)
     if scores not in ("softmax_chosen", "softmax_all"):
@@ -47,6 +48,9 @@ def route_top(
     n, e = logits.shape
     if not 1 <= top <= min(e, MAX_ROUTE_TOP):
         raise KernelError(f"{top} of {e} experts: the kernel takes 1..{min(e, MAX_ROUTE_TOP)}")
+    count, keep = groups if groups is not None else (1, 1)
+    if count < 1 or e % count != 0 or not 1 <= keep <= count or top > keep * (e // count):
+        raise KernelError(f"{keep} of {count} groups of {e} experts do not hold {top} choices")
     chosen = torch.empty((n, top), dtype=torch.int32, device=logits.device)
     weights = torch.empty((n, top), dtype=torch.float32, device=logits.device)
     lib = _build.load("routed")
@@ -54,7 +58,8 @@ def route_top(
         lib,
         lib.cwm_route_top(
             _ptr(logits), _ptr(chosen), _ptr(weights), ctypes.c_int(n), ctypes.c_int(e), ctypes.c_int(top),
-            ctypes.c_int(int(scores == "softmax_all")), _ptr(correction), ctypes.c_float(scale), ctypes.c_int(int(renormalize)), _stream(),
+            ctypes.c_int(int(scores == "softmax_all")), _ptr(correction), ctypes.c_float(scale), ctypes.c_int(int(renormalize)),
+            ctypes.c_int(count), ctypes.c_int(keep), _stream(),
         ),
     )
     return chosen, weights
@@ -133,14 +138,15 @@ def _grouped(
 class GatedActivation:
     """What a gated feed-forward makes of g = W_gate x and u = W_up x.
     "silu": silu(g) * u.
-    "clamped_swish": g' * sigmoid(alpha * g') * (u' + 1) with g' = min(g, limit) and u' = clamp(u, -limit, limit)."""
+    "clamped_swish": g' * sigmoid(alpha * g') * (u' + 1) with g' = min(g, limit) and u' = clamp(u, -limit, limit).
+    "gelu_tanh": gelu(g) * u with the tanh form of gelu."""
 
     kind: str = "silu"
     alpha: float = 1.0
     limit: float = 0.0
 
     def code(self) -> int:
-        kinds = {"silu": 0, "clamped_swish": 1}
+        kinds = {"silu": 0, "clamped_swish": 1, "gelu_tanh": 2}
         if self.kind not in kinds:
             raise ValueError(f"gated activation {self.kind!r}: known are {', '.join(kinds)}")
         return kinds[self.kind]
@@ -204,30 +210,19 @@ def combine_routed(rows: torch.Tensor, groups: ExpertGroups, weights: torch.Tens
     return out
 
 
-def absorb_queries(q: torch.Tensor, lead: int, weight: torch.Tensor) -> torch.Tensor:
-    """Per head h: out[t, h] = [q[t, h, :lead] | W_h^T-applied rest], i.e. out[t, h, lead + j] = sum_d weight[h, j, d] * q[t, h, lead + d].
-    `q` [T, H, lead + d] contiguous, `weight` [H, n, d]; returns [T, H, lead + n] in the type of `q`."""
+def absorb_queries(rest: torch.Tensor, ask: torch.Tensor, lead: int, weight: torch.Tensor) -> torch.Tensor:
+    """Per head h: ask[t, h, lead + j] = sum_d weight[h, j, d] * rest[t, h, d]; the leading elements of `ask` stay as they are.
+    `rest` [T, H, d] (heads and tokens may lie apart), `ask` [T, H, lead + n] contiguous, `weight` [H, n, d]; returns `ask`."""
     KernelError = _base()[0]
-    if q.dim() != 3 or not q.is_contiguous() or weight.dim() != 3 or weight.shape[0] != q.shape[1] or weight.shape[2] != q.shape[2] - lead:
-        raise KernelError(f"q {tuple(q.shape)} does not fit the heads' weights {tuple(weight.shape)} after {lead} leading elements")
-    n_tokens, heads, width = q.shape
-    n = weight.shape[1]
-    out = torch.empty((n_tokens, heads, lead + n), dtype=q.dtype, device=q.device)
-    if lead and n_tokens:
-        # the leading elements of every head as they are: rows of `width` into rows of `lead + n`, one a (token, head)
-        _, _check, _code, _i32, _need_gpu, _ptr, _stream = _base()
-        lib = _build.load("groupnorm")
-        _check(
-            lib,
-            lib.cwm_copy_columns(
-                _ptr(q), ctypes.c_long(width), _ptr(out), ctypes.c_long(lead + n), ctypes.c_int(_code(q.dtype)),
-                ctypes.c_long(n_tokens * heads), ctypes.c_int(lead), _stream(),
-            ),
-        )
+    n_tokens, heads, width = ask.shape
+    if not ask.is_contiguous() or weight.dim() != 3 or weight.shape[0] != heads or weight.shape[1] != width - lead or ask.dtype != rest.dtype:
+        raise KernelError(f"the heads' weights {tuple(weight.shape)} do not fill rows {tuple(ask.shape)} from element {lead} on")
+    if rest.dim() != 3 or tuple(rest.shape) != (n_tokens, heads, weight.shape[2]) or rest.stride(2) != 1:
+        raise KernelError(f"unrotated parts {tuple(rest.shape)} do not fit the heads' weights {tuple(weight.shape)}")
     if n_tokens:
         tiles = _tiles_a_block(n_tokens)
-        _grouped(q.view(-1)[lead:], heads * width, width, None, weight, None, out.view(-1)[lead:], heads * (lead + n), lead + n, n_tokens, heads, tiles)
-    return out
+        _grouped(rest, max(rest.stride(0), heads * rest.shape[2]), rest.stride(1), None, weight, None, ask.view(-1)[lead:], heads * width, width, n_tokens, heads, tiles)
+    return ask
 
 
 def expand_values(mixed: torch.Tensor, lead: int, weight: torch.Tensor) -> torch.Tensor:

@@ -14,6 +14,7 @@ from .base import (
     Embedding,
     FeedForward,
     Head,
+    KeptFirstKVSpec,
     LayerCall,
     LayerPlan,
     Mixer,
@@ -35,9 +36,9 @@ from . import norm, rope, attention, feedforward, block, embedding, token_shift,
 from .linear import LinearWeights
 from .norm import GroupRMSNorm, LayerNorm, RMSNorm, StreamRMSNorm, StreamUpdate
 from .rope import NoPositionEncoding, RotaryEncoding, llama3_scale_frequencies, rotary_inverse_frequencies
-from .attention import HeadNormAttention, PagedAttention, SideBySide, SinkAttention, TalkingAttention
+from .attention import ConvAttention, HeadNormAttention, PagedAttention, SideBySide, SinkAttention, TalkingAttention
 from .feedforward import ActivatedMLP, GatedMLP, SwiGLU
-from .block import ConnectedPreNormBlock, ParallelPreNormBlock, PostNormBlock, PreNormBlock, SharedNormParallelBlock
+from .block import ConnectedPreNormBlock, ParallelPreNormBlock, PostNormBlock, PreNormBlock, SandwichNormBlock, SharedNormParallelBlock
 from .connection import HyperConnection, ResidualSum
 from .embedding import LinearHead, NormedTokenEmbedding, SinusoidalTokenEmbedding, TokenEmbedding
 from .token_shift import TokenShift

@@ -7,7 +7,9 @@ from typing import Any, Dict, Mapping, Optional, Tuple
 import torch
 
 from .. import ops
-from .base import ChunkedKVSpec, Mixer, PagedKVSpec, PartChoice, PositionEncoding, Runtime, TensorSpec, register_part
+from .base import (
+    CacheSpec, ChunkedKVSpec, KeptFirstKVSpec, Mixer, PagedKVSpec, PartChoice, PositionEncoding, Runtime, StateSpec, TensorSpec, register_part,
+)
 from .linear import LinearWeights
 
 
@@ -611,6 +613,170 @@ class HeadNormAttention(Mixer):
 
 
 register_part("mixer", "head_norm_attention", HeadNormAttention)
+
+
+class _Carried(Mixer):
+    """One cache need of a mixer that has several (`Mixer.children`): it only names what the cache manager is to keep."""
+
+    def __init__(self, spec: CacheSpec) -> None:
+        self.spec = spec
+
+    def cache_spec(self) -> CacheSpec:
+        return self.spec
+
+
+class ConvAttention(Mixer):
+    """Grouped-query attention over a paged cache whose queries and keys pass a short causal convolution and a norm over
+    the whole projection, whose values are the convolved keys, and whose heads are gated.
+
+        u = W x + b for q and k                                  `n_heads` and `n_kv_heads` heads of `head_dim`; biases where `bias`
+        y_t = sum_(lag = 0 .. taps - 1) w[taps - 1 - lag] u_(t - lag)     each channel, u before the sequence's start is 0
+        v = y of the key heads
+        q <- y / sqrt(mean(y^2) + eps) * w_q, k likewise         over all heads of the projection at once (`qk_norm`; float32)
+        rotation of q and k by the position encoding             its table may turn fewer than head_dim dimensions, in
+                                                                 adjacent pairs or in halves of the turned part
+        softmax over the keys j <= i with i - j < window or j < keep_first (`window` None: all): kept keys stay where they
+            are; with `unit_sink` its denominator is 1 + sum_j exp(s_j)
+        out = W_o [sigmoid(W_g x)_h * sum_j p_j v_j of every head]        the gate where `gate`, one number a head
+
+    The last taps - 1 rows of u are a sequence's state beside its pages: the mixer has two cache needs and lists them as
+    `children()` (one where taps is 1 or `taps` is None, which is no convolution).  Rotation in halves is served by an order
+    of the projections' rows; the values then come in that order too, and W_o's columns follow it.  Keys and values are
+    cached with `head_dim` rounded up to a multiple of 16.  `names`: the tensors' local names for the roles q, k, o, g,
+    q_bias, k_bias, q_conv, k_conv, q_norm and k_norm."""
+
+    replayable = True
+    DEFAULT_NAMES = {
+        "q": "q", "k": "k", "o": "o", "g": "g", "q_bias": "q.b", "k_bias": "k.b", "q_conv": "q.conv", "k_conv": "k.conv",
+        "q_norm": "q.norm", "k_norm": "k.norm",
+    }
+
+    def __init__(
+        self,
+        dim: int,
+        n_heads: int,
+        n_kv_heads: int,
+        head_dim: int,
+        scale: float,
+        window: Optional[int] = None,
+        keep_first: int = 0,
+        taps: Optional[int] = None,
+        bias: bool = True,
+        qk_norm: bool = True,
+        eps: float = 1e-6,
+        unit_sink: bool = False,
+        gate: bool = True,
+        position_encoding: Optional[PartChoice] = None,
+        names: Optional[Mapping[str, str]] = None,
+    ) -> None:
+        if n_heads % n_kv_heads != 0:
+            raise ValueError(f"{n_heads} query heads do not divide into {n_kv_heads} key/value heads")
+        padded = -(-head_dim // 16) * 16
+        if head_dim < 1 or padded > MAX_HEAD_DIM:
+            raise ValueError(f"heads of {head_dim} are outside 1..{MAX_HEAD_DIM}, the sizes the attention kernels take")
+        if window is not None and window < 1:
+            raise ValueError("a window holds at least the query's own key")
+        if keep_first < 0:
+            raise ValueError("the number of kept first keys cannot be negative")
+        if taps is not None and not 1 <= taps <= ops.MAX_CONV_QK_TAPS:
+            raise ValueError(f"a convolution of {taps} taps is outside 1..{ops.MAX_CONV_QK_TAPS}, what the kernel takes")
+        self.channels = (n_heads + n_kv_heads) * head_dim
+        if self.channels > ops.MAX_CONV_QK_CHANNELS:
+            raise ValueError(f"{self.channels} channels of queries and keys are more than the {ops.MAX_CONV_QK_CHANNELS} the kernel takes")
+        self.dim, self.n_heads, self.n_kv_heads, self.head_dim, self.padded = dim, n_heads, n_kv_heads, head_dim, padded
+        self.scale, self.window, self.keep_first = float(scale), window, keep_first if window is not None else 0
+        self.taps, self.bias, self.qk_norm, self.eps, self.unit_sink, self.gate = taps, bias, qk_norm, float(eps), unit_sink, gate
+        self.names = {**self.DEFAULT_NAMES, **dict(names or {})}
+        self.position_encoding: Optional[PositionEncoding] = (
+            position_encoding.build("position_encoding") if position_encoding is not None else None
+        )
+
+    def children(self):
+        if self.keep_first > 0:
+            pages: PagedKVSpec = KeptFirstKVSpec(n_kv_heads=self.n_kv_heads, head_dim=self.padded, window=self.window, keep_first=self.keep_first)
+        else:
+            pages = PagedKVSpec(n_kv_heads=self.n_kv_heads, head_dim=self.padded, window=self.window)
+        if self.taps is None or self.taps == 1:
+            return [_Carried(pages)]
+        return [_Carried(pages), _Carried(StateSpec(((self.taps - 1) * self.channels,), torch.float32))]
+
+    def cache_spec(self):
+        raise TypeError("this mixer has a cache and a state; the block asks `children()`")
+
+    def tensor_specs(self) -> Dict[str, TensorSpec]:
+        n = self.names
+        outs = {"q": self.n_heads * self.head_dim, "k": self.n_kv_heads * self.head_dim}
+        specs: Dict[str, TensorSpec] = {}
+        for r, out in outs.items():
+            specs[n[r]] = TensorSpec((out, self.dim))
+            if self.bias:
+                specs[n[r + "_bias"]] = TensorSpec((out,), precision="stored")
+            if self.taps is not None:
+                specs[n[r + "_conv"]] = TensorSpec((out, self.taps))
+            if self.qk_norm:
+                specs[n[r + "_norm"]] = TensorSpec((out,), init="norm", precision="stored")
+        if self.gate:
+            specs[n["g"]] = TensorSpec((self.n_heads, self.dim))
+        specs[n["o"]] = TensorSpec((self.dim, self.n_heads * self.head_dim))
+        return specs
+
+    def bind(self, tensors: Mapping[str, torch.Tensor], runtime: Runtime) -> None:
+        super().bind(tensors, runtime)
+        n, hd = self.names, self.head_dim
+        device = tensors[n["q"]].device
+        order = torch.arange(hd, device=device)  # the order of a head's elements in which the kernels turn adjacent pairs
+        self.table: Optional[torch.Tensor] = None
+        if self.position_encoding is not None:
+            self.position_encoding.bind({}, runtime)
+            table = self.position_encoding.rotary_table()
+            if table is not None:
+                turned = 2 * table.numel()
+                if turned > hd:
+                    raise ValueError(f"{turned} rotated dimensions exceed the head's {hd}")
+                if self.position_encoding.rotary_pairing() == "halves":
+                    half = turned // 2
+                    order = torch.cat([torch.stack([torch.arange(half), torch.arange(half) + half], dim=1).reshape(-1), torch.arange(turned, hd)]).to(device)
+                # a frequency of 0 leaves its pair alone: the head's other dimensions, and the padding
+                self.table = torch.zeros(self.padded // 2, dtype=torch.float32, device=device)
+                self.table[: table.numel()] = table.to(device)
+        rows = {
+            r: (torch.arange(heads, device=device)[:, None] * hd + order[None, :]).reshape(-1)
+            for r, heads in (("q", self.n_heads), ("k", self.n_kv_heads))
+        }
+        matrices = [tensors[n[r]][rows[r]] for r in ("q", "k")]
+        if self.gate:
+            matrices.append(tensors[n["g"]])
+        self.proj = LinearWeights.joined(matrices, [None] * len(matrices), stream_copy=runtime.stream_copies)
+        joined = lambda role: torch.cat([tensors[n[r + role]].float()[rows[r]] for r in ("q", "k")])  # noqa: E731
+        self.qk_bias = joined("_bias").contiguous() if self.bias else None
+        if self.taps is not None:
+            self.by_tap = joined("_conv").t().contiguous()  # a row a tap: what the kernel reads channel by channel
+        else:
+            self.by_tap = torch.ones((1, self.channels), dtype=torch.float32, device=device)
+        self.q_weight = tensors[n["q_norm"]].float()[rows["q"]].contiguous() if self.qk_norm else None
+        self.k_weight = tensors[n["k_norm"]].float()[rows["k"]].contiguous() if self.qk_norm else None
+        wo = tensors[n["o"]].reshape(self.dim, self.n_heads, hd)[:, :, order]
+        if self.padded != hd:  # the attention kernels return heads of the cached size
+            wo = torch.cat([wo, wo.new_zeros((self.dim, self.n_heads, self.padded - hd))], dim=2)
+        self.wo = LinearWeights(wo.reshape(self.dim, self.n_heads * self.padded), stream_copy=runtime.stream_copies)
+        self.sinks = torch.zeros(self.n_heads, dtype=torch.float32, device=device) if self.unit_sink else None  # exp(0) = 1
+
+    def forward(self, x: torch.Tensor, batch: Any, cache: Any, write_cache: bool = True) -> torch.Tensor:
+        if not write_cache:
+            raise ValueError("this mixer writes its own cache")
+        pages, carried = cache if isinstance(cache, tuple) else (cache, None)
+        proj = self.proj(x, partials_ok=True)
+        q, gates = ops.conv_qk_rope_write(
+            proj, self.n_heads, self.n_kv_heads, self.head_dim, self.padded, self.qk_bias, self.by_tap, self.q_weight, self.k_weight, self.eps,
+            batch, self.table, self.runtime.act_dtype, pages.cache, pages.block_table, carried.state if carried is not None else None, gate=self.gate,
+        )
+        attn = ops.paged_attention(
+            q, pages.cache, pages.block_table, batch, self.window, self.scale, sink=self.sinks, keep_first=self.keep_first, out_scale=gates,
+        )
+        return self.wo(attn, partials_ok=True)  # added into the residual by the next norm
+
+
+register_part("mixer", "conv_attention", ConvAttention)
 
 
 class SideBySide(Mixer):

@@ -134,6 +134,24 @@ class ChunkedKVSpec(PagedKVSpec):
 
 
 @dataclass(frozen=True)
+class KeptFirstKVSpec(PagedKVSpec):
+    """Keys and values in pages for a mixer whose queries read a window and, however far back they lie, the sequence's
+    first `keep_first` keys: the pages that hold those are never given back before the request ends."""
+
+    keep_first: int = 0
+
+    def __post_init__(self) -> None:
+        if self.window is None or self.keep_first < 0:
+            raise ValueError("kept first keys go with a window, and their number is not negative")
+
+    def retention(self) -> Hashable:
+        return ("keep_first", self.keep_first, self.window)
+
+    def pinned_keys(self) -> int:
+        return self.keep_first
+
+
+@dataclass(frozen=True)
 class StateSpec:
     """Per-request state of fixed size, zero when a request is admitted."""
 
@@ -211,6 +229,9 @@ class PositionEncoding(Part):
 
 
 class Mixer(Part):
+    """A mixer that needs several caches or states (several mixers side by side; pages and a state beside them) lists one
+    mixer a need as `children()`; its `forward` then gets a tuple of views in that order."""
+
     def cache_spec(self) -> CacheSpec:
         return None
 
@@ -322,12 +343,18 @@ class Block(Part):
 
     def mixers(self) -> List[Mixer]:
         """The block's mixers in the order in which `forward` gets their caches: each has a cache slot of its
-        own per entry of the run order.  By default the mixers among the parts, in the order of the plan (a
-        block that keeps its parts itself and has one `mixer` attribute is served too)."""
+        own per entry of the run order.  By default the mixers among the parts, in the order of the plan, each replaced
+        by its `children()` where it lists some (a block that keeps its parts itself and has one `mixer` attribute
+        is served too)."""
         parts = getattr(self, "parts", None)
         if parts is None:
             return [self.mixer]  # type: ignore[attr-defined]
-        return [part for part in parts.values() if isinstance(part, Mixer)]
+        found: List[Mixer] = []
+        for part in parts.values():
+            if isinstance(part, Mixer):
+                children = getattr(part, "children", None)
+                found.extend(children() if children is not None else [part])
+        return found
 
     def forward(
         self,

@@ -34,10 +34,6 @@ class PreNormBlock(Block):
         self.norm2 = norm2
         self.feed_forward = feed_forward
 
-    def mixers(self):
-        children = getattr(self.mixer, "children", None)
-        return list(children()) if children is not None else [self.mixer]
-
     def forward(self, h: torch.Tensor, delta: Any, batch: Any, cache: Any, write_cache: bool = True) -> Any:
         x = self.norm1.forward(h, delta)
         mixed = self.mixer.forward(x, batch, cache, write_cache)
@@ -48,6 +44,39 @@ class PreNormBlock(Block):
 
 
 register_part("block", "pre_norm", PreNormBlock)
+
+
+class SandwichNormBlock(Block):
+    """h += norm1b(mixer(norm1(h))); h += norm2b(feed_forward(norm2(h))): every sublayer reads a norm of the residual, and its
+    result passes another norm before it joins the residual.  The result's norm and the sum are left to the norm that reads
+    the residual next (an `ops.NormedSum` of one term), so that the three are one kernel; a feed-forward whose result is a
+    weighted sum of rows leaves that to it as well.  A layer without a feed-forward names none of `norm2`, `feed_forward`
+    and `norm2b`."""
+
+    def __init__(
+        self, names: Mapping[str, str], norm1: Norm, mixer: Mixer, norm1b: Norm, norm2: Optional[Norm] = None,
+        feed_forward: Optional[FeedForward] = None, norm2b: Optional[Norm] = None,
+    ) -> None:
+        if not ((feed_forward is None) == (norm2 is None) == (norm2b is None)):
+            raise ValueError("a feed-forward comes with its two norms")
+        parts = dict(norm1=norm1, mixer=mixer, norm1b=norm1b)
+        if feed_forward is not None:
+            parts.update(norm2=norm2, feed_forward=feed_forward, norm2b=norm2b)
+        super().__init__(names, **parts)
+        self.norm1, self.mixer, self.norm1b = norm1, mixer, norm1b
+        self.norm2, self.feed_forward, self.norm2b = norm2, feed_forward, norm2b
+
+    def forward(self, h: torch.Tensor, delta: Any, batch: Any, cache: Any, write_cache: bool = True) -> Any:
+        x = self.norm1.forward(h, delta)
+        delta = self.norm1b.pending(self.mixer.forward(x, batch, cache, write_cache))
+        if self.feed_forward is None:
+            return delta
+        x = self.norm2.forward(h, delta)
+        deferred = getattr(self.feed_forward, "forward_deferred", None) if getattr(self.feed_forward, "shared", None) is None else None
+        return self.norm2b.pending(deferred(x, batch) if deferred is not None else self.feed_forward.forward(x, batch))
+
+
+register_part("block", "sandwich_norm", SandwichNormBlock)
 
 
 class PostNormBlock(Block):
@@ -150,10 +179,6 @@ class ParallelPreNormBlock(Block):
         super().__init__(names, **parts)
         self.norm1, self.mixer, self.norm2, self.feed_forward = norm1, mixer, norm2, feed_forward
 
-    def mixers(self):
-        children = getattr(self.mixer, "children", None)
-        return list(children()) if children is not None else [self.mixer]
-
     def forward(self, h: torch.Tensor, delta: Any, batch: Any, cache: Any, write_cache: bool = True) -> Any:
         from .. import ops
 
@@ -200,11 +225,6 @@ class SharedNormParallelBlock(Block):
             parts["token_input"] = token_input
         super().__init__(names, **parts)
         self.norm, self.conv, self.mixer, self.feed_forward, self.token_input = norm, conv, mixer, feed_forward, token_input
-
-    def mixers(self):
-        children = getattr(self.mixer, "children", None)
-        own = list(children()) if children is not None else [self.mixer]
-        return ([self.conv] if self.conv is not None else []) + own
 
     def forward(self, h: torch.Tensor, delta: Any, batch: Any, cache: Any, write_cache: Any = True) -> Any:
         from .. import ops

@@ -2,7 +2,7 @@
 
 from __future__ import annotations
 
-from typing import Any, Dict, Mapping, Optional
+from typing import Any, Dict, Mapping, Optional, Tuple
 
 import torch
 
@@ -17,6 +17,8 @@ class RoutedExperts(FeedForward):
     Other routers and experts by argument.  `scores` "softmax_all": s = softmax(z) over all experts; the `top`
     experts with the largest s + correction (tensor `correction` [experts], if `correction`) are chosen and weighted
     by `weight_scale` * s, the correction not included, divided by the chosen scores' sum first if `renormalize`.
+    `groups` (count, keep): the experts form `count` equal groups of neighbours, and only those of the `keep` groups with
+    the best members can be chosen.
     `activation` "clamped_swish": an expert makes g' * sigmoid(act_alpha * g') * (u' + 1) of g = W_gate x and
     u = W_up x, with g' = min(g, act_limit) and u' = clamp(u, -act_limit, act_limit).
 
@@ -34,7 +36,7 @@ class RoutedExperts(FeedForward):
     def __init__(
         self, dim: int, hidden_dim: int, n_experts: int, top: int, scores: str = "softmax_chosen", correction: bool = False,
         weight_scale: float = 1.0, renormalize: bool = False, activation: str = "silu", act_alpha: float = 1.0, act_limit: float = 0.0,
-        router_bias: bool = False, shared: Optional[PartChoice] = None, shared_prefix: str = "shared.",
+        router_bias: bool = False, groups: Optional[Tuple[int, int]] = None, shared: Optional[PartChoice] = None, shared_prefix: str = "shared.",
     ) -> None:
         if not 1 <= top <= n_experts:
             raise ValueError(f"{top} experts a token out of {n_experts}")
@@ -44,6 +46,9 @@ class RoutedExperts(FeedForward):
             raise ValueError(f"router scores {scores!r}: 'softmax_chosen' and 'softmax_all' are known")
         if scores == "softmax_chosen" and (correction or weight_scale != 1.0 or renormalize):
             raise ValueError("a correction, a scale and renormalised weights belong to router scores over all experts")
+        if groups is not None and (n_experts % groups[0] != 0 or not 1 <= groups[1] <= groups[0] or top > groups[1] * (n_experts // groups[0])):
+            raise ValueError(f"{groups[1]} of {groups[0]} groups of {n_experts} experts do not hold {top} choices")
+        self.groups = (int(groups[0]), int(groups[1])) if groups is not None else None
         self.dim, self.hidden_dim, self.n_experts, self.top = dim, hidden_dim, n_experts, top
         self.scores, self.correction, self.weight_scale, self.renormalize = scores, correction, float(weight_scale), renormalize
         self.activation = ops.GatedActivation(activation, float(act_alpha), float(act_limit))
@@ -91,7 +96,7 @@ class RoutedExperts(FeedForward):
         """The same without the last kernel: every pair's row and the weights, for a consumer that adds a token's
         rows up itself (a norm that takes a `RoutedSum` as the pending result)."""
         logits = ops.linear(x, self.router, self.router_b, torch.float32)
-        chosen, weights = ops.route_top(logits, self.top, self.scores, self.choice_correction, self.weight_scale, self.renormalize)
+        chosen, weights = ops.route_top(logits, self.top, self.scores, self.choice_correction, self.weight_scale, self.renormalize, self.groups)
         groups = ops.group_by_expert(chosen, self.n_experts)
         if self.activation.kind == "silu":
             hidden = ops.grouped_gate_up(x, groups, self.gate, self.up)

@@ -84,7 +84,7 @@ register_part("feed_forward", "activated_mlp", ActivatedMLP)
 class GatedMLP(FeedForward):
     """W_down act(W_gate x, W_up x), no biases, with the gated activation as an argument (`ops.GatedActivation`):
     "silu": silu(g) * u;  "clamped_swish": g' * sigmoid(act_alpha * g') * (u' + 1) with g' = min(g, act_limit) and
-    u' = clamp(u, -act_limit, act_limit).  With `row_gate` (a tensor's local name, [1, dim]) the whole result is
+    u' = clamp(u, -act_limit, act_limit);  "gelu_tanh": gelu(g) * u, the tanh form.  With `row_gate` (a tensor's local name, [1, dim]) the whole result is
     multiplied by sigmoid(w . x), one number a token: the gate's row rides as one more output of the joined gate/up
     product and scales the activation's rows, which the linear down product carries through.  The activation is
     computed in float32 on the product's sums and rounded once.  `gate`, `up`, `down`: the tensors' local names."""

@@ -49,6 +49,15 @@ class RMSNorm(Norm):
         if self.scalar or self.gain != 1.0:
             self.weight = (self.weight.float() * self.gain).expand(self.dim).contiguous()
 
+    def pending(self, y: Any) -> "ops.NormedSum":
+        """This norm of a sublayer's result `y` (a tensor, partial sums or an `ops.RoutedSum`), as the residual update that
+        the norm reading the residual next applies."""
+        if isinstance(y, ops.ScaledSum):
+            raise TypeError("a sum of several results is normalised as a whole: it has to be added up first")
+        if self.weight.dtype != torch.float32:
+            self.weight = self.weight.float()
+        return ops.NormedSum([(y, self.weight, 1.0)], self.eps)
+
     def forward(self, h: torch.Tensor, delta: Any, rows: Optional[torch.Tensor] = None) -> torch.Tensor:
         if isinstance(delta, ops.NormedSum):
             if self.weight.dtype != torch.float32:

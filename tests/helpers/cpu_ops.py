@@ -103,7 +103,7 @@ def qkv_rope_write(x, weight, bias, n_q_heads, n_kv_heads, head_dim, positions, 
     return qkv
 
 
-def paged_attention(q, cache, block_table, batch, window, scale, sink=None, softcap=None, chunk=None, distance_bias=None):
+def paged_attention(q, cache, block_table, batch, window, scale, sink=None, softcap=None, chunk=None, distance_bias=None, keep_first=0, out_scale=None):
     n_tokens, n_q, hd = q.shape
     n_kv = cache.shape[2]
     page_size = cache.shape[3] // hd
@@ -116,7 +116,8 @@ def paged_attention(q, cache, block_table, batch, window, scale, sink=None, soft
         if chunk is not None:
             lo = p - p % chunk
         keys, vals = [], []
-        for j in range(lo, p + 1):
+        read = list(range(min(lo, keep_first))) + list(range(lo, p + 1))
+        for j in read:
             page = int(block_table[b, j // page_size])
             assert page >= 0, f"key {j} of sequence {b} has no page"
             slot = j % page_size
@@ -132,12 +133,14 @@ def paged_attention(q, cache, block_table, batch, window, scale, sink=None, soft
                 s = softcap * torch.tanh(s / softcap)
             if distance_bias is not None:
                 slope, rate = (float(t[h]) for t in distance_bias)
-                s = s - slope * torch.log1p(rate * (p - torch.arange(lo, p + 1)).float())
+                s = s - slope * torch.log1p(rate * (p - torch.tensor(read)).float())
             if sink is not None:  # one more term of the denominator, without a key or a value
                 w = torch.softmax(torch.cat([s, sink[h].float().reshape(1)]), -1)[:-1]
             else:
                 w = torch.softmax(s, -1)
             out[t, h] = w @ vv[g]
+            if out_scale is not None:
+                out[t, h] *= out_scale[t, h]
     return out.reshape(n_tokens, n_q * hd).to(q.dtype)
 
 
@@ -263,18 +266,31 @@ def selective_scan(xbc, dt, dt_bias, a_log, d_skip, state, batch, heads, head_di
     return y
 
 
-def route_top(logits, top, scores="softmax_chosen", correction=None, scale=1.0, renormalize=False):
+def route_top(logits, top, scores="softmax_chosen", correction=None, scale=1.0, renormalize=False, groups=None):
+    def closed(choice):
+        """The choice with the experts of the groups that do not stay open at -inf."""
+        if groups is None:
+            return choice
+        members = choice.reshape(choice.shape[0], groups[0], -1)
+        order = torch.sort(members.max(-1).values, dim=-1, descending=True, stable=True).indices[:, : groups[1]]
+        stays = torch.zeros(choice.shape[0], groups[0], dtype=torch.bool).scatter(1, order, True)
+        return members.masked_fill(~stays[..., None], float("-inf")).reshape(choice.shape)
+
     if scores == "softmax_all":
         s = torch.softmax(logits.float(), -1)
-        choice = s + correction.float() if correction is not None else s
+        choice = closed(s + correction.float() if correction is not None else s)
         chosen = torch.sort(choice, dim=-1, descending=True, stable=True).indices[:, :top]
         w = torch.gather(s, 1, chosen)
         if renormalize:
             w = w / w.sum(-1, keepdim=True)
         return chosen.to(torch.int32), w * scale
-    order = torch.sort(logits, dim=-1, descending=True, stable=True)
+    order = torch.sort(closed(logits), dim=-1, descending=True, stable=True)
     values, chosen = order.values[:, :top], order.indices[:, :top]
     return chosen.to(torch.int32), torch.softmax(values, -1)
+
+
+def _gelu_tanh(z):
+    return 0.5 * z * (1.0 + torch.tanh(math.sqrt(2.0 / math.pi) * (z + 0.044715 * z ** 3)))
 
 
 def group_by_expert(chosen, n_experts):
@@ -290,6 +306,8 @@ def grouped_gate_up(x, groups, gate, up, activation=None):
         g = g.clamp(max=activation.limit)
         u = u.clamp(-activation.limit, activation.limit)
         return (g * torch.sigmoid(activation.alpha * g) * (u + 1)).to(x.dtype)
+    if activation is not None and activation.kind == "gelu_tanh":
+        return (_gelu_tanh(g) * u).to(x.dtype)
     return (g * torch.sigmoid(g) * u).to(x.dtype)
 
 
@@ -302,9 +320,9 @@ def combine_routed(rows, groups, weights):
     return (rows.reshape(n, top, -1) * weights[:, :, None]).sum(1)
 
 
-def absorb_queries(q, lead, weight):
-    rest = torch.einsum("thd,hnd->thn", q[:, :, lead:].float(), weight.float())
-    return torch.cat([q[:, :, :lead].float(), rest], -1).to(q.dtype).contiguous()
+def absorb_queries(rest, ask, lead, weight):
+    ask[:, :, lead:] = torch.einsum("thd,hnd->thn", rest.float(), weight.float()).to(ask.dtype)
+    return ask
 
 
 def expand_values(mixed, lead, weight):
@@ -482,6 +500,8 @@ def gated_act_rows(x, hidden, activation, out_dtype, row_gate_col=None):
         g = torch.clamp(g, max=activation.limit)
         u = torch.clamp(u, min=-activation.limit, max=activation.limit)
         y = g * torch.sigmoid(activation.alpha * g) * (u + 1.0)
+    elif activation.kind == "gelu_tanh":
+        y = _gelu_tanh(g) * u
     else:
         y = g * torch.sigmoid(g) * u
     if row_gate_col is not None:
@@ -595,6 +615,8 @@ def embedding_sinusoid(tokens, table, positions, turns, scale=1.0):
 def add_normed_rmsnorm(h, delta, weight, eps, out_dtype, rows=None):
     total = torch.zeros_like(h)
     for t, w, c in delta.terms:
+        if hasattr(t, "groups"):  # a routed sum
+            t = combine_routed(t.rows, t.groups, t.weights)
         y = t.float().sum(0) if t.dim() == 3 else t.float()
         total += c * y * torch.rsqrt((y * y).mean(-1, keepdim=True) + delta.eps) * w.float()
     return add_rmsnorm(h, total, weight, eps, out_dtype, rows)
@@ -646,7 +668,49 @@ def wkv(r, k, v, gate, decay_logits, bonus, weight, state, batch, heads, dim, vd
     return (y * (g * torch.sigmoid(g))).reshape(n, heads * vdim).to(r.dtype)
 
 
+def latent_rows(q_src, kv_src, n_heads, lead, n_rest, rank, row, weight, eps, batch, inv_freq, out_dtype, cache=None, block_table=None):
+    total = lambda x: x.sum(0) if x.dim() == 3 else x.float()  # noqa: E731
+    n = batch.n_tokens
+    q = total(q_src)[:, : n_heads * (lead + n_rest)].reshape(n, n_heads, lead + n_rest)
+    turn = (lambda x: _rotate(x, batch.positions, inv_freq[: lead // 2])) if inv_freq is not None and lead else (lambda x: x)
+    ask = torch.zeros((n, n_heads, row), dtype=out_dtype)
+    ask[:, :, :lead] = turn(q[:, :, :lead]).to(out_dtype)
+    if kv_src is not None:
+        kv = total(kv_src)
+        c = kv[:, lead : lead + rank]
+        c = c * torch.rsqrt((c * c).mean(-1, keepdim=True) + eps) * weight
+        rows = torch.zeros((n, 1, row), dtype=torch.float32)
+        rows[:, 0, :lead] = turn(kv[:, None, :lead])[:, 0]
+        rows[:, 0, lead : lead + rank] = c
+        rows = rows.to(out_dtype)
+        rope_kv_write(rows.clone(), rows, rows, batch.positions, None, cache, block_table, batch.seq_of_token)
+    return ask, q[:, :, lead:].to(out_dtype)
+
+
+def conv_qk_rope_write(proj, n_q_heads, n_kv_heads, dim, head_dim, bias, by_tap, q_weight, k_weight, eps, batch, inv_freq, out_dtype,
+                       cache, block_table, state, gate=False):
+    proj = proj.sum(0) if proj.dim() == 3 else proj.float()
+    taps, channels = by_tap.shape
+    u = proj[:, :channels] + (bias if bias is not None else 0.0)
+    y = torch.empty_like(u)
+    for b in range(batch.n_seqs):
+        t0, t1 = int(batch.cu_q[b]), int(batch.cu_q[b + 1])
+        full = u[t0:t1]
+        if taps > 1:
+            kept = state[int(batch.state_slots[b]), : (taps - 1) * channels]
+            full = torch.cat([kept.reshape(taps - 1, channels), full])
+            kept.copy_(full[full.shape[0] - (taps - 1) :].reshape(-1))
+        for t in range(t1 - t0):
+            y[t0 + t] = (by_tap * full[t : t + taps]).sum(0)
+    q_width = n_q_heads * dim
+    joined = torch.cat([y, y[:, q_width:]], dim=1)  # the values are the keys as they are here
+    q = qk_norm_rope_write(joined, n_q_heads, n_kv_heads, dim, dim, head_dim, q_weight, k_weight, eps, batch.positions, inv_freq, out_dtype,
+                           cache, block_table, batch.seq_of_token)
+    return q, torch.sigmoid(proj[:, channels : channels + n_q_heads]) if gate else None
+
+
 STAND_INS = (
+    "latent_rows", "conv_qk_rope_write",
     "embedding_sinusoid", "add_normed_rmsnorm", "token_mixes", "min_gru", "wkv",
     "talking_attention", "gated_linear_attention", "short_conv", "token_side", "gated_act_rows",
     "add_layernorm", "head_norm_rope_write", "matrix_memory",

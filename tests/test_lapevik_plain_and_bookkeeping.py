@@ -152,7 +152,7 @@ def test_plan_names_the_folder_tensors_and_states():
                 # every head's state (the kernel may pad it) and the convolution's last inputs
                 assert isinstance(spec, StateSpec) and spec.shape[0] >= m["heads"] * m["state"] * m["vdim"] + (m["conv"] - 1) * (m["heads"] * m["vdim"] + 2 * m["groups"] * m["state"])
             else:
-                assert isinstance(spec, PagedKVSpec) and spec.n_kv_heads == 1 and spec.head_dim == m["kv_rank"] + m["rot_dim"] and spec.window is None
+                assert isinstance(spec, PagedKVSpec) and spec.n_kv_heads == 1 and spec.head_dim == -(-(m["kv_rank"] + m["rot_dim"]) // 16) * 16 and spec.window is None
 
 
 # ---- everything around the kernels ----------------------------------------------------------------------------- #

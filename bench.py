@@ -2,7 +2,7 @@
 
     python bench.py [--gpus 1] [--steps K] [--warmup W] [--layers L] [--dtype bf16|fp32]
     python bench.py --shape llama8b --serve 64     (requests through the scheduler instead)
-    python bench.py --compare lapevik|segedra|dogotar|digasun|sunusun   (another design beside the dense decoder of equal size instead)
+    python bench.py --compare lapevik|segedra|dogotar|digasun|sunusun|sorovik   (another design beside the dense decoder of equal size instead)
 
 Default run: the layer sizes of the CWM-32B shape with random weights, a batch of 8
 requests at a context of 32,768 tokens each; a step is one decode step of the whole
@@ -439,10 +439,42 @@ SUNUSUN_SIZES = {
     "w4096": (dict(width=4096, layers=8, heads=32, kv_heads=8, recurrent=4096, wkv_heads=64, ff=9216), 6144),
 }
 
+def sorovik_config(width, layers, heads, kv_heads, kv_rank, window, keep_first, taps, ff_dense, ff, experts, top, groups, keep, vocab=32768):
+    """A Sorovik model of `layers` layers in the order latent attention, latent attention on the rows of the layer before,
+    attention, latent attention: latent heads of 128 and 64 rotated elements, attention heads of 128 of which half turn, a
+    dense feed-forward in the first layer and routed experts in the others."""
+    def latent(kv_from=None):
+        mixer = {"heads": heads, "dim": 128, "rot_dim": 64, "vdim": 128, "kv_rank": kv_rank, "scale": 192 ** -0.5, "mask": {"size": window},
+                 "rot": {"base": 10000.0, "dims": 64}}
+        if kv_from is not None:
+            mixer["kv_from"] = kv_from
+        return {"type": "latent_attention", "mixer": mixer}
+
+    attention = {
+        "type": "attention",
+        "mixer": {"heads": heads, "kv_heads": kv_heads, "dim": 128, "vdim": 128, "scale": 128 ** -0.5, "conv": taps,
+                  "mask": {"size": window, "keep_first": keep_first}, "rot": {"base": 10000.0, "dims": 64}},
+    }
+    moe = {"kind": "moe", "expert": {"ff": ff}, "router": {"experts": experts, "top": top, "groups": {"count": groups, "keep": keep}}}
+    dense = {"kind": "dense", "ff": ff_dense}
+    made = []
+    for i in range(layers):
+        layer = latent(i - 1) if i % 4 == 1 else (attention if i % 4 == 2 else latent())
+        made.append(dict(layer, mlp=dense if i == 0 else moe))
+    return {"architecture": "Sorovik", "vocab": vocab, "width": width, "norm": {"eps": 1e-6}, "layers": made}
+
+
+# the same two widths; beside it also the models whose attention is the most alike: through a latent, and with a norm over the projections
+SOROVIK_SIZES = {
+    "w2048": (dict(width=2048, layers=8, heads=16, kv_heads=8, kv_rank=192, window=8192, keep_first=16, taps=3, ff_dense=4096, ff=1024, experts=16, top=4, groups=4, keep=2), 4096),
+    "w4096": (dict(width=4096, layers=8, heads=32, kv_heads=8, kv_rank=192, window=8192, keep_first=16, taps=3, ff_dense=6144, ff=1536, experts=32, top=4, groups=8, keep=4), 6144),
+}
+
 # design -> (sizes, maker of its configuration, other designs measured beside it at the size of the same name)
 COMPARISONS = {
     "lapevik": (LAPEVIK_SIZES, lapevik_config, ()), "segedra": (SEGEDRA_SIZES, segedra_config, ()), "dogotar": (DOGOTAR_SIZES, dogotar_config, ()),
     "digasun": (DIGASUN_SIZES, digasun_config, ()), "sunusun": (SUNUSUN_SIZES, sunusun_config, ("dogotar",)),
+    "sorovik": (SOROVIK_SIZES, sorovik_config, ("lapevik", "segedra")),
 }
 
 

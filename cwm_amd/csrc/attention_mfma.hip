@@ -501,7 +501,7 @@ attention_mfma_kernel(const bf16_t* __restrict__ q, long q_stride, bf16_t* __res
 #define LDS_BLOCKS_A_UNIT (HEAD_DIM > 128 ? 1 : 2)
 #define DMA_K_BYTES (32 * HEAD_DIM * 2)
 #define DMA_TILE_BYTES (2 * DMA_K_BYTES)
-#define DMA_HEAD_DIM_OK (HEAD_DIM == 64 || HEAD_DIM == 128)
+#define DMA_HEAD_DIM_OK (HEAD_DIM == 64 || HEAD_DIM == 128 || HEAD_DIM == 256)
 
 // MIN_BLOCKS blocks share a compute unit.  With two (at most 256 registers a wavefront) or three
 // (168) the compiler keeps the matrix-core accumulators in ordinary vector registers; from the
@@ -908,44 +908,39 @@ attention_lds_kernel(const bf16_t* __restrict__ q, long q_stride, bf16_t* __rest
     // tile t waits in registers set t % 2 and is multiplied from LDS buffer t % 2; its fetch is
     // issued three tiles ahead of its use and has two iterations to arrive
     Staged sa, sb;
-    auto fetch_tile = [&](Staged& st, int tile, int page) { fetch(st, first_key(tile), tile < kept_tiles, page); };
-    auto stash_tile = [&](const Staged& st, int tile, int buf) { stash(st, first_key(tile), tile < kept_tiles, buf); };
-    auto compute_tile = [&](int tile, int buf) { compute(first_key(tile), tile < kept_tiles, lds_k[buf], lds_v[buf]); };
-    auto page_of_tile = [&](int tile) { return tile_page(first_key(tile)); };
-    fetch_tile(sa, 0, page_of_tile(0));
-    fetch_tile(sb, 1, page_of_tile(1));
-    int page_next = page_of_tile(2);
-    stash_tile(sa, 0, 0);
-    fetch_tile(sa, 2, page_next);
-    page_next = page_of_tile(3);
+    auto is_kept = [&](int tile) { return tile < kept_tiles; };
+    fetch(sa, first_key(0), is_kept(0), tile_page(first_key(0)));
+    fetch(sb, first_key(1), is_kept(1), tile_page(first_key(1)));
+    int page_next = tile_page(first_key(2));
+    stash(sa, first_key(0), is_kept(0), 0);
+    fetch(sa, first_key(2), is_kept(2), page_next);
+    page_next = tile_page(first_key(3));
     __syncthreads();
     for (int it = 0; it < n_tiles; it += 2) {
-      compute_tile(it, 0);
-      stash_tile(sb, it + 1, 1);
-      fetch_tile(sb, it + 3, page_next);
-      page_next = page_of_tile(it + 4);
+      compute(first_key(it), is_kept(it), lds_k[0], lds_v[0]);
+      stash(sb, first_key(it + 1), is_kept(it + 1), 1);
+      fetch(sb, first_key(it + 3), is_kept(it + 3), page_next);
+      page_next = tile_page(first_key(it + 4));
       __syncthreads();
-      if (it + 1 < n_tiles) compute_tile(it + 1, 1);
-      stash_tile(sa, it + 2, 0);
-      fetch_tile(sa, it + 4, page_next);
-      page_next = page_of_tile(it + 5);
+      if (it + 1 < n_tiles) compute(first_key(it + 1), is_kept(it + 1), lds_k[1], lds_v[1]);
+      stash(sa, first_key(it + 2), is_kept(it + 2), 0);
+      fetch(sa, first_key(it + 4), is_kept(it + 4), page_next);
+      page_next = tile_page(first_key(it + 5));
       __syncthreads();
     }
   } else {
     Staged sa;
-    auto fetch_tile = [&](int tile) { fetch(sa, first_key(tile), tile < kept_tiles, 0); };
-    auto stash_tile = [&](int tile, int buf) { stash(sa, first_key(tile), tile < kept_tiles, buf); };
-    fetch_tile(0);
-    stash_tile(0, 0);
-    if (n_tiles > 1) fetch_tile(1);
+    fetch(sa, first_key(0), 0 < kept_tiles, 0);
+    stash(sa, first_key(0), 0 < kept_tiles, 0);
+    if (n_tiles > 1) fetch(sa, first_key(1), 1 < kept_tiles, 0);
     __syncthreads();
     for (int it = 0; it < n_tiles; ++it) {
       const int buf = it & 1;
       compute(first_key(it), it < kept_tiles, lds_k[buf], lds_v[buf]);
       // tile it + 1 (fetched an iteration ago) goes into the other buffer, which every wavefront
       // left at the last barrier; then tile it + 2 is fetched
-      if (it + 1 < n_tiles) stash_tile(it + 1, buf ^ 1);
-      if (it + 2 < n_tiles) fetch_tile(it + 2);
+      if (it + 1 < n_tiles) stash(sa, first_key(it + 1), it + 1 < kept_tiles, buf ^ 1);
+      if (it + 2 < n_tiles) fetch(sa, first_key(it + 2), it + 2 < kept_tiles, 0);
       __syncthreads();
     }
   }
@@ -1148,10 +1143,15 @@ extern "C" int cwm_attention_mfma(const void* q, long q_stride, void* out, long 
       // the values' offset from the keys of a page must fit the loads' 32-bit offsets
       if ((unsigned long long)n_kv_heads * page_size * HEAD_DIM * 2 >= (1ull << 31))
         CWM_LAUNCH_LDS(LDS_STAGED, 2, LDS_BLOCKS_A_UNIT);
+#if HEAD_DIM > 128
+      else  // one block a compute unit, whose buffers fill 128 KB of its LDS
+        CWM_LAUNCH_LDS(LDS_DMA, 4, LDS_BLOCKS_A_UNIT);
+#else
       else if (wide_three_blocks)  // the caller's choice: three blocks a compute unit
         CWM_LAUNCH_LDS(LDS_DMA, 3, 3);
       else
         CWM_LAUNCH_LDS(LDS_DMA, 4, 2);
+#endif
 #else
       CWM_LAUNCH_LDS(LDS_STAGED, 2, LDS_BLOCKS_A_UNIT);
 #endif

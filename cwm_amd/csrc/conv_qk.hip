@@ -20,7 +20,7 @@
 
 CWM_DEFINE_ERROR_API
 
-#define CONVQK_THREADS 512
+#define CONVQK_THREADS 1024  // at most
 #define CONVQK_MAX_TAPS 16
 #define CONVQK_MAX_HEAD 256
 #define CONVQK_TOKENS 4
@@ -36,8 +36,44 @@ __device__ __forceinline__ float convqk_input(const TS* __restrict__ src, long s
   return v;
 }
 
-// MAXT: room for that many taps in registers (taps <= MAXT); TB: tokens a block
-template <typename TS, typename TO, int MAXT, int TB>
+// W consecutive elements (1 or 4) of a float32 vector, and of a row of the projection
+template <int W>
+__device__ __forceinline__ void convqk_floats(const float* __restrict__ p, float (&v)[W]) {
+  if constexpr (W == 4) {
+    const float4 x = *(const float4*)p;
+    v[0] = x.x, v[1] = x.y, v[2] = x.z, v[3] = x.w;
+  } else {
+    v[0] = *p;
+  }
+}
+template <typename TS, int W>
+__device__ __forceinline__ void convqk_row(const TS* __restrict__ src, long stride, int n_partials, long partial_stride, long t, int d, float (&v)[W]) {
+  const TS* row = src + (size_t)t * stride + d;
+  if constexpr (W == 1) {
+    v[0] = convqk_input(src, stride, n_partials, partial_stride, t, d);
+  } else if constexpr (sizeof(TS) == 2) {
+    const uint2 x = *(const uint2*)row;  // partial sums are float32: one row here
+    v[0] = __uint_as_float(x.x << 16), v[1] = __uint_as_float(x.x & 0xffff0000u);
+    v[2] = __uint_as_float(x.y << 16), v[3] = __uint_as_float(x.y & 0xffff0000u);
+  } else {
+    v[0] = v[1] = v[2] = v[3] = 0.f;
+    for (int p = 0; p < n_partials; p += 4) {
+      // four partial sums in flight at a time; what lies past the last is the last again, times zero
+      float4 z[4];
+#pragma unroll
+      for (int u = 0; u < 4; ++u) z[u] = *(const float4*)(row + (size_t)min(p + u, n_partials - 1) * partial_stride);
+#pragma unroll
+      for (int u = 0; u < 4; ++u) {
+        const float keep = p + u < n_partials ? 1.f : 0.f;
+        v[0] = fmaf(keep, z[u].x, v[0]), v[1] = fmaf(keep, z[u].y, v[1]), v[2] = fmaf(keep, z[u].z, v[2]), v[3] = fmaf(keep, z[u].w, v[3]);
+      }
+    }
+  }
+}
+
+// MAXT: room for that many taps in registers (taps <= MAXT); TB: tokens a block; W: channels a thread takes at a time (4:
+// sizes are multiples of 4 and rows start at multiples of four elements)
+template <typename TS, typename TO, int MAXT, int TB, int W>
 __global__ void __launch_bounds__(CONVQK_THREADS)
 conv_qk_kernel(const TS* __restrict__ src, long src_stride, int n_partials, long partial_stride, const float* __restrict__ bias,
                const float* __restrict__ taps_w, int taps, float* __restrict__ state, long state_ld, const int* __restrict__ slots,
@@ -46,13 +82,26 @@ conv_qk_kernel(const TS* __restrict__ src, long src_stride, int n_partials, long
                const int* __restrict__ positions, const float* __restrict__ inv_freq, TO* __restrict__ cache,
                const int* __restrict__ block_table, int table_width, int page_size, int num_pages, int n_tokens, int n_q_heads,
                int n_kv_heads, int dim, int head_dim) {
-  extern __shared__ float y_all[];  // [TB][channels]
+  extern __shared__ __attribute__((aligned(16))) float y_all[];  // [TB][channels]
   __shared__ float cs[TB][CONVQK_MAX_HEAD];
   __shared__ float sums[2 * TB][CONVQK_THREADS / CWM_WAVE];
   const int t0 = blockIdx.x * TB;
   const int n = min(TB, n_tokens - t0);
   const int q_width = n_q_heads * dim, channels = q_width + n_kv_heads * dim;
   const int half = head_dim / 2;
+  int seq_of[TB], start_of[TB], pos_of[TB], page_of[TB];
+  float* state_of[TB];
+#pragma unroll
+  for (int k = 0; k < TB; ++k) {
+    const int t = min(t0 + k, n_tokens - 1);
+    seq_of[k] = seq_of_token[t];
+    pos_of[k] = positions[t];
+    start_of[k] = cu_q[seq_of[k]];
+    const int slot = slots[seq_of[k]];
+    state_of[k] = state && slot >= 0 && slot < n_slots ? state + (size_t)slot * state_ld : nullptr;
+    const int lp = pos_of[k] / page_size;
+    page_of[k] = lp < table_width ? block_table[(size_t)seq_of[k] * table_width + lp] : -1;
+  }
   for (int i = threadIdx.x; i < n * half; i += blockDim.x) {
     const int k = i / half, pair = i - k * half;
     float c = 1.f, s = 0.f;
@@ -61,65 +110,76 @@ conv_qk_kernel(const TS* __restrict__ src, long src_stride, int n_partials, long
     cs[k][2 * pair] = c;
     cs[k][2 * pair + 1] = s;
   }
-  // ---- the convolutions, a channel a thread at a time ---------------------------------------------------------- //
+  // ---- the convolutions, W channels a thread at a time ----------------------------------------------------------- //
   float sq[TB], sk[TB];
 #pragma unroll
   for (int k = 0; k < TB; ++k) sq[k] = sk[k] = 0.f;
-  for (int d = threadIdx.x; d < channels; d += blockDim.x) {
-    float w[MAXT], u[MAXT];  // u[j] meets tap j; the newest input is u[taps - 1]
+  for (int d = W * threadIdx.x; d < channels; d += W * blockDim.x) {
+    float w[MAXT][W], u[MAXT][W], b[W];  // u[j] meets tap j; the newest input is u[taps - 1]
 #pragma unroll
     for (int j = 0; j < MAXT; ++j) {
-      w[j] = j < taps ? taps_w[(size_t)j * channels + d] : 0.f;
-      u[j] = 0.f;
+#pragma unroll
+      for (int i = 0; i < W; ++i) w[j][i] = u[j][i] = 0.f;
+      if (j < taps) convqk_floats<W>(taps_w + (size_t)j * channels + d, w[j]);
     }
-    const float b = bias ? bias[d] : 0.f;
-    int seq = -1;
+#pragma unroll
+    for (int i = 0; i < W; ++i) b[i] = 0.f;
+    if (bias) convqk_floats<W>(bias + d, b);
 #pragma unroll
     for (int k = 0; k < TB; ++k) {
-      if (k < n) {
-        const int t = t0 + k;
-        const int sq_of = seq_of_token[t];
-        float* srow = nullptr;
-        if (sq_of != seq || moves_state) {
-          const int slot = slots[sq_of];
-          if (state && slot >= 0 && slot < n_slots) srow = state + (size_t)slot * state_ld;
-        }
-        if (sq_of != seq) {
-          // the block's first token of this sequence: the inputs before it come from the step's rows or from the state
-          const int start = cu_q[sq_of];
+      if (k >= n) continue;
+      const int t = t0 + k;
+      if (k == 0 || seq_of[k] != seq_of[k == 0 ? 0 : k - 1]) {
+        // the block's first token of this sequence: the inputs before it come from the step's rows or from the state
 #pragma unroll
-          for (int j = 0; j < MAXT; ++j) {
-            if (j < taps - 1) {
-              const int s = t - (taps - 1) + j;
-              if (s >= start)
-                u[j] = convqk_input(src, src_stride, n_partials, partial_stride, s, d) + b;
-              else
-                u[j] = srow ? srow[(size_t)(taps - 1 + (s - start)) * channels + d] : 0.f;
-            }
+        for (int j = 0; j < MAXT - 1; ++j) {
+          if (j >= taps - 1) continue;
+          const int s = t - (taps - 1) + j;
+          if (s >= start_of[k]) {
+            convqk_row<TS, W>(src, src_stride, n_partials, partial_stride, s, d, u[j]);
+#pragma unroll
+            for (int i = 0; i < W; ++i) u[j][i] += b[i];
+          } else if (state_of[k]) {
+            convqk_floats<W>(state_of[k] + (size_t)(taps - 1 + (s - start_of[k])) * channels + d, u[j]);
+          } else {
+#pragma unroll
+            for (int i = 0; i < W; ++i) u[j][i] = 0.f;
           }
-          seq = sq_of;
-        } else {
-#pragma unroll
-          for (int j = 0; j < MAXT - 1; ++j) u[j] = u[j + 1];
         }
-        const float own = convqk_input(src, src_stride, n_partials, partial_stride, t, d) + b;
-        float acc = 0.f;
+      } else {
 #pragma unroll
-        for (int j = 0; j < MAXT; ++j) {
-          if (j == taps - 1) u[j] = own;
-          if (j < taps) acc = fmaf(w[j], u[j], acc);
-        }
-        if (moves_state && srow) {
+        for (int j = 0; j < MAXT - 1; ++j)
 #pragma unroll
-          for (int j = 1; j < MAXT; ++j)
-            if (j < taps) srow[(size_t)(j - 1) * channels + d] = u[j];
-        }
-        y_all[(size_t)k * channels + d] = acc;
-        if (d < q_width)
-          sq[k] += acc * acc;
-        else
-          sk[k] += acc * acc;
+          for (int i = 0; i < W; ++i) u[j][i] = u[j + 1][i];
       }
+      float own[W], acc[W];
+      convqk_row<TS, W>(src, src_stride, n_partials, partial_stride, t, d, own);
+#pragma unroll
+      for (int i = 0; i < W; ++i) acc[i] = 0.f;
+#pragma unroll
+      for (int j = 0; j < MAXT; ++j)
+#pragma unroll
+        for (int i = 0; i < W; ++i) {
+          if (j == taps - 1) u[j][i] = own[i] + b[i];
+          if (j < taps) acc[i] = fmaf(w[j][i], u[j][i], acc[i]);
+        }
+      if (moves_state && state_of[k]) {
+#pragma unroll
+        for (int j = 1; j < MAXT; ++j)
+          if (j < taps)
+#pragma unroll
+            for (int i = 0; i < W; ++i) state_of[k][(size_t)(j - 1) * channels + d + i] = u[j][i];
+      }
+      float ss = 0.f;
+#pragma unroll
+      for (int i = 0; i < W; ++i) {
+        y_all[(size_t)k * channels + d + i] = acc[i];
+        ss += acc[i] * acc[i];
+      }
+      if (d < q_width)
+        sq[k] += ss;
+      else
+        sk[k] += ss;
     }
   }
   // ---- the root mean squares of a token's queries and keys ------------------------------------------------------ //
@@ -133,7 +193,9 @@ conv_qk_kernel(const TS* __restrict__ src, long src_stride, int n_partials, long
     }
   }
   __syncthreads();
-  for (int k = 0; k < n; ++k) {
+#pragma unroll
+  for (int k = 0; k < TB; ++k) {
+    if (k >= n) continue;
     float tq = 0.f, tk = 0.f;
     for (int w2 = 0; w2 < waves; ++w2) {
       tq += sums[2 * k][w2];
@@ -141,16 +203,13 @@ conv_qk_kernel(const TS* __restrict__ src, long src_stride, int n_partials, long
     }
     const float q_rstd = 1.0f / sqrtf(tq / (float)q_width + eps), k_rstd = 1.0f / sqrtf(tk / (float)(channels - q_width) + eps);
     const int t = t0 + k;
-    const int pos = positions[t];
     const float* y = y_all + (size_t)k * channels;
-    const int lp = pos / page_size;
-    const int slot = pos - lp * page_size;
-    const int page = lp < table_width ? block_table[(size_t)seq_of_token[t] * table_width + lp] : -1;
+    const int slot = pos_of[k] % page_size;
     TO* kdst = nullptr;
     TO* vdst = nullptr;
-    if (page >= 0 && page < num_pages) {
+    if (page_of[k] >= 0 && page_of[k] < num_pages) {
       const size_t plane = (size_t)n_kv_heads * page_size * head_dim;
-      kdst = cache + (size_t)page * 2 * plane;
+      kdst = cache + (size_t)page_of[k] * 2 * plane;
       vdst = kdst + plane;
     }
     const int v_block = (page_size % 8 == 0) ? 8 : page_size;
@@ -244,22 +303,27 @@ extern "C" int cwm_conv_qk(const void* src, int src_dtype, long src_stride, int 
   if (n_tokens == 0) return 0;
   const bool moves = write_state == 2 && taps > 1;
   // a block walks down several tokens where there are many of them and their rows fit
-  const int tb = n_tokens >= 1024 && (long)CONVQK_TOKENS * channels * 4 <= CONVQK_MAX_LDS ? CONVQK_TOKENS : 1;
+  const int tb = n_tokens >= 1024 && taps <= 4 && (long)CONVQK_TOKENS * channels * 4 <= CONVQK_MAX_LDS ? CONVQK_TOKENS : 1;
   const size_t lds = (size_t)tb * channels * sizeof(float);
-#define CWM_CONVQK_GO(TS, TO, MAXT, TB)                                                                                                 \
+  const uintptr_t row_bytes = src_dtype == CWM_F32 ? 16 : 8;
+  const bool vec = taps <= 4 && (n_q_heads * dim) % 4 == 0 && channels % 4 == 0 && src_stride % 4 == 0 && partial_stride % 4 == 0 && state_ld % 4 == 0 &&
+                   ((uintptr_t)src % row_bytes) == 0 && ((uintptr_t)bias % 16) == 0 && ((uintptr_t)taps_w % 16) == 0 && ((uintptr_t)state % 16) == 0;
+  int threads = ((vec ? channels / 4 : channels) + CWM_WAVE - 1) / CWM_WAVE * CWM_WAVE;
+  if (threads < 256) threads = 256;
+  if (threads > CONVQK_THREADS) threads = CONVQK_THREADS;
+#define CWM_CONVQK_GO(TS, TO, MAXT, TB, W)                                                                                              \
+  hipLaunchKernelGGL((conv_qk_kernel<TS, TO, MAXT, TB, W>), dim3((n_tokens + TB - 1) / TB), dim3(threads), lds, stream,                 \
+                     (const TS*)src, src_stride, n_partials, partial_stride, bias, taps_w, taps, state, state_ld, slots, cu_q,          \
+                     seq_of_token, n_slots, moves, (TO*)q_out, gate_out, q_weight, k_weight, eps, positions, inv_freq, (TO*)cache,      \
+                     block_table, table_width, page_size, num_pages, n_tokens, n_q_heads, n_kv_heads, dim, head_dim)
+#define CWM_CONVQK(TS, TO)                                                                                                              \
   do {                                                                                                                                  \
-    hipLaunchKernelGGL((conv_qk_kernel<TS, TO, MAXT, TB>), dim3((n_tokens + TB - 1) / TB), dim3(CONVQK_THREADS), lds, stream,           \
-                       (const TS*)src, src_stride, n_partials, partial_stride, bias, taps_w, taps, state, state_ld, slots, cu_q,        \
-                       seq_of_token, n_slots, moves, (TO*)q_out, gate_out, q_weight, k_weight, eps, positions, inv_freq, (TO*)cache,    \
-                       block_table, table_width, page_size, num_pages, n_tokens, n_q_heads, n_kv_heads, dim, head_dim);                 \
-  } while (0)
-#define CWM_CONVQK(TS, TO)                                                     \
-  do {                                                                         \
-    if (taps <= 4 && tb == 1) CWM_CONVQK_GO(TS, TO, 4, 1);                     \
-    else if (taps <= 4) CWM_CONVQK_GO(TS, TO, 4, CONVQK_TOKENS);               \
-    else if (tb == 1) CWM_CONVQK_GO(TS, TO, CONVQK_MAX_TAPS, 1);               \
-    else CWM_CONVQK_GO(TS, TO, CONVQK_MAX_TAPS, CONVQK_TOKENS);                \
-    if (write_state == 1 && taps > 1)                                          \
+    if (taps > 4) CWM_CONVQK_GO(TS, TO, CONVQK_MAX_TAPS, 1, 1);                                                                         \
+    else if (tb == 1 && vec) CWM_CONVQK_GO(TS, TO, 4, 1, 4);                                                                            \
+    else if (tb == 1) CWM_CONVQK_GO(TS, TO, 4, 1, 1);                                                                                   \
+    else if (vec) CWM_CONVQK_GO(TS, TO, 4, CONVQK_TOKENS, 4);                                                                           \
+    else CWM_CONVQK_GO(TS, TO, 4, CONVQK_TOKENS, 1);                                                                                    \
+    if (write_state == 1 && taps > 1)                                                                                                   \
       hipLaunchKernelGGL((conv_qk_state_kernel<TS>), dim3(n_seqs, (channels + 255) / 256), dim3(256), 0, stream, (const TS*)src, src_stride, \
                          n_partials, partial_stride, bias, state, state_ld, slots, cu_q, n_slots, channels, taps);                     \
   } while (0)

@@ -82,6 +82,7 @@ def cache_windows(config: SorovikConfig) -> Dict[int, Optional[int]]:
 def build_plan(config: SorovikConfig) -> ModelPlan:
     width, eps = config.width, config.norm.eps
     norm = PartChoice("rmsnorm", {"dim": width, "eps": eps, "tensor": ""})
+    unread = PartChoice("rmsnorm", {"dim": width, "eps": eps, "tensor": "", "optional": True})
     spans = cache_windows(config)
     layers, order = [], []
     for i, layer in enumerate(config.layers):
@@ -104,6 +105,9 @@ def build_plan(config: SorovikConfig) -> ModelPlan:
             parts["norm2"] = PartSlot("norm", norm, "norm2")
             parts["feed_forward"] = PartSlot("feed_forward", _feed_forward(width, layer.mlp), "mlp.")
             parts["norm2b"] = PartSlot("norm", norm, "norm2b")
+        else:  # a folder may hold the norms of a sublayer that the layer does not have
+            parts["norm2"] = PartSlot("norm", unread, "norm2")
+            parts["norm2b"] = PartSlot("norm", unread, "norm2b")
         layers.append(LayerPlan(prefix=f"l{i}.", block="sandwich_norm", parts=parts))
         order.append(call)
     sizes = {"vocab_size": config.vocab, "dim": width, "tensor": ""}

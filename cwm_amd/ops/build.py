@@ -71,7 +71,7 @@ SOURCES: Dict[str, Tuple[Mapping[str, int], ...]] = {
     "latent_rows": ({},),
     "conv_qk": ({},),
     "attention_mfma": tuple({"HEAD_DIM": hd} for hd in (16, 32, 48, 64, 80, 96, 128, 256)) + tuple({"DISTANCE_BIAS": 1, "HEAD_DIM": hd} for hd in (32, 48, 64, 128))
-    + tuple({"HEAD_DIM": hd, "KEPT_KEYS": 1} for hd in (16, 32, 48, 64, 80, 96, 128)),
+    + tuple({"HEAD_DIM": hd, "KEPT_KEYS": 1} for hd in (16, 32, 48, 64, 80, 96, 128, 192)),
 }
 
 

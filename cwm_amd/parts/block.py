@@ -50,19 +50,17 @@ class SandwichNormBlock(Block):
     """h += norm1b(mixer(norm1(h))); h += norm2b(feed_forward(norm2(h))): every sublayer reads a norm of the residual, and its
     result passes another norm before it joins the residual.  The result's norm and the sum are left to the norm that reads
     the residual next (an `ops.NormedSum` of one term), so that the three are one kernel; a feed-forward whose result is a
-    weighted sum of rows leaves that to it as well.  A layer without a feed-forward names none of `norm2`, `feed_forward`
-    and `norm2b`."""
+    weighted sum of rows leaves that to it as well.  A layer without a feed-forward names none (the two norms around
+    one that it names all the same are not read)."""
 
     def __init__(
         self, names: Mapping[str, str], norm1: Norm, mixer: Mixer, norm1b: Norm, norm2: Optional[Norm] = None,
         feed_forward: Optional[FeedForward] = None, norm2b: Optional[Norm] = None,
     ) -> None:
-        if not ((feed_forward is None) == (norm2 is None) == (norm2b is None)):
+        if feed_forward is not None and (norm2 is None or norm2b is None):
             raise ValueError("a feed-forward comes with its two norms")
-        parts = dict(norm1=norm1, mixer=mixer, norm1b=norm1b)
-        if feed_forward is not None:
-            parts.update(norm2=norm2, feed_forward=feed_forward, norm2b=norm2b)
-        super().__init__(names, **parts)
+        parts = dict(norm1=norm1, mixer=mixer, norm1b=norm1b, norm2=norm2, feed_forward=feed_forward, norm2b=norm2b)
+        super().__init__(names, **{role: part for role, part in parts.items() if part is not None})
         self.norm1, self.mixer, self.norm1b = norm1, mixer, norm1b
         self.norm2, self.feed_forward, self.norm2b = norm2, feed_forward, norm2b
 

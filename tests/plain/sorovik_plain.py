@@ -30,6 +30,7 @@ from typing import Dict, List, Optional, Tuple
 import torch
 
 F = torch.float64
+ANGLES = F  # float32: angles as an engine rounds them, which shows how much a model's logits hang on their last bits
 
 
 def bf16_round(t: torch.Tensor) -> torch.Tensor:
@@ -63,7 +64,7 @@ def turn_halves(x: torch.Tensor, positions: torch.Tensor, dims: int, base: float
     half = dims // 2
     i = torch.arange(half, dtype=F)
     freq = base ** (-2.0 * i / max(dims, 1))
-    a = positions.to(F)[:, None] * freq[None, :]
+    a = (positions.to(ANGLES)[:, None] * freq.to(ANGLES)[None, :]).to(F)
     c, s = torch.cos(a)[:, None, :], torch.sin(a)[:, None, :]
     u, v = x[..., :half], x[..., half:dims]
     return torch.cat([u * c - v * s, v * c + u * s, x[..., dims:]], dim=-1)

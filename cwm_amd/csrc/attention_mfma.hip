@@ -482,10 +482,11 @@ attention_mfma_kernel(const bf16_t* __restrict__ q, long q_stride, bf16_t* __res
 // lies outside the block's span of keys is zeroed when the tile is written to LDS) and two tiles
 // are in flight in registers, so that the wavefront counts its loads and waits only for the older
 // tile.
-// LDS_DMA (the same, head sizes 64 and 128): the loads write LDS themselves
+// LDS_DMA (the same, head sizes 64, 128 and 256): the loads write LDS themselves
 // (global_load_lds_dwordx4: lane l of a wavefront fills bytes 16 l .. 16 l + 15 after a uniform
 // address), DMA_BUFFERS - 1 tiles ahead into DMA_BUFFERS buffers, so a tile costs no registers, no
-// LDS write instructions and one barrier.  Built twice: four buffers and two blocks a compute unit,
+// LDS write instructions and one barrier.  For 256: four buffers, 128 KB of LDS, one block a compute unit.  For the others
+// built twice: four buffers and two blocks a compute unit,
 // which finishes a launch of few, uneven blocks soonest, and three buffers with at most 168
 // registers for three blocks a compute unit, which hides more latency when there are many blocks.
 // The rows of keys are not padded; the 16-byte piece p of row r lies at piece p ^ r (p ^ (r / 2)

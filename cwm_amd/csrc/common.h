@@ -59,6 +59,13 @@ __device__ __forceinline__ float wave_max(float v) {
   return v;
 }
 
+// Sine and cosine of position * freq.  The product is exact (float64) and its whole turns are taken off before it is
+// rounded, so a far position is as exact as a near one (a float32 product of some hundred radians is off by up to 3e-5).
+__device__ __forceinline__ void sincos_turn(int position, float freq, float* s, float* c) {
+  const double turns = (double)position * (double)freq * 0.15915494309189535;
+  sincospif((float)(2.0 * (turns - rint(turns))), s, c);
+}
+
 // Sum over a block of up to 1024 threads in a fixed order (wave shuffles, then the
 // wave partials in index order); every thread gets the result.  `scratch` holds at
 // least 16 floats of LDS.  Safe to call repeatedly.

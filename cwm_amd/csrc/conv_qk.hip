@@ -106,7 +106,7 @@ conv_qk_kernel(const TS* __restrict__ src, long src_stride, int n_partials, long
     const int k = i / half, pair = i - k * half;
     float c = 1.f, s = 0.f;
     const float f = inv_freq ? inv_freq[pair] : 0.f;
-    if (f != 0.f) sincosf((float)positions[t0 + k] * f, &s, &c);
+    if (f != 0.f) sincos_turn(positions[t0 + k], f, &s, &c);
     cs[k][2 * pair] = c;
     cs[k][2 * pair + 1] = s;
   }

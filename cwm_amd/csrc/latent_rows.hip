@@ -33,7 +33,7 @@ latent_rows_kernel(const TS* __restrict__ q_src, long q_stride, int q_partials, 
   for (int i = threadIdx.x; 2 * i < lead; i += blockDim.x) {
     float c = 1.f, s = 0.f;
     const float f = inv_freq ? inv_freq[i] : 0.f;
-    if (f != 0.f) sincosf((float)pos * f, &s, &c);
+    if (f != 0.f) sincos_turn(pos, f, &s, &c);
     cs[2 * i] = c;
     cs[2 * i + 1] = s;
   }
